@@ -242,8 +242,8 @@ def test_recurrence_prepare_scan_and_head_norm(ops, ref, dtype, heads, kv_heads,
     qk = qk * 0.3
     sa = rnd(g, 5, heads, dim, vdim)
     sb, before = sa.clone(), sa.clone()
-    a = ops.linear_scan(qk, main, 2 * qs, decay, beta, sa, slots, cu, 20, heads, kv_heads, dim, vdim, delta_rule)
-    b = ref.linear_scan(qk, main, 2 * qs, decay, beta, sb, slots, cu, 20, heads, kv_heads, dim, vdim, delta_rule)
+    a = ops.linear_scan(qk, main, 2 * qs, decay, beta, sa, slots, cu, 20, heads, kv_heads, dim, vdim, "delta" if delta_rule else "additive")
+    b = ref.linear_scan(qk, main, 2 * qs, decay, beta, sb, slots, cu, 20, heads, kv_heads, dim, vdim, "delta" if delta_rule else "additive")
     near(a, b, 3e-5, "read-out")
     near(sa, sb, 3e-5, "state")
     assert torch.equal(sa[4], before[4])  # a slot that no sequence of the step uses
@@ -273,7 +273,7 @@ def test_a_long_portion_equals_its_pieces_and_its_first_token_is_kept(ops, ref, 
         for c in cuts:
             cu = torch.tensor([0, c], dtype=torch.int32).cuda()
             outs.append(operations.linear_scan(qk[at:at + c].clone(), v[at:at + c].clone(), 0, decay[at:at + c].clone(),
-                                               None if beta is None else beta[at:at + c].clone(), state, slot, cu, c, heads, kv_heads, dim, vdim, delta_rule))
+                                               None if beta is None else beta[at:at + c].clone(), state, slot, cu, c, heads, kv_heads, dim, vdim, "delta" if delta_rule else "additive"))
             at += c
         return torch.cat(outs), state
 

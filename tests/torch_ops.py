@@ -173,14 +173,14 @@ class TorchOps:
         return out
 
     def rotate_pad_write(self, qkv, num_heads, num_kv_heads, dim, vdim, cached_dim, positions, cos, sin, slot_mapping, k_cache, v_cache, block_size, write_kv=True,
-                         interleaved=False):
+                         interleaved=False, post_norm_eps=0.0, values_are_keys=False):
         """Rotates the first ``2 * cos.shape[1]`` channels of every q and k head (halves layout, or pairs (2i, 2i + 1)), writes k and v into the
         pages at ``cached_dim`` channels a head (zeros in the padding) and returns q as [T, heads * cached_dim]."""
         t = qkv.shape[0]
         q_size, k_size = num_heads * dim, num_kv_heads * dim
         q = qkv[:, :q_size].float().view(t, num_heads, dim)
         k = qkv[:, q_size:q_size + k_size].float().view(t, num_kv_heads, dim)
-        v = qkv[:, q_size + k_size:].float().view(t, num_kv_heads, vdim)
+        v = k if values_are_keys else qkv[:, q_size + k_size:].float().view(t, num_kv_heads, vdim)
         if cos is not None:
             half = cos.shape[1]
             c, s_ = cos[positions.long()][:, None, :], sin[positions.long()][:, None, :]
@@ -192,6 +192,8 @@ class TorchOps:
                 return torch.cat([a * c - b * s_, b * c + a * s_, x[..., 2 * half:]], -1)
 
             q, k = rotate(q), rotate(k)
+        if post_norm_eps > 0:
+            q, k = (x / torch.sqrt((x * x).mean(-1, keepdim=True) + post_norm_eps) for x in (q, k))
         out = torch.zeros((t, num_heads, cached_dim), dtype=qkv.dtype, device=qkv.device)
         out[:, :, :dim] = q.to(qkv.dtype)
         if write_kv:
@@ -225,9 +227,37 @@ class TorchOps:
             beta = torch.sigmoid(beta_source[:, beta_at:beta_at + heads].float()).contiguous()
         return qk, decay, beta
 
-    def linear_scan(self, qk, v_source, v_at, decay, beta, state, slots, cu_q, max_q_len, heads, kv_heads, dim, vdim, delta):
+    def removal_prepare(self, main, r_at, k_at, a_at, low_at, rank, heads, dim, a_bias, w2, w0, decay_scale):
+        """-> vectors float32 [T, heads, 3, dim] (r; the unit key u; sigmoid(a) u), decay [T, heads * dim], lengths [T, heads]."""
+        t, size = main.shape[0], heads * dim
+        r, k, a = (main[:, at:at + size].float() for at in (r_at, k_at, a_at))
+        k = k.view(t, heads, dim)
+        lengths = torch.sqrt((k * k).sum(-1) + 1e-6)
+        u = k / lengths[..., None]
+        removal = torch.sigmoid(a + a_bias).view(t, heads, dim) * u
+        z = torch.tanh(main[:, low_at:low_at + rank].float()) @ w2.float().T + w0
+        return torch.stack([r.view(t, heads, dim), u, removal], 2).contiguous(), torch.exp(-decay_scale * torch.sigmoid(z)), lengths
+
+    def gated_scan(self, projected, width, gate_bias, input_bias, shift, state, slots, cu_q, max_q_len):
+        """``S <- (1 - z) S + z c`` per channel from ``state[slot]``, which is written back; -> ``S * silu(g)``."""
+        z = torch.sigmoid(projected[:, :width].float() + gate_bias)
+        u = projected[:, width:2 * width].float() + input_bias
+        g = projected[:, 2 * width:].float()
+        candidate = torch.where(u >= 0, u + shift, torch.sigmoid(u))
+        out = torch.empty_like(z)
+        bounds = cu_q.tolist()
+        for b, slot in enumerate(slots.tolist()):
+            s = state[slot].clone()
+            for i in range(bounds[b], bounds[b + 1]):
+                s = (1.0 - z[i]) * s + z[i] * candidate[i]
+                out[i] = s * (g[i] * torch.sigmoid(g[i]))
+            state[slot] = s
+        return out.to(projected.dtype)
+
+    def linear_scan(self, qk, v_source, v_at, decay, beta, state, slots, cu_q, max_q_len, heads, kv_heads, dim, vdim, rule):
         """Per sequence and head, token by token from ``state[slot, head]`` ([dim, vdim] float32), which is written back:
-        ``S <- g S`` (rows); ``u = beta (v - S^T k)`` (delta) or ``u = v``; ``o = S^T q + (k . q) u``; ``S <- S + k u^T``.
+        ``S <- g S`` (rows); ``u = beta (v - S^T k)`` (delta) or ``u = v`` (additive); ``o = S^T q + (k . q) u``; ``S <- S + k u^T``.  removal:
+        a third vector ``b``, ``S <- g S - b (k^T S) + k (beta v)^T``, both terms on the old state; ``o = S^T q``.
         Returns float32 [T, heads * vdim]."""
         t = qk.shape[0]
         out = torch.empty((t, heads, vdim), dtype=torch.float32, device=qk.device)
@@ -240,9 +270,14 @@ class TorchOps:
             for i in range(bounds[b], bounds[b + 1]):
                 q = qk[i, :, 0].repeat_interleave(repeat, 0)  # [heads, dim]
                 k = qk[i, :, 1].repeat_interleave(repeat, 0)
-                s = s * g[i][:, :, None]
                 u = v[i]
-                if delta:
+                if rule == "removal":
+                    held = torch.einsum("hde,hd->he", s, k)
+                    s = s * g[i][:, :, None] - qk[i, :, 2].repeat_interleave(repeat, 0)[:, :, None] * held[:, None, :] + k[:, :, None] * (beta[i][:, None] * u)[:, None, :]
+                    out[i] = torch.einsum("hde,hd->he", s, q)
+                    continue
+                s = s * g[i][:, :, None]
+                if rule == "delta":
                     u = beta[i][:, None] * (u - torch.einsum("hde,hd->he", s, k))
                 out[i] = torch.einsum("hde,hd->he", s, q) + (k * q).sum(-1, keepdim=True) * u
                 s = s + k[:, :, None] * u[:, None, :]
@@ -252,7 +287,7 @@ class TorchOps:
     def gated_head_norm(self, read, weight, eps, gate_source, gate_at, gate_kind, heads, vdim, out_dtype):
         t = read.shape[0]
         o = read.view(t, heads, vdim)
-        o = o / torch.sqrt((o * o).mean(-1, keepdim=True) + eps) * weight.float()
+        o = o / torch.sqrt((o * o).mean(-1, keepdim=True) + eps) * (weight.float().view(heads, vdim) if weight.numel() != vdim else weight.float())
         gate = gate_source[:, gate_at:gate_at + heads * vdim].float().view(t, heads, vdim)
         gate = gate * torch.sigmoid(gate) if gate_kind == "silu" else torch.sigmoid(gate)
         return (o * gate).view(t, heads * vdim).to(out_dtype)
@@ -303,6 +338,22 @@ class TorchOps:
         var = (y * y).sum(-1, keepdim=True) / y.shape[-1]
         residual += mult * (y / torch.sqrt(var + eps) * weight.float())
         return residual if out_dtype == torch.float32 else residual.to(out_dtype)
+
+    def norm_add_norm(self, residual, delta, delta_weight, delta_eps, weight, eps, out_dtype, rows=None):
+        y = delta.float().sum(0) if delta.dim() == 3 else delta.float()
+        x = residual
+        if rows is not None:
+            x, y = residual[rows.long()], y[rows.long()]
+        x = x + y / torch.sqrt((y * y).mean(-1, keepdim=True) + delta_eps) * delta_weight
+        if rows is None:
+            residual.copy_(x)
+        return (x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps) * weight).to(out_dtype)
+
+    def poly_norm(self, x, coefficients, eps):
+        z = x.float()
+        a, b, c, e = coefficients.tolist()
+        powers = [p / torch.sqrt((p * p).mean(-1, keepdim=True) + eps) for p in (z, z * z, z * z * z)]
+        return (a * powers[0] + b * powers[1] + c * powers[2] + e).to(x.dtype)
 
     def qk_norm_write(self, qkv, num_heads, num_kv_heads, dim, vdim, cached_dim, q_norm, k_norm, whole, eps, q_temp, positions, first_values,
                       mix_weight, slot_mapping, k_cache, v_cache, block_size, write_kv=True):
@@ -502,8 +553,12 @@ class TorchOps:
         if shared is not None:
             out = out + shared.float()
         if output_norm is not None:  # the sum goes to the norm as it is, in float32
-            from velox_amd.parts.base import ResidualCopy
+            from velox_amd.parts.base import ReadyInput, ResidualCopy
 
+            if output_norm.following is not None:
+                assert output_norm.mult == 1.0
+                form = output_norm.following.deferred_form()
+                return ReadyInput(self.norm_add_norm(output_norm.residual, out, output_norm.weight, output_norm.eps, form[0], form[1], out_dtype), output_norm.following)
             return ResidualCopy(self.norm_add(output_norm.residual, out, output_norm.weight, output_norm.eps, output_norm.mult, out_dtype))
         return out.to(out_dtype)
 

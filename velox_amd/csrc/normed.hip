@@ -4,6 +4,9 @@
 //   add_cast:       residual += delta; out = residual in the run dtype
 //   norm_add:       residual += mult * y * rsqrt(mean(y^2) + eps) * w; out = residual in the run dtype   (the norm on a
 //                   sub-layer's OUTPUT, float32 throughout, one rounding for the copy)
+//   norm_add_norm:  the same with the norm that reads the residual next in the same kernel: a norm behind one sub-layer, the
+//                   residual sum, the norm before the next sub-layer
+//   poly_norm:      a y1 + b y2 + c y3 + e with y_k = z^k / sqrt(mean(z^2k) + eps) over a row
 //   qk_norm_write:  RMS norm of the queries and of the keys (over the whole projection or per head), the query
 //                   temperature, the blend of the values with an earlier layer's, queries written at the kernels' head
 //                   size, keys and values into the paged cache (zeros in the padding channels)
@@ -190,6 +193,235 @@ extern "C" int velox_norm_add(float* residual, const void* y, int y_dtype, const
   if (hidden < 1 || partials < 1 || (partials > 1 && y_dtype != VELOX_F32)) return -1;
   if (y_dtype == VELOX_BF16) norm_add_launch<bf16_t>(residual, y, weight, out_bf16, tokens, hidden, eps, mult, partials, partial_stride, stream);
   else norm_add_launch<float>(residual, y, weight, out_bf16, tokens, hidden, eps, mult, partials, partial_stride, stream);
+  VELOX_RETURN_LAUNCH_STATUS();
+}
+
+// ---------------------------------------------------------------------------------------------
+// norm_add_norm: one workgroup per output row.  y' = y / sqrt(mean(y^2) + eps_y) * w_y;  r = residual + y' (written back unless
+// `rows` picks rows);  out = r / sqrt(mean(r^2) + eps) * w.  y may come as stacked float32 partial sums.  The row stays in
+// registers between the passes: PIECES pieces of four neighbours per lane (16-byte accesses; the launch picks the width), or,
+// for rows that are no multiple of four, in LDS.
+// ---------------------------------------------------------------------------------------------
+struct NormAddNormArgs {
+  float* residual;
+  const void* y;
+  const float* y_weight;
+  const float* weight;
+  const int* rows;
+  void* out;
+  int out_bf16, hidden, partials;
+  size_t partial_stride;
+  float y_eps, eps;
+};
+
+template <typename TD, int PIECES>
+__global__ void __launch_bounds__(1024) norm_add_norm_vec_kernel(const NormAddNormArgs a) {
+  __shared__ float scratch[16];
+  const size_t src = a.rows ? (size_t)a.rows[blockIdx.x] : (size_t)blockIdx.x;
+  const TD* y = (const TD*)a.y + src * a.hidden;
+  float* res = a.residual + src * a.hidden;
+  float4_t held[PIECES], old[PIECES], yw[PIECES];
+  float sumsq = 0.f;
+#pragma unroll
+  for (int c = 0; c < PIECES; ++c) {
+    const int at = (threadIdx.x + c * blockDim.x) * 4;
+    held[c] = old[c] = yw[c] = float4_t{0.f, 0.f, 0.f, 0.f};
+    if (at < a.hidden) {
+      for (int p = 0; p < a.partials; ++p) {
+        const Piece4<TD> q = *reinterpret_cast<const Piece4<TD>*>(y + p * a.partial_stride + at);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) held[c][j] += q.get(j);
+      }
+      old[c] = *reinterpret_cast<const float4_t*>(res + at);  // (asked for before the reduction: the wait hides behind it)
+      yw[c] = *reinterpret_cast<const float4_t*>(a.y_weight + at);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) sumsq += held[c][j] * held[c][j];
+    }
+  }
+  const float y_inv = 1.f / sqrtf(block_sum(sumsq, scratch) / (float)a.hidden + a.y_eps);
+  sumsq = 0.f;
+#pragma unroll
+  for (int c = 0; c < PIECES; ++c) {
+    const int at = (threadIdx.x + c * blockDim.x) * 4;
+    if (at < a.hidden) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        old[c][j] += held[c][j] * y_inv * yw[c][j];
+        sumsq += old[c][j] * old[c][j];
+      }
+      if (!a.rows) *reinterpret_cast<float4_t*>(res + at) = old[c];
+      yw[c] = *reinterpret_cast<const float4_t*>(a.weight + at);
+    }
+  }
+  const float inv = 1.f / sqrtf(block_sum(sumsq, scratch) / (float)a.hidden + a.eps);
+#pragma unroll
+  for (int c = 0; c < PIECES; ++c) {
+    const int at = (threadIdx.x + c * blockDim.x) * 4;
+    if (at < a.hidden) {
+      const float4_t o = old[c] * inv * yw[c];
+      const size_t to = (size_t)blockIdx.x * a.hidden + at;
+      if (a.out_bf16) {
+        short4_t bits;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) bits[j] = bf16_bits(o[j]);
+        *reinterpret_cast<short4_t*>((bf16_t*)a.out + to) = bits;
+      } else {
+        *reinterpret_cast<float4_t*>((float*)a.out + to) = o;
+      }
+    }
+  }
+}
+
+template <typename TD>
+__global__ void __launch_bounds__(256) norm_add_norm_kernel(const NormAddNormArgs a) {
+  extern __shared__ float held_row[];
+  __shared__ float scratch[16];
+  const size_t src = a.rows ? (size_t)a.rows[blockIdx.x] : (size_t)blockIdx.x;
+  const TD* y = (const TD*)a.y + src * a.hidden;
+  float* res = a.residual + src * a.hidden;
+  float sumsq = 0.f;
+  for (int i = threadIdx.x; i < a.hidden; i += 256) {  // (every lane reads back only what it wrote itself)
+    float v = 0.f;
+    for (int p = 0; p < a.partials; ++p) v += to_f32(y[p * a.partial_stride + i]);
+    held_row[i] = v;
+    sumsq += v * v;
+  }
+  const float y_inv = 1.f / sqrtf(block_sum(sumsq, scratch) / (float)a.hidden + a.y_eps);
+  sumsq = 0.f;
+  for (int i = threadIdx.x; i < a.hidden; i += 256) {
+    const float r = res[i] + held_row[i] * y_inv * a.y_weight[i];
+    held_row[i] = r;
+    if (!a.rows) res[i] = r;
+    sumsq += r * r;
+  }
+  const float inv = 1.f / sqrtf(block_sum(sumsq, scratch) / (float)a.hidden + a.eps);
+  for (int i = threadIdx.x; i < a.hidden; i += 256) {
+    const float o = held_row[i] * inv * a.weight[i];
+    const size_t to = (size_t)blockIdx.x * a.hidden + i;
+    if (a.out_bf16) ((bf16_t*)a.out)[to] = (bf16_t)o;
+    else ((float*)a.out)[to] = o;
+  }
+}
+
+template <typename TD>
+static void norm_add_norm_launch(const NormAddNormArgs& a, int count, hipStream_t stream) {
+  const uintptr_t addresses = (uintptr_t)a.residual | (uintptr_t)a.y | (uintptr_t)a.y_weight | (uintptr_t)a.weight | (uintptr_t)a.out;
+  if (a.hidden % 4 == 0 && addresses % 16 == 0 && a.partial_stride % 4 == 0) {
+    const int pieces = a.hidden / 4;
+    // few rows: a lane per piece as long as that is possible (the kernel is a chain of waits); many rows: two pieces a lane
+    int lanes = count <= 64 || pieces <= 256 ? pieces : (pieces + 1) / 2;
+    lanes = (lanes + 63) / 64 * 64;
+    if (lanes > 1024) lanes = 1024;
+    const int per_lane = (pieces + lanes - 1) / lanes;
+    if (per_lane <= 1) norm_add_norm_vec_kernel<TD, 1><<<count, lanes, 0, stream>>>(a);
+    else if (per_lane <= 2) norm_add_norm_vec_kernel<TD, 2><<<count, lanes, 0, stream>>>(a);
+    else norm_add_norm_vec_kernel<TD, 4><<<count, lanes, 0, stream>>>(a);  // (hidden <= 16,384)
+    return;
+  }
+  norm_add_norm_kernel<TD><<<count, 256, (size_t)a.hidden * sizeof(float), stream>>>(a);
+}
+
+extern "C" int velox_norm_add_norm(float* residual, const void* y, int y_dtype, const float* y_weight, float y_eps, const float* weight, float eps,
+                                   const int* rows, void* out, int out_dtype, int count, int hidden, int partials, long long partial_stride,
+                                   hipStream_t stream) {
+  if (count <= 0) return 0;
+  if (hidden < 1 || hidden > 16384 - 32 || partials < 1 || (partials > 1 && y_dtype != VELOX_F32)) return (int)hipErrorInvalidValue;
+  NormAddNormArgs a{residual, y, y_weight, weight, rows, out, out_dtype == VELOX_BF16, hidden, partials, (size_t)partial_stride, y_eps, eps};
+  if (y_dtype == VELOX_BF16) norm_add_norm_launch<bf16_t>(a, count, stream);
+  else norm_add_norm_launch<float>(a, count, stream);
+  VELOX_RETURN_LAUNCH_STATUS();
+}
+
+// ---------------------------------------------------------------------------------------------
+// poly_norm: one workgroup per row of `width` values z; out = a z / n1 + b z^2 / n2 + c z^3 / n3 + e with n_k = sqrt(mean(z^2k) + eps);
+// coef = (a, b, c, e) float32 on the device.  Rows of a multiple of four lie in registers as pieces of four (PIECES a lane);
+// others, and longer ones, are read twice.
+// ---------------------------------------------------------------------------------------------
+__device__ __forceinline__ void block_sum3(float& x, float& y, float& z, float* scratch) {
+  const int lane = threadIdx.x & (VELOX_WAVE - 1), wave = threadIdx.x / VELOX_WAVE, waves = (blockDim.x + VELOX_WAVE - 1) / VELOX_WAVE;
+  x = wave_sum(x);
+  y = wave_sum(y);
+  z = wave_sum(z);
+  if (lane == 0) { scratch[wave] = x; scratch[16 + wave] = y; scratch[32 + wave] = z; }
+  __syncthreads();
+  x = y = z = 0.f;
+  for (int w = 0; w < waves; ++w) { x += scratch[w]; y += scratch[16 + w]; z += scratch[32 + w]; }
+}
+
+template <typename T, int PIECES>
+__global__ void __launch_bounds__(1024) poly_norm_kernel(const T* __restrict__ in, T* __restrict__ out, const float* __restrict__ coef, int width, float eps) {
+  __shared__ float scratch[48];
+  const T* src = in + (size_t)blockIdx.x * width;
+  T* dst = out + (size_t)blockIdx.x * width;
+  const float ca = coef[0], cb = coef[1], cc = coef[2], ce = coef[3];
+  float s1 = 0.f, s2 = 0.f, s3 = 0.f;
+  Piece4<T> held[PIECES > 0 ? PIECES : 1];
+  if constexpr (PIECES > 0) {
+#pragma unroll
+    for (int p = 0; p < PIECES; ++p) {
+      const int at = (threadIdx.x + p * blockDim.x) * 4;
+      if (at < width) {
+        held[p] = *reinterpret_cast<const Piece4<T>*>(src + at);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const float z = held[p].get(j), q = z * z;
+          s1 += q; s2 += q * q; s3 += q * q * q;
+        }
+      }
+    }
+  } else {
+    for (int i = threadIdx.x; i < width; i += blockDim.x) {
+      const float z = to_f32(src[i]), q = z * z;
+      s1 += q; s2 += q * q; s3 += q * q * q;
+    }
+  }
+  block_sum3(s1, s2, s3, scratch);
+  const float n1 = ca / sqrtf(s1 / (float)width + eps), n2 = cb / sqrtf(s2 / (float)width + eps), n3 = cc / sqrtf(s3 / (float)width + eps);
+  if constexpr (PIECES > 0) {
+#pragma unroll
+    for (int p = 0; p < PIECES; ++p) {
+      const int at = (threadIdx.x + p * blockDim.x) * 4;
+      if (at < width) {
+        Piece4<T> o;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const float z = held[p].get(j);
+          const float v = z * (n1 + z * (n2 + z * n3)) + ce;
+          if constexpr (sizeof(T) == 2) o.v[j] = bf16_bits(v);
+          else o.v[j] = v;
+        }
+        *reinterpret_cast<Piece4<T>*>(dst + at) = o;
+      }
+    }
+  } else {
+    for (int i = threadIdx.x; i < width; i += blockDim.x) {
+      const float z = to_f32(src[i]);
+      dst[i] = from_f32<T>(z * (n1 + z * (n2 + z * n3)) + ce);
+    }
+  }
+}
+
+template <typename T>
+static void poly_norm_launch(const void* in, void* out, const float* coef, int tokens, int width, float eps, hipStream_t stream) {
+  const T* src = (const T*)in;
+  T* dst = (T*)out;
+  const bool aligned = width % 4 == 0 && (((uintptr_t)in | (uintptr_t)out) & 15) == 0;
+  const int pieces = width / 4;
+  int lanes = tokens <= 64 ? pieces : (pieces + 3) / 4;
+  lanes = (lanes + 63) / 64 * 64;
+  lanes = lanes < 64 ? 64 : lanes > 1024 ? 1024 : lanes;
+  const int per_lane = (pieces + lanes - 1) / lanes;
+  if (!aligned || per_lane > 8) poly_norm_kernel<T, 0><<<tokens, 1024, 0, stream>>>(src, dst, coef, width, eps);
+  else if (per_lane <= 1) poly_norm_kernel<T, 1><<<tokens, lanes, 0, stream>>>(src, dst, coef, width, eps);
+  else if (per_lane <= 4) poly_norm_kernel<T, 4><<<tokens, lanes, 0, stream>>>(src, dst, coef, width, eps);
+  else poly_norm_kernel<T, 8><<<tokens, lanes, 0, stream>>>(src, dst, coef, width, eps);
+}
+
+extern "C" int velox_poly_norm(const void* in, void* out, const float* coef, int tokens, int width, float eps, int dtype, hipStream_t stream) {
+  if (tokens <= 0) return 0;
+  if (width < 1) return (int)hipErrorInvalidValue;
+  if (dtype == VELOX_BF16) poly_norm_launch<bf16_t>(in, out, coef, tokens, width, eps, stream);
+  else poly_norm_launch<float>(in, out, coef, tokens, width, eps, stream);
   VELOX_RETURN_LAUNCH_STATUS();
 }
 

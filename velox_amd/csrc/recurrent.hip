@@ -4,6 +4,7 @@
 //   short_conv          causal convolution over a few taps per channel, the inputs before a portion's start from the state slot
 //   rotate_pad_write    partial rotation of q and k, q at the attention kernels' head size, k and v into the paged cache
 //   recurrence_prepare  unit q and k, decay and beta of a linear recurrence, all float32
+//   removal_prepare     the same for the generalized delta rule: unit keys and their lengths, removal vectors, the decay's map
 //   linear_scan         the recurrence itself, token by token from the state slot (portions of prompts staged through LDS)
 //   gated_head_norm     RMS norm of each head's read-out, a shared weight, a gate
 // Everything between a load and a store is float32; stores round once.  No result depends on how a sequence's tokens
@@ -373,14 +374,17 @@ extern "C" int velox_short_conv(const void* x, int ld, int channels, const float
 // channels of every query and key head are rotated (channel i with i + half, or 2i with 2i + 1 when `interleaved`; cos/sin
 // float32 [positions, half]; (u, v) -> (u cos - v sin, v cos + u sin)); queries go to
 // q_out [T, heads * D], keys to k_cache [pages, kv_heads, page, D], values to v_cache [pages, kv_heads, D, page]; channels from
-// dim (vdim) to D are zeros.
+// dim (vdim) to D are zeros.  With `post_norm_eps` > 0 a rotated query or key head is divided by sqrt(mean(x^2) + eps) over its
+// `dim` channels (a head is one workgroup's, its sum one reduction in a fixed order).  With `values_are_keys` a row holds no
+// values: a value head is its key head as it stands in the row.
 // ---------------------------------------------------------------------------------------------
 template <typename T>
 __global__ void __launch_bounds__(256) rotate_pad_write_kernel(const T* __restrict__ qkv, int ld, T* __restrict__ q_out, const int* __restrict__ positions,
                                                                const float* __restrict__ cos_t, const float* __restrict__ sin_t, int half,
                                                                const int* __restrict__ slot_mapping, T* __restrict__ k_cache, T* __restrict__ v_cache,
                                                                int heads, int kv_heads, int dim, int vdim, int D, int page_shift, int write_kv,
-                                                               int interleaved) {
+                                                               int interleaved, float post_norm_eps, int values_are_keys) {
+  __shared__ float scratch[16];
   const int t = blockIdx.x;
   const T* row = qkv + (size_t)t * ld;
   const int q_size = heads * dim, k_size = kv_heads * dim;
@@ -397,7 +401,7 @@ __global__ void __launch_bounds__(256) rotate_pad_write_kernel(const T* __restri
   for (int h = blockIdx.y; h < all_heads; h += gridDim.y) {  // (a step of few tokens has a workgroup per head, a long one a few per token)
     if (h >= heads + kv_heads) {  // a value head
       const int g = h - heads - kv_heads;
-      const T* values = row + q_size + k_size + g * vdim;
+      const T* values = values_are_keys ? row + q_size + g * dim : row + q_size + k_size + g * vdim;
       for (int c = threadIdx.x; c < D; c += blockDim.x)
         v_cache[(((size_t)page * kv_heads + g) * D + c) * page_size + offset] = c < vdim ? values[c] : from_f32<T>(0.f);
       continue;
@@ -406,40 +410,46 @@ __global__ void __launch_bounds__(256) rotate_pad_write_kernel(const T* __restri
     const int g = is_q ? h : h - heads;
     const T* src = row + (is_q ? h * dim : q_size + g * dim);
     T* dst = is_q ? q_out + ((size_t)t * heads + h) * D : k_cache + (((size_t)page * kv_heads + g) * page_size + offset) * D;
-    for (int c = threadIdx.x; c < D; c += blockDim.x) {
-      float v = 0.f;
-      if (c < dim) {
-        v = to_f32(src[c]);
-        if (interleaved) {
-          if (c < 2 * half) {
-            const int i = c >> 1;
-            v = (c & 1) ? v * cs[i] + to_f32(src[c - 1]) * sn[i] : v * cs[i] - to_f32(src[c + 1]) * sn[i];
-          }
-        } else if (c < half) v = v * cs[c] - to_f32(src[c + half]) * sn[c];
-        else if (c < 2 * half) v = v * cs[c - half] + to_f32(src[c - half]) * sn[c - half];
+    auto rotated = [&](int c) -> float {  // channel c < dim behind the rotation
+      const float v = to_f32(src[c]);
+      if (interleaved) {
+        if (c >= 2 * half) return v;
+        const int i = c >> 1;
+        return (c & 1) ? v * cs[i] + to_f32(src[c - 1]) * sn[i] : v * cs[i] - to_f32(src[c + 1]) * sn[i];
       }
-      dst[c] = from_f32<T>(v);
+      if (c < half) return v * cs[c] - to_f32(src[c + half]) * sn[c];
+      if (c < 2 * half) return v * cs[c - half] + to_f32(src[c - half]) * sn[c - half];
+      return v;
+    };
+    float inv = 1.f;
+    if (post_norm_eps > 0.f) {
+      float sum = 0.f;
+      for (int c = threadIdx.x; c < dim; c += blockDim.x) { const float v = rotated(c); sum += v * v; }
+      inv = 1.f / sqrtf(block_sum(sum, scratch) / (float)dim + post_norm_eps);
     }
+    for (int c = threadIdx.x; c < D; c += blockDim.x) dst[c] = from_f32<T>(c < dim ? rotated(c) * inv : 0.f);
   }
 }
 
 extern "C" int velox_rotate_pad_write(const void* qkv, int ld, void* q_out, const int* positions, const float* cos_t, const float* sin_t, int half,
                                       const int* slot_mapping, void* k_cache, void* v_cache, int tokens, int heads, int kv_heads, int dim, int vdim, int D,
-                                      int page_size, int write_kv, int dtype, int interleaved, hipStream_t stream) {
+                                      int page_size, int write_kv, int dtype, int interleaved, float post_norm_eps, int values_are_keys, hipStream_t stream) {
   if (tokens <= 0) return 0;
   int shift = 0;
   while ((1 << shift) < page_size) ++shift;
-  if ((1 << shift) != page_size || 2 * half > dim || dim > D || vdim > D) return (int)hipErrorInvalidValue;
+  if ((1 << shift) != page_size || 2 * half > dim || dim > D || vdim > D || (values_are_keys && vdim != dim)) return (int)hipErrorInvalidValue;
   const int all_heads = heads + (write_kv ? 2 * kv_heads : 0);
   const dim3 grid(tokens, tokens <= 256 ? all_heads : (all_heads < 4 ? all_heads : 4));
   int lanes = (D + 63) / 64 * 64;
   if (lanes > 256) lanes = 256;
   if (dtype == VELOX_BF16)
     rotate_pad_write_kernel<bf16_t><<<grid, lanes, 0, stream>>>((const bf16_t*)qkv, ld, (bf16_t*)q_out, positions, cos_t, sin_t, half, slot_mapping,
-                                                              (bf16_t*)k_cache, (bf16_t*)v_cache, heads, kv_heads, dim, vdim, D, shift, write_kv, interleaved);
+                                                              (bf16_t*)k_cache, (bf16_t*)v_cache, heads, kv_heads, dim, vdim, D, shift, write_kv, interleaved,
+                                                              post_norm_eps, values_are_keys);
   else
     rotate_pad_write_kernel<float><<<grid, lanes, 0, stream>>>((const float*)qkv, ld, (float*)q_out, positions, cos_t, sin_t, half, slot_mapping,
-                                                             (float*)k_cache, (float*)v_cache, heads, kv_heads, dim, vdim, D, shift, write_kv, interleaved);
+                                                             (float*)k_cache, (float*)v_cache, heads, kv_heads, dim, vdim, D, shift, write_kv, interleaved,
+                                                             post_norm_eps, values_are_keys);
   VELOX_RETURN_LAUNCH_STATUS();
 }
 
@@ -508,9 +518,120 @@ extern "C" int velox_recurrence_prepare(const void* qkv, int qkv_dtype, int ld, 
 }
 
 // ---------------------------------------------------------------------------------------------
+// removal_prepare: what the generalized delta rule reads besides its values, all float32, from a row of the input product
+//   (`main`: read vectors at r_at, keys at k_at, removal logits at a_at, heads * dim each, and the low-rank map's inner row
+//   at low_at, `rank` long).  Per head, with n = sqrt(sum(k^2) + 1e-6), u = k / n and a = sigmoid(a_logit + a_bias):
+//   vectors [T, heads, 3, dim] = r, u, a * u;   lengths [T, heads] = n (so that the key itself is n * u);
+//   decay [T, heads * dim] = exp(-scale * sigmoid(w0 + w2 . tanh(inner row))),  w2 [heads * dim, rank] in the run dtype.
+// Grid (heads, groups of TOK tokens), 256 lanes: waves take the group's tokens in turn for the vectors; for the decays a
+// lane takes one channel and up to REMOVAL_TOKENS tokens at a time, so a row of w2 is read once for several tokens.  A sum
+// over the inner row runs from first to last whatever the group.
+// ---------------------------------------------------------------------------------------------
+#define REMOVAL_TOKENS 4
+struct RemovalArgs {
+  const void* main;
+  int ld, r_at, k_at, a_at, low_at, rank, heads, dim;
+  const float* a_bias;
+  const void* w2;
+  const float* w0;
+  float scale;
+  float* vectors;
+  float* decay;
+  float* lengths;
+  int tokens, group;
+};
+
+template <typename T>
+__global__ void __launch_bounds__(256) removal_prepare_kernel(const RemovalArgs a) {
+  extern __shared__ float inner[];  // [group, rank], behind the tanh
+  const int h = blockIdx.x, t0 = blockIdx.y * a.group;
+  const int count = a.tokens - t0 < a.group ? a.tokens - t0 : a.group;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int dim = a.dim, rank = a.rank;
+  const T* rows = (const T*)a.main + (size_t)t0 * a.ld;
+  for (int i = threadIdx.x; i < count * rank; i += 256) {
+    const int j = i / rank;
+    inner[i] = tanhf(to_f32(rows[(size_t)j * a.ld + a.low_at + (i - j * rank)]));
+  }
+  const float* bias = a.a_bias + (size_t)h * dim;
+  for (int j = wave; j < count; j += 4) {
+    const T* row = rows + (size_t)j * a.ld + (size_t)h * dim;
+    float s = 0.f;
+    for (int c = lane; c < dim; c += 64) { const float v = to_f32(row[a.k_at + c]); s += v * v; }
+    const float n = sqrtf(wave_sum(s) + 1e-6f), inv = 1.f / n;
+    const size_t pair = (size_t)(t0 + j) * a.heads + h;
+    float* dst = a.vectors + pair * 3 * dim;
+    for (int c = lane; c < dim; c += 64) {
+      const float u = to_f32(row[a.k_at + c]) * inv;
+      dst[c] = to_f32(row[a.r_at + c]);
+      dst[dim + c] = u;
+      dst[2 * dim + c] = sigmoid_f32(to_f32(row[a.a_at + c]) + bias[c]) * u;
+    }
+    if (lane == 0) a.lengths[pair] = n;
+  }
+  __syncthreads();
+  const int quads = (count + REMOVAL_TOKENS - 1) / REMOVAL_TOKENS;
+  const bool vec = sizeof(T) == 2 && rank % 8 == 0 && ((uintptr_t)a.w2 & 15) == 0;
+  for (int i = threadIdx.x; i < dim * quads; i += 256) {
+    const int c = i % dim, j0 = (i / dim) * REMOVAL_TOKENS;
+    const size_t channel = (size_t)h * dim + c;
+    const T* w = (const T*)a.w2 + channel * rank;
+    float z[REMOVAL_TOKENS];
+    const float* x[REMOVAL_TOKENS];
+#pragma unroll
+    for (int j = 0; j < REMOVAL_TOKENS; ++j) {
+      z[j] = 0.f;
+      x[j] = inner + (j0 + j < count ? j0 + j : count - 1) * rank;  // (a place beyond the group follows the last token and is not stored)
+    }
+    if (vec) {
+      for (int m = 0; m < rank; m += 8) {
+        const float4_t raw = *reinterpret_cast<const float4_t*>(w + m);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const unsigned bits = __float_as_uint(raw[e]);
+          const float lo = __uint_as_float(bits << 16), hi = __uint_as_float(bits & 0xffff0000u);
+#pragma unroll
+          for (int j = 0; j < REMOVAL_TOKENS; ++j) {
+            z[j] += lo * x[j][m + 2 * e];
+            z[j] += hi * x[j][m + 2 * e + 1];
+          }
+        }
+      }
+    } else {
+      for (int m = 0; m < rank; ++m) {
+        const float wm = to_f32(w[m]);
+#pragma unroll
+        for (int j = 0; j < REMOVAL_TOKENS; ++j) z[j] += wm * x[j][m];
+      }
+    }
+    const float start = a.w0[channel];
+#pragma unroll
+    for (int j = 0; j < REMOVAL_TOKENS; ++j)
+      if (j0 + j < count) a.decay[(size_t)(t0 + j0 + j) * a.heads * dim + channel] = expf(-a.scale * sigmoid_f32(start + z[j]));
+  }
+}
+
+extern "C" int velox_removal_prepare(const void* main, int dtype, int ld, int r_at, int k_at, int a_at, int low_at, int rank, int heads, int dim,
+                                     const float* a_bias, const void* w2, const float* w0, float scale, float* vectors, float* decay, float* lengths,
+                                     int tokens, hipStream_t stream) {
+  if (tokens <= 0) return 0;
+  if (rank < 1 || rank > 8192 || heads < 1 || dim < 1) return (int)hipErrorInvalidValue;
+  int group = tokens <= 16 ? 1 : tokens <= 256 ? REMOVAL_TOKENS : 16;  // (few tokens: a workgroup per token and head)
+  while (group > 1 && group * rank > 8192) group >>= 1;
+  const int groups = (tokens + group - 1) / group;
+  if (groups > 65535) return (int)hipErrorInvalidValue;
+  RemovalArgs a{main, ld, r_at, k_at, a_at, low_at, rank, heads, dim, a_bias, w2, w0, scale, vectors, decay, lengths, tokens, group};
+  const size_t lds = (size_t)group * rank * sizeof(float);
+  if (dtype == VELOX_BF16) removal_prepare_kernel<bf16_t><<<dim3(heads, groups), 256, lds, stream>>>(a);
+  else removal_prepare_kernel<float><<<dim3(heads, groups), 256, lds, stream>>>(a);
+  VELOX_RETURN_LAUNCH_STATUS();
+}
+
+// ---------------------------------------------------------------------------------------------
 // linear_scan.  Per sequence and head a state S of dim x vdim float32 numbers (rows: key channels) in state[slot, head].
 // Every column of S is a recurrence of its own:   s <- g * s;  u = beta (v_e - k . s)  (delta rule)  or  u = v_e;
-// s <- s + k u;  o_e = q . s.   A column is held by R lanes of a wave, SCAN_ROWS consecutive rows each (R the smallest power of
+// s <- s + k u;  o_e = q . s.   With a third vector b per token (`removal`: the generalized delta rule; k is then a unit vector
+// and beta its length):   d = k . s;  s <- g * s - b d + k (beta v_e)  (d from the old s);  o_e = q . s.   A column is held by R lanes of a wave, SCAN_ROWS consecutive rows each (R the smallest power of
 // two with R * SCAN_ROWS >= dim: a function of dim alone, so the order of every sum is too); the two dot products are
 // summed in four interleaved parts per lane and then over those lanes (scan_token, the one place where a token is worked).
 // With eight rows to a lane a head of 128 key channels spreads over sixteen lanes, and a workgroup holds sixteen columns.
@@ -547,7 +668,7 @@ __device__ __forceinline__ float sum_over_lanes(float v) {
 }
 
 struct ScanArgs {
-  const float* qk;       // [T, kv_heads, 2, dim]
+  const float* qk;       // [T, kv_heads, 2, dim]: q and k of a head; with the removal rule [T, kv_heads, 3, dim]: q, k, b
   const void* v;         // [T, v_ld], a token's values at v_at
   int v_bf16, v_ld, v_at;
   const float* decay;    // [T, heads * dim] or [T, heads]
@@ -574,10 +695,23 @@ __device__ __forceinline__ void scan_load_rows(const float* __restrict__ p, int 
 }
 
 // One token of one column: returns the read-out (complete in every lane of the column).
-template <int R>
+template <int R, bool REMOVAL>
 __device__ __forceinline__ float scan_token(float (&s)[SCAN_ROWS], const float (&q)[SCAN_ROWS], const float (&k)[SCAN_ROWS], const float (&dec)[SCAN_ROWS],
-                                            float val, float bet, int delta) {
+                                            const float (&rem)[SCAN_ROWS], float val, float bet, int delta) {
   float d[4] = {0.f, 0.f, 0.f, 0.f};
+  if constexpr (REMOVAL) {
+#pragma unroll
+    for (int i = 0; i < SCAN_ROWS; ++i) d[i & 3] += s[i] * k[i];
+    const float dot = sum_over_lanes<R>((d[0] + d[1]) + (d[2] + d[3]));
+    const float write = bet * val;
+    float p[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < SCAN_ROWS; ++i) {
+      s[i] = s[i] * dec[i] + (k[i] * write - rem[i] * dot);
+      p[i & 3] += s[i] * q[i];
+    }
+    return sum_over_lanes<R>((p[0] + p[1]) + (p[2] + p[3]));
+  }
 #pragma unroll
   for (int i = 0; i < SCAN_ROWS; ++i) {
     s[i] *= dec[i];
@@ -597,7 +731,7 @@ __device__ __forceinline__ float scan_token(float (&s)[SCAN_ROWS], const float (
   return sum_over_lanes<R>((p[0] + p[1]) + (p[2] + p[3]));
 }
 
-template <int R>
+template <int R, bool REMOVAL>
 __global__ void __launch_bounds__(256) linear_scan_kernel(const ScanArgs a) {
   const int r = threadIdx.x % R;
   const int e = blockIdx.x * (256 / R) + threadIdx.x / R;
@@ -615,12 +749,13 @@ __global__ void __launch_bounds__(256) linear_scan_kernel(const ScanArgs a) {
 #pragma unroll
   for (int i = 0; i < SCAN_ROWS; ++i) s[i] = d0 + i < dim ? S[(size_t)(d0 + i) * vdim] : 0.f;
 
-  float q[SCAN_ROWS], k[SCAN_ROWS], dec[SCAN_ROWS], qn[SCAN_ROWS], kn[SCAN_ROWS], decn[SCAN_ROWS];
+  float q[SCAN_ROWS], k[SCAN_ROWS], dec[SCAN_ROWS], rem[SCAN_ROWS], qn[SCAN_ROWS], kn[SCAN_ROWS], decn[SCAN_ROWS], remn[SCAN_ROWS];
   float val, bet, valn = 0.f, betn = 1.f;
-  auto fetch = [&](int t, float (&fq)[SCAN_ROWS], float (&fk)[SCAN_ROWS], float (&fd)[SCAN_ROWS], float& fv, float& fb) {
-    const float* base = a.qk + ((size_t)t * a.kv_heads + g) * 2 * dim;
+  auto fetch = [&](int t, float (&fq)[SCAN_ROWS], float (&fk)[SCAN_ROWS], float (&fd)[SCAN_ROWS], float (&fr)[SCAN_ROWS], float& fv, float& fb) {
+    const float* base = a.qk + ((size_t)t * a.kv_heads + g) * (REMOVAL ? 3 : 2) * dim;
     scan_load_rows(base, d0, dim, vec, 0.f, fq);
     scan_load_rows(base + dim, d0, dim, vec, 0.f, fk);
+    if constexpr (REMOVAL) scan_load_rows(base + 2 * dim, d0, dim, vec, 0.f, fr);
     if (a.decay_per_channel) {
       scan_load_rows(a.decay + ((size_t)t * a.heads + h) * dim, d0, dim, vec, 1.f, fd);
     } else {
@@ -631,13 +766,13 @@ __global__ void __launch_bounds__(256) linear_scan_kernel(const ScanArgs a) {
     fv = load_as_f32(a.v, a.v_bf16, (size_t)t * a.v_ld + a.v_at + (size_t)h * vdim + col);
     fb = a.beta ? a.beta[(size_t)t * a.heads + h] : 1.f;
   };
-  fetch(lo, q, k, dec, val, bet);
+  fetch(lo, q, k, dec, rem, val, bet);
   for (int t = lo; t < hi; ++t) {
-    if (t + 1 < hi) fetch(t + 1, qn, kn, decn, valn, betn);
-    const float o = scan_token<R>(s, q, k, dec, val, bet, a.delta);
+    if (t + 1 < hi) fetch(t + 1, qn, kn, decn, remn, valn, betn);
+    const float o = scan_token<R, REMOVAL>(s, q, k, dec, rem, val, bet, a.delta);
     if (live && r == 0) a.out[((size_t)t * a.heads + h) * vdim + e] = o;
 #pragma unroll
-    for (int i = 0; i < SCAN_ROWS; ++i) { q[i] = qn[i]; k[i] = kn[i]; dec[i] = decn[i]; }
+    for (int i = 0; i < SCAN_ROWS; ++i) { q[i] = qn[i]; k[i] = kn[i]; dec[i] = decn[i]; rem[i] = remn[i]; }
     val = valn; bet = betn;
   }
   if (live) {
@@ -647,12 +782,12 @@ __global__ void __launch_bounds__(256) linear_scan_kernel(const ScanArgs a) {
   }
 }
 
-// A token's place in a staging buffer, in floats: q [dim], k [dim], the decay per channel [dim] if there is one, the values of
+// A token's place in a staging buffer, in floats: q [dim], k [dim] (and b [dim] with the removal rule), the decay per channel [dim] if there is one, the values of
 // the workgroup's columns [256 / R], then beta and the head's decay (and two floats that keep the next token 16-byte aligned).
 #define STAGE_PIECES 8  // 16-byte pieces of q, k and decay that one lane carries per block of tokens, at most
 #define STAGE_VALUES 4  // values that one lane carries per block, at most
 
-template <int R>
+template <int R, bool REMOVAL>
 __global__ void __launch_bounds__(256) linear_scan_staged_kernel(const ScanArgs a, const int block_tokens) {
   extern __shared__ float4_t stage_pieces[];
   float* stage = reinterpret_cast<float*>(stage_pieces);
@@ -669,9 +804,10 @@ __global__ void __launch_bounds__(256) linear_scan_staged_kernel(const ScanArgs 
   const int d0 = r * SCAN_ROWS;
   const int g = h / (heads / a.kv_heads);
   const int per_channel = a.decay_per_channel;
-  const int qk_pieces = dim / 2;                                     // (2 * dim floats in pieces of 4)
+  constexpr int VECTORS = REMOVAL ? 3 : 2;
+  const int qk_pieces = VECTORS * dim / 4;                           // (VECTORS * dim floats in pieces of 4; dim is a multiple of 4)
   const int pieces_per_token = qk_pieces + (per_channel ? dim / 4 : 0);
-  const int values_at = 2 * dim + (per_channel ? dim : 0);
+  const int values_at = VECTORS * dim + (per_channel ? dim : 0);
   const int scalars_at = values_at + COLS;
   const int stride = scalars_at + 4;
 
@@ -693,7 +829,7 @@ __global__ void __launch_bounds__(256) linear_scan_staged_kernel(const ScanArgs 
     for (int p = 0; p < STAGE_PIECES; ++p) {
       const int t = t0 + piece_token[p];
       if (piece_token[p] >= 0 && t < hi) {
-        const float* from = piece_from[p] >= 0 ? a.qk + ((size_t)t * a.kv_heads + g) * 2 * dim + piece_from[p]
+        const float* from = piece_from[p] >= 0 ? a.qk + ((size_t)t * a.kv_heads + g) * VECTORS * dim + piece_from[p]
                                                : a.decay + ((size_t)t * heads + h) * dim + (-1 - piece_from[p]);
         carried[p] = *reinterpret_cast<const float4_t*>(from);
       }
@@ -737,9 +873,10 @@ __global__ void __launch_bounds__(256) linear_scan_staged_kernel(const ScanArgs 
 #pragma unroll
   for (int i = 0; i < SCAN_ROWS; ++i) s[i] = d0 + i < dim ? S[(size_t)(d0 + i) * vdim] : 0.f;
 
-  float q[SCAN_ROWS], k[SCAN_ROWS], dec[SCAN_ROWS], qn[SCAN_ROWS], kn[SCAN_ROWS], decn[SCAN_ROWS];  // two sets of operands, used in turn
+  // two sets of operands, used in turn
+  float q[SCAN_ROWS], k[SCAN_ROWS], dec[SCAN_ROWS], rem[SCAN_ROWS], qn[SCAN_ROWS], kn[SCAN_ROWS], decn[SCAN_ROWS], remn[SCAN_ROWS];
   float val, bet, valn = 0.f, betn = 1.f;
-  auto fetch = [&](int at, float (&fq)[SCAN_ROWS], float (&fk)[SCAN_ROWS], float (&fd)[SCAN_ROWS], float& fv, float& fb) {
+  auto fetch = [&](int at, float (&fq)[SCAN_ROWS], float (&fk)[SCAN_ROWS], float (&fd)[SCAN_ROWS], float (&fr)[SCAN_ROWS], float& fv, float& fb) {
     const float one = stage[at + scalars_at + 1];
 #pragma unroll
     for (int i = 0; i < SCAN_ROWS; i += 4) {
@@ -748,8 +885,12 @@ __global__ void __launch_bounds__(256) linear_scan_staged_kernel(const ScanArgs 
         const float4_t y = *reinterpret_cast<const float4_t*>(&stage[at + dim + d0 + i]);
         fq[i] = x[0]; fq[i + 1] = x[1]; fq[i + 2] = x[2]; fq[i + 3] = x[3];
         fk[i] = y[0]; fk[i + 1] = y[1]; fk[i + 2] = y[2]; fk[i + 3] = y[3];
+        if constexpr (REMOVAL) {
+          const float4_t b4 = *reinterpret_cast<const float4_t*>(&stage[at + 2 * dim + d0 + i]);
+          fr[i] = b4[0]; fr[i + 1] = b4[1]; fr[i + 2] = b4[2]; fr[i + 3] = b4[3];
+        }
         if (per_channel) {
-          const float4_t z = *reinterpret_cast<const float4_t*>(&stage[at + 2 * dim + d0 + i]);
+          const float4_t z = *reinterpret_cast<const float4_t*>(&stage[at + VECTORS * dim + d0 + i]);
           fd[i] = z[0]; fd[i + 1] = z[1]; fd[i + 2] = z[2]; fd[i + 3] = z[3];
         } else {
           fd[i] = fd[i + 1] = fd[i + 2] = fd[i + 3] = one;
@@ -757,6 +898,7 @@ __global__ void __launch_bounds__(256) linear_scan_staged_kernel(const ScanArgs 
       } else {
         fq[i] = fq[i + 1] = fq[i + 2] = fq[i + 3] = 0.f;
         fk[i] = fk[i + 1] = fk[i + 2] = fk[i + 3] = 0.f;
+        if constexpr (REMOVAL) fr[i] = fr[i + 1] = fr[i + 2] = fr[i + 3] = 0.f;
         fd[i] = fd[i + 1] = fd[i + 2] = fd[i + 3] = 1.f;
       }
     }
@@ -773,18 +915,18 @@ __global__ void __launch_bounds__(256) linear_scan_staged_kernel(const ScanArgs 
     if (more) load_block(t0 + block_tokens);
     const int count = hi - t0 < block_tokens ? hi - t0 : block_tokens;
     const int at = buffer * block_tokens * stride;
-    fetch(at, q, k, dec, val, bet);
+    fetch(at, q, k, dec, rem, val, bet);
     int j = 0;
     for (; j + 1 < count; j += 2) {  // (a token's operands are read from LDS while the token before it is worked)
-      fetch(at + (j + 1) * stride, qn, kn, decn, valn, betn);
-      const float o0 = scan_token<R>(s, q, k, dec, val, bet, a.delta);
+      fetch(at + (j + 1) * stride, qn, kn, decn, remn, valn, betn);
+      const float o0 = scan_token<R, REMOVAL>(s, q, k, dec, rem, val, bet, a.delta);
       if (live && r == 0) a.out[((size_t)(t0 + j) * heads + h) * vdim + e] = o0;
-      if (j + 2 < count) fetch(at + (j + 2) * stride, q, k, dec, val, bet);
-      const float o1 = scan_token<R>(s, qn, kn, decn, valn, betn, a.delta);
+      if (j + 2 < count) fetch(at + (j + 2) * stride, q, k, dec, rem, val, bet);
+      const float o1 = scan_token<R, REMOVAL>(s, qn, kn, decn, remn, valn, betn, a.delta);
       if (live && r == 0) a.out[((size_t)(t0 + j + 1) * heads + h) * vdim + e] = o1;
     }
     if (j < count) {
-      const float o = scan_token<R>(s, q, k, dec, val, bet, a.delta);
+      const float o = scan_token<R, REMOVAL>(s, q, k, dec, rem, val, bet, a.delta);
       if (live && r == 0) a.out[((size_t)(t0 + j) * heads + h) * vdim + e] = o;
     }
     if (more) store_block(buffer ^ 1);  // (the buffer that the block before this one was worked from: everyone is past the barrier behind it)
@@ -838,14 +980,15 @@ __device__ __forceinline__ void send_to_lds_2(const void* src, const void* to) {
   asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tglobal_load_lds_ushort %1, off" : : "s"(lds_address_of_wave(to)), "v"(src) : "memory", "m0");
 }
 
-// A staging buffer of linear_scan_wave_kernel, in floats: q and k of the block's tokens [tokens, 2 dim], the decays per channel
+// A staging buffer of linear_scan_wave_kernel, in floats: q and k (and b with the removal rule) of the block's tokens
+// [tokens, 2 or 3 times dim], the decays per channel
 // [tokens, dim] if there are such, the values of the workgroup's columns [tokens, 8] as they lie in memory (float32, or
 // bfloat16 in the low half of a word), beta [tokens] and the head's decay [tokens].
-__host__ __device__ __forceinline__ int wave_buffer_floats(int tokens, int dim, int per_channel) {
-  return tokens * (2 * dim + (per_channel ? dim : 0) + WAVE_COLS + 2);
+__host__ __device__ __forceinline__ int wave_buffer_floats(int tokens, int dim, int per_channel, int vectors) {
+  return tokens * (vectors * dim + (per_channel ? dim : 0) + WAVE_COLS + 2);
 }
 
-template <int RW>
+template <int RW, bool REMOVAL>
 __global__ void __launch_bounds__(512) linear_scan_wave_kernel(const ScanArgs a, const int block_tokens) {
   extern __shared__ float4_t stage_pieces[];
   float* stage = reinterpret_cast<float*>(stage_pieces);
@@ -860,12 +1003,13 @@ __global__ void __launch_bounds__(512) linear_scan_wave_kernel(const ScanArgs a,
   const int d0 = lane * RW;
   const int g = h / (heads / a.kv_heads);
   const int per_channel = a.decay_per_channel;
-  const int qk_pieces = dim / 2, decay_pieces = dim / 4;  // 16-byte pieces of a token's q and k, of its decays
-  const int decays_at = block_tokens * 2 * dim;
+  constexpr int VECTORS = REMOVAL ? 3 : 2;
+  const int qk_pieces = VECTORS * dim / 4, decay_pieces = dim / 4;  // 16-byte pieces of a token's vectors, of its decays
+  const int decays_at = block_tokens * VECTORS * dim;
   const int values_at = decays_at + (per_channel ? block_tokens * dim : 0);
   const int betas_at = values_at + block_tokens * WAVE_COLS;
   const int head_decays_at = betas_at + block_tokens;
-  const int buffer_floats = wave_buffer_floats(block_tokens, dim, per_channel);
+  const int buffer_floats = wave_buffer_floats(block_tokens, dim, per_channel, VECTORS);
 
   // Sends for the block of tokens from t0: every wave instruction fills 64 consecutive pieces of LDS, each lane from its own
   // place in memory.  Lanes whose token lies beyond the sequence's end send nothing (nobody reads those rows).
@@ -874,7 +1018,7 @@ __global__ void __launch_bounds__(512) linear_scan_wave_kernel(const ScanArgs a,
     for (int first = wave * 64; first < block_tokens * qk_pieces; first += 512) {
       const int index = first + lane, token = index / qk_pieces, piece = index - token * qk_pieces;
       if (token < block_tokens && t0 + token < hi)
-        send_to_lds_16(a.qk + ((size_t)(t0 + token) * a.kv_heads + g) * 2 * dim + piece * 4, to + first * 4);
+        send_to_lds_16(a.qk + ((size_t)(t0 + token) * a.kv_heads + g) * VECTORS * dim + piece * 4, to + first * 4);
     }
     if (per_channel) {
       for (int first = wave * 64; first < block_tokens * decay_pieces; first += 512) {
@@ -902,23 +1046,39 @@ __global__ void __launch_bounds__(512) linear_scan_wave_kernel(const ScanArgs a,
 #pragma unroll
   for (int i = 0; i < RW; ++i) s[i] = S[(size_t)(d0 + i) * vdim];
 
-  float q[RW], k[RW], dec[RW], qn[RW], kn[RW], decn[RW];  // two sets of operands, used in turn
+  float q[RW], k[RW], dec[RW], rem[RW], qn[RW], kn[RW], decn[RW], remn[RW];  // two sets of operands, used in turn
   float val, bet, valn = 0.f, betn = 1.f;
   const int has_beta = a.beta != nullptr, v_bf16 = a.v_bf16;
-  auto fetch = [&](const float* from, int j, float (&fq)[RW], float (&fk)[RW], float (&fd)[RW], float& fv, float& fb) {
+  auto fetch = [&](const float* from, int j, float (&fq)[RW], float (&fk)[RW], float (&fd)[RW], float (&fr)[RW], float& fv, float& fb) {
     const float one = per_channel ? 1.f : from[head_decays_at + j];
 #pragma unroll
     for (int i = 0; i < RW; ++i) {
-      fq[i] = from[j * 2 * dim + d0 + i];
-      fk[i] = from[j * 2 * dim + dim + d0 + i];
+      fq[i] = from[j * VECTORS * dim + d0 + i];
+      fk[i] = from[j * VECTORS * dim + dim + d0 + i];
+      if constexpr (REMOVAL) fr[i] = from[j * VECTORS * dim + 2 * dim + d0 + i];
       fd[i] = per_channel ? from[decays_at + j * dim + d0 + i] : one;
     }
     const float raw = from[values_at + j * WAVE_COLS + wave];
     fv = v_bf16 ? __uint_as_float(__float_as_uint(raw) << 16) : raw;
     fb = has_beta ? from[betas_at + j] : 1.f;
   };
-  auto work = [&](const float (&wq)[RW], const float (&wk)[RW], const float (&wd)[RW], float wv, float wb) -> float {
+  auto work = [&](const float (&wq)[RW], const float (&wk)[RW], const float (&wd)[RW], const float (&wr)[RW], float wv, float wb) -> float {
     float dot = 0.f;
+    if constexpr (REMOVAL) {
+#pragma unroll
+      for (int i = 0; i < RW; ++i) dot += s[i] * wk[i];
+      float kept[RW];  // (what does not wait for the sum over the wave)
+#pragma unroll
+      for (int i = 0; i < RW; ++i) kept[i] = s[i] * wd[i] + wk[i] * (wb * wv);
+      dot = wave_total(dot);
+      float part = 0.f;
+#pragma unroll
+      for (int i = 0; i < RW; ++i) {
+        s[i] = kept[i] - wr[i] * dot;
+        part += s[i] * wq[i];
+      }
+      return wave_total(part);
+    }
 #pragma unroll
     for (int i = 0; i < RW; ++i) {
       s[i] *= wd[i];
@@ -954,17 +1114,17 @@ __global__ void __launch_bounds__(512) linear_scan_wave_kernel(const ScanArgs a,
     const int count = hi - t0 < block_tokens ? hi - t0 : block_tokens;
     const float* from = stage + buffer * buffer_floats;
     float* outs = stage + outs_at + buffer * block_tokens * WAVE_COLS + wave;
-    fetch(from, 0, q, k, dec, val, bet);
+    fetch(from, 0, q, k, dec, rem, val, bet);
     int j = 0;
     for (; j + 1 < count; j += 2) {  // (a token's operands leave LDS while the token before it is worked)
-      fetch(from, j + 1, qn, kn, decn, valn, betn);
-      const float o0 = work(q, k, dec, val, bet);
-      if (j + 2 < count) fetch(from, j + 2, q, k, dec, val, bet);
-      const float o1 = work(qn, kn, decn, valn, betn);
+      fetch(from, j + 1, qn, kn, decn, remn, valn, betn);
+      const float o0 = work(q, k, dec, rem, val, bet);
+      if (j + 2 < count) fetch(from, j + 2, q, k, dec, rem, val, bet);
+      const float o1 = work(qn, kn, decn, remn, valn, betn);
       if (lane == 0) { outs[j * WAVE_COLS] = o0; outs[(j + 1) * WAVE_COLS] = o1; }
     }
     if (j < count) {
-      const float o = work(q, k, dec, val, bet);
+      const float o = work(q, k, dec, rem, val, bet);
       if (lane == 0) outs[j * WAVE_COLS] = o;
     }
     wait_for_loads<0>();  // this wave's pieces of the next block have landed (and its stores of read-outs, long since)
@@ -982,73 +1142,83 @@ __global__ void __launch_bounds__(512) linear_scan_wave_kernel(const ScanArgs a,
 }
 
 // Tokens per staging block: as many as the lanes can carry and two buffers of LDS can hold, 16 at most; 0: no staging.
-static int scan_block_tokens(int dim, int lanes, int per_channel) {
+static int scan_block_tokens(int dim, int lanes, int per_channel, int vectors) {
   if (dim % 4 != 0) return 0;
   const int cols = 256 / lanes;
-  const int pieces = dim / 2 + (per_channel ? dim / 4 : 0);
-  const int stride = 2 * dim + (per_channel ? dim : 0) + cols + 4;
+  const int pieces = vectors * dim / 4 + (per_channel ? dim / 4 : 0);
+  const int stride = vectors * dim + (per_channel ? dim : 0) + cols + 4;
   int tokens = 16;
   while (tokens >= 2 && (tokens * pieces > 256 * STAGE_PIECES || tokens * cols > 256 * STAGE_VALUES || 2 * tokens * stride * (int)sizeof(float) > 60 * 1024))
     tokens >>= 1;
   return tokens >= 2 ? tokens : 0;
 }
 
-extern "C" int velox_linear_scan(const float* qk, const void* v, int v_dtype, int v_ld, int v_at, const float* decay, int decay_per_channel, const float* beta,
-                                 float* state, const int* slots, const int* cu_q, float* out, int num_seqs, int max_q_len, int heads, int kv_heads, int dim,
-                                 int vdim, int delta, hipStream_t stream) {
-  if (num_seqs <= 0) return 0;
-  const int lanes = velox_linear_scan_lanes(dim);
-  if (lanes > 64 || heads > 65535 || num_seqs > 65535 || kv_heads < 1 || heads % kv_heads != 0 || (delta && !beta)) return (int)hipErrorInvalidValue;
-  ScanArgs a{qk, v, v_dtype == VELOX_BF16, v_ld, v_at, decay, decay_per_channel, beta, state, slots, cu_q, out, heads, kv_heads, dim, vdim, delta};
+template <bool REMOVAL>
+static void linear_scan_launch(const ScanArgs& a, int lanes, int num_seqs, int max_q_len, hipStream_t stream) {
+  const int dim = a.dim, vectors = REMOVAL ? 3 : 2;
   const int cols = 256 / lanes;
-  const dim3 grid((vdim + cols - 1) / cols, heads, num_seqs);
+  const dim3 grid((a.vdim + cols - 1) / cols, a.heads, num_seqs);
   if (max_q_len > 2 && (dim == 64 || dim == 128 || dim == 256 || dim == 512)) {
     int tokens = 16;
-    while (2 * wave_buffer_floats(tokens, dim, decay_per_channel) * (int)sizeof(float) > 60 * 1024) tokens >>= 1;  // (dim = 512 with a decay per channel: 4)
-    const size_t lds = (size_t)2 * (wave_buffer_floats(tokens, dim, decay_per_channel) + tokens * WAVE_COLS) * sizeof(float);  // (+ two blocks of read-outs)
-    const dim3 wave_grid((vdim + WAVE_COLS - 1) / WAVE_COLS, heads, num_seqs);
+    while (2 * wave_buffer_floats(tokens, dim, a.decay_per_channel, vectors) * (int)sizeof(float) > 60 * 1024) tokens >>= 1;  // (dim = 512 with a decay per channel: 4, or 2)
+    const size_t lds = (size_t)2 * (wave_buffer_floats(tokens, dim, a.decay_per_channel, vectors) + tokens * WAVE_COLS) * sizeof(float);  // (+ two blocks of read-outs)
+    const dim3 wave_grid((a.vdim + WAVE_COLS - 1) / WAVE_COLS, a.heads, num_seqs);
     switch (dim) {
-      case 64: linear_scan_wave_kernel<1><<<wave_grid, 512, lds, stream>>>(a, tokens); break;
-      case 128: linear_scan_wave_kernel<2><<<wave_grid, 512, lds, stream>>>(a, tokens); break;
-      case 256: linear_scan_wave_kernel<4><<<wave_grid, 512, lds, stream>>>(a, tokens); break;
-      default: linear_scan_wave_kernel<8><<<wave_grid, 512, lds, stream>>>(a, tokens); break;
+      case 64: linear_scan_wave_kernel<1, REMOVAL><<<wave_grid, 512, lds, stream>>>(a, tokens); break;
+      case 128: linear_scan_wave_kernel<2, REMOVAL><<<wave_grid, 512, lds, stream>>>(a, tokens); break;
+      case 256: linear_scan_wave_kernel<4, REMOVAL><<<wave_grid, 512, lds, stream>>>(a, tokens); break;
+      default: linear_scan_wave_kernel<8, REMOVAL><<<wave_grid, 512, lds, stream>>>(a, tokens); break;
     }
-    VELOX_RETURN_LAUNCH_STATUS();
+    return;
   }
-  const int block_tokens = max_q_len > 2 ? scan_block_tokens(dim, lanes, decay_per_channel) : 0;
+  const int block_tokens = max_q_len > 2 ? scan_block_tokens(dim, lanes, a.decay_per_channel, vectors) : 0;
   if (block_tokens > 0) {
-    const int stride = 2 * dim + (decay_per_channel ? dim : 0) + cols + 4;
+    const int stride = vectors * dim + (a.decay_per_channel ? dim : 0) + cols + 4;
     const size_t lds = (size_t)2 * block_tokens * stride * sizeof(float);
     switch (lanes) {
-      case 1: linear_scan_staged_kernel<1><<<grid, 256, lds, stream>>>(a, block_tokens); break;
-      case 2: linear_scan_staged_kernel<2><<<grid, 256, lds, stream>>>(a, block_tokens); break;
-      case 4: linear_scan_staged_kernel<4><<<grid, 256, lds, stream>>>(a, block_tokens); break;
-      case 8: linear_scan_staged_kernel<8><<<grid, 256, lds, stream>>>(a, block_tokens); break;
-      case 16: linear_scan_staged_kernel<16><<<grid, 256, lds, stream>>>(a, block_tokens); break;
-      case 32: linear_scan_staged_kernel<32><<<grid, 256, lds, stream>>>(a, block_tokens); break;
-      default: linear_scan_staged_kernel<64><<<grid, 256, lds, stream>>>(a, block_tokens); break;
+      case 1: linear_scan_staged_kernel<1, REMOVAL><<<grid, 256, lds, stream>>>(a, block_tokens); break;
+      case 2: linear_scan_staged_kernel<2, REMOVAL><<<grid, 256, lds, stream>>>(a, block_tokens); break;
+      case 4: linear_scan_staged_kernel<4, REMOVAL><<<grid, 256, lds, stream>>>(a, block_tokens); break;
+      case 8: linear_scan_staged_kernel<8, REMOVAL><<<grid, 256, lds, stream>>>(a, block_tokens); break;
+      case 16: linear_scan_staged_kernel<16, REMOVAL><<<grid, 256, lds, stream>>>(a, block_tokens); break;
+      case 32: linear_scan_staged_kernel<32, REMOVAL><<<grid, 256, lds, stream>>>(a, block_tokens); break;
+      default: linear_scan_staged_kernel<64, REMOVAL><<<grid, 256, lds, stream>>>(a, block_tokens); break;
     }
-    VELOX_RETURN_LAUNCH_STATUS();
+    return;
   }
   switch (lanes) {
-    case 1: linear_scan_kernel<1><<<grid, 256, 0, stream>>>(a); break;
-    case 2: linear_scan_kernel<2><<<grid, 256, 0, stream>>>(a); break;
-    case 4: linear_scan_kernel<4><<<grid, 256, 0, stream>>>(a); break;
-    case 8: linear_scan_kernel<8><<<grid, 256, 0, stream>>>(a); break;
-    case 16: linear_scan_kernel<16><<<grid, 256, 0, stream>>>(a); break;
-    case 32: linear_scan_kernel<32><<<grid, 256, 0, stream>>>(a); break;
-    default: linear_scan_kernel<64><<<grid, 256, 0, stream>>>(a); break;
+    case 1: linear_scan_kernel<1, REMOVAL><<<grid, 256, 0, stream>>>(a); break;
+    case 2: linear_scan_kernel<2, REMOVAL><<<grid, 256, 0, stream>>>(a); break;
+    case 4: linear_scan_kernel<4, REMOVAL><<<grid, 256, 0, stream>>>(a); break;
+    case 8: linear_scan_kernel<8, REMOVAL><<<grid, 256, 0, stream>>>(a); break;
+    case 16: linear_scan_kernel<16, REMOVAL><<<grid, 256, 0, stream>>>(a); break;
+    case 32: linear_scan_kernel<32, REMOVAL><<<grid, 256, 0, stream>>>(a); break;
+    default: linear_scan_kernel<64, REMOVAL><<<grid, 256, 0, stream>>>(a); break;
   }
+}
+
+// rule 0: additive, 1: delta, 2: removal (three vectors per token, a decay per channel; beta holds the keys' lengths)
+extern "C" int velox_linear_scan(const float* qk, const void* v, int v_dtype, int v_ld, int v_at, const float* decay, int decay_per_channel, const float* beta,
+                                 float* state, const int* slots, const int* cu_q, float* out, int num_seqs, int max_q_len, int heads, int kv_heads, int dim,
+                                 int vdim, int rule, hipStream_t stream) {
+  if (num_seqs <= 0) return 0;
+  const int lanes = velox_linear_scan_lanes(dim);
+  if (lanes > 64 || heads > 65535 || num_seqs > 65535 || kv_heads < 1 || heads % kv_heads != 0 || rule < 0 || rule > 2 || (rule != 0 && !beta))
+    return (int)hipErrorInvalidValue;
+  ScanArgs a{qk, v, v_dtype == VELOX_BF16, v_ld, v_at, decay, decay_per_channel, beta, state, slots, cu_q, out, heads, kv_heads, dim, vdim, rule == 1};
+  if (rule == 2) linear_scan_launch<true>(a, lanes, num_seqs, max_q_len, stream);
+  else linear_scan_launch<false>(a, lanes, num_seqs, max_q_len, stream);
   VELOX_RETURN_LAUNCH_STATUS();
 }
 
 // ---------------------------------------------------------------------------------------------
 // gated_head_norm: one wave per (token, head): out = o / sqrt(mean(o^2) + eps) * w * gate, gate = silu(z) (kind 0) or
-// sigmoid(z) (kind 1), z a token's row of gate_src at gate_at.
+// sigmoid(z) (kind 1), z a token's row of gate_src at gate_at; w has vdim entries that all heads share, or heads * vdim
+// (weight_stride = vdim).
 // ---------------------------------------------------------------------------------------------
 __global__ void __launch_bounds__(256) gated_head_norm_kernel(const float* __restrict__ read, const float* __restrict__ weight, float eps,
                                                               const void* __restrict__ gate_src, int gate_bf16, int gate_ld, int gate_at, int kind,
-                                                              void* __restrict__ out, int out_bf16, int heads, int vdim, size_t pairs) {
+                                                              void* __restrict__ out, int out_bf16, int heads, int vdim, size_t pairs, int weight_stride) {
   const size_t pair = (size_t)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (pair >= pairs) return;
   const int lane = threadIdx.x & 63;
@@ -1062,15 +1232,15 @@ __global__ void __launch_bounds__(256) gated_head_norm_kernel(const float* __res
   for (int c = lane; c < vdim; c += 64) {
     const float z = load_as_f32(gate_src, gate_bf16, t * gate_ld + gate_at + (size_t)h * vdim + c);
     const float gate = kind == 0 ? z * sigmoid_f32(z) : sigmoid_f32(z);
-    store_from_f32(out, out_bf16, pair * vdim + c, o[c] * inv * weight[c] * gate);
+    store_from_f32(out, out_bf16, pair * vdim + c, o[c] * inv * weight[(size_t)h * weight_stride + c] * gate);
   }
 }
 
 extern "C" int velox_gated_head_norm(const float* read, const float* weight, float eps, const void* gate_src, int gate_dtype, int gate_ld, int gate_at,
-                                     int kind, void* out, int out_dtype, int tokens, int heads, int vdim, hipStream_t stream) {
+                                     int kind, void* out, int out_dtype, int tokens, int heads, int vdim, int weight_per_head, hipStream_t stream) {
   if (tokens <= 0) return 0;
   const size_t pairs = (size_t)tokens * heads;
   gated_head_norm_kernel<<<(unsigned)((pairs + 3) / 4), 256, 0, stream>>>(read, weight, eps, gate_src, gate_dtype == VELOX_BF16, gate_ld, gate_at, kind, out,
-                                                                         out_dtype == VELOX_BF16, heads, vdim, pairs);
+                                                                         out_dtype == VELOX_BF16, heads, vdim, pairs, weight_per_head ? vdim : 0);
   VELOX_RETURN_LAUNCH_STATUS();
 }

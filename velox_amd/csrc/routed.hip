@@ -524,12 +524,14 @@ __global__ void __launch_bounds__(256) routed_combine_kernel(const float* __rest
 }
 
 // The same sum, handed straight to a norm on the experts' output: residual[t, :] += mult * v * rsqrt(mean(v^2) + eps) * w, with v the
-// sum above in float32 (never rounded to T), and `copy` (nullable) the updated residual in T.  One workgroup per token holds
-// the row in registers: hidden <= 16 * blockDim.x.
+// sum above in float32 (never rounded to T), and `copy` (nullable) the updated residual in T; with `next_weight` `copy` is instead
+// what the norm that reads the residual next makes of it, r * rsqrt(mean(r^2) + next_eps) * next_weight.  One workgroup per
+// token holds the row in registers: hidden <= 16 * blockDim.x.
 template <typename T>
 __global__ void routed_combine_norm_kernel(const float* __restrict__ y, const int* __restrict__ place, const T* __restrict__ shared, int top, int hidden,
                                            const T* __restrict__ x, const float* __restrict__ pair_weight, int scale_rows, float* __restrict__ residual,
-                                           const float* __restrict__ norm_weight, float eps, float mult, T* __restrict__ copy) {
+                                           const float* __restrict__ norm_weight, float eps, float mult, T* __restrict__ copy,
+                                           const float* __restrict__ next_weight, float next_eps) {
   __shared__ int rows[64];
   __shared__ float scratch[16];
   const int t = blockIdx.x;
@@ -558,14 +560,24 @@ __global__ void routed_combine_norm_kernel(const float* __restrict__ y, const in
   }
   const float total = block_sum(sumsq, scratch);
   const float inv = 1.f / sqrtf(total / (float)hidden + eps);
+  sumsq = 0.f;
 #pragma unroll
   for (int c = 0; c < 16; ++c) {
     const int i = threadIdx.x + c * blockDim.x;
     if (i < hidden) {
       const float r = residual[(size_t)t * hidden + i] + mult * (held[c] * inv * norm_weight[i]);
       residual[(size_t)t * hidden + i] = r;
-      if (copy) copy[(size_t)t * hidden + i] = from_f32<T>(r);
+      if (copy && !next_weight) copy[(size_t)t * hidden + i] = from_f32<T>(r);
+      held[c] = r;
+      sumsq += r * r;
     }
+  }
+  if (!next_weight) return;
+  const float next_inv = 1.f / sqrtf(block_sum(sumsq, scratch) / (float)hidden + next_eps);
+#pragma unroll
+  for (int c = 0; c < 16; ++c) {
+    const int i = threadIdx.x + c * blockDim.x;
+    if (i < hidden) copy[(size_t)t * hidden + i] = from_f32<T>(held[c] * next_inv * next_weight[i]);
   }
 }
 
@@ -573,18 +585,19 @@ __global__ void routed_combine_norm_kernel(const float* __restrict__ y, const in
 // (hidden > 16,384): the caller then runs the two kernels one after the other.
 extern "C" int velox_routed_combine_norm(const float* y, const int* plan, const void* shared, int tokens, int top, int experts, int hidden, int dtype,
                                          const void* x, const float* pair_weight, int scale_rows, float* residual, const float* norm_weight, float eps,
-                                         float mult, void* copy, hipStream_t stream) {
+                                         float mult, void* copy, const float* next_weight, float next_eps, hipStream_t stream) {
   if (tokens <= 0) return 0;
+  if (next_weight && !copy) return (int)hipErrorInvalidValue;
   if (hidden > 16 * 1024) return -1;
   const int* place = plan + 1 + (experts + 1) + (size_t)tokens * top;
   int threads = tokens <= 64 ? 512 : 256;  // (few rows: more threads each with less to do)
   while (16 * threads < hidden) threads *= 2;
   if (dtype == VELOX_BF16)
     routed_combine_norm_kernel<bf16_t><<<tokens, threads, 0, stream>>>(y, place, (const bf16_t*)shared, top, hidden, (const bf16_t*)x, pair_weight, scale_rows,
-                                                                       residual, norm_weight, eps, mult, (bf16_t*)copy);
+                                                                       residual, norm_weight, eps, mult, (bf16_t*)copy, next_weight, next_eps);
   else
     routed_combine_norm_kernel<float><<<tokens, threads, 0, stream>>>(y, place, (const float*)shared, top, hidden, (const float*)x, pair_weight, scale_rows,
-                                                                      residual, norm_weight, eps, mult, (float*)copy);
+                                                                      residual, norm_weight, eps, mult, (float*)copy, next_weight, next_eps);
   VELOX_RETURN_LAUNCH_STATUS();
 }
 

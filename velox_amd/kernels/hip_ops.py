@@ -20,7 +20,7 @@ from typing import Tuple, Dict, Optional
 
 import torch
 
-from ..parts.base import DeferredNorm, ResidualCopy, ResidualSink, SumOf
+from ..parts.base import DeferredNorm, ReadyInput, ResidualCopy, ResidualSink, SumOf
 from . import build
 
 logger = logging.getLogger(__name__)
@@ -155,7 +155,7 @@ class HipOps:
         c.velox_grouped_down.argtypes = [_P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P]
         c.velox_routed_combine.argtypes = [_P, _P, _P, _P, _I, _I, _I, _I, _I, _P, _P, _I, _P]
         c.velox_routed_products_bf16.argtypes = [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _F, _F, _I, _P]
-        c.velox_routed_combine_norm.argtypes = [_P, _P, _P, _I, _I, _I, _I, _I, _P, _P, _I, _P, _P, _F, _F, _P, _P]
+        c.velox_routed_combine_norm.argtypes = [_P, _P, _P, _I, _I, _I, _I, _I, _P, _P, _I, _P, _P, _F, _F, _P, _P, _F, _P]
         c.velox_routed_combine_norm.restype = _I
         c.velox_add_sinusoid.argtypes = [_P, _P, _P, _I, _I, _P]
         c.velox_add_cast.argtypes = [_P, _P, _I, _P, ctypes.c_longlong, _P]
@@ -165,11 +165,19 @@ class HipOps:
         c.velox_embed_copies.argtypes = [_P, _P, _I, _P, _I, _I, _I, _F, _I, _P]
         c.velox_gated_act_mul.argtypes = [_P, _P, _I, _I, _I, _I, _P]
         c.velox_short_conv.argtypes = [_P, _I, _I, _P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _I, _P]
-        c.velox_rotate_pad_write.argtypes = [_P, _I, _P, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I, _P]
+        c.velox_rotate_pad_write.argtypes = [_P, _I, _P, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _P]
         c.velox_recurrence_prepare.argtypes = [_P, _I, _I, _I, _I, _I, _I, _I, _F, _P, _I, _I, _I, _I, _I, _P, _P, _F, _P, _I, _I, _I, _P, _P, _P, _I, _P]
         c.velox_linear_scan.argtypes = [_P, _P, _I, _I, _I, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P]
         c.velox_linear_scan_lanes.argtypes = [_I]
-        c.velox_gated_head_norm.argtypes = [_P, _P, _F, _P, _I, _I, _I, _I, _P, _I, _I, _I, _I, _P]
+        c.velox_gated_head_norm.argtypes = [_P, _P, _F, _P, _I, _I, _I, _I, _P, _I, _I, _I, _I, _I, _P]
+        c.velox_removal_prepare.argtypes = [_P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _P, _P, _P, _F, _P, _P, _P, _I, _P]
+        c.velox_gated_scan.argtypes = [_P, _I, _I, _P, _P, _F, _P, _P, _P, _P, _P, _I, _I, _P]
+        c.velox_gated_scan_scratch_elems.argtypes = [_I, _I, _I]
+        c.velox_gated_scan_scratch_elems.restype = ctypes.c_longlong
+        c.velox_norm_add_norm.argtypes = [_P, _P, _I, _P, _F, _P, _F, _P, _P, _I, _I, _I, _I, ctypes.c_longlong, _P]
+        c.velox_poly_norm.argtypes = [_P, _P, _P, _I, _I, _F, _I, _P]
+        for fn in (c.velox_removal_prepare, c.velox_gated_scan, c.velox_norm_add_norm, c.velox_poly_norm):
+            fn.restype = _I
         c.velox_embed_bigram.argtypes = [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _P, _P, _P, _P, _P]
         c.velox_add_dynamic_tanh.argtypes = [_P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, ctypes.c_longlong, _P, _I, _P]
         c.velox_scale.argtypes = [_P, ctypes.c_longlong, _F, _P]
@@ -543,6 +551,45 @@ class HipOps:
         self._launched(self._core.velox_norm_add(_ptr(residual), _ptr(delta), _code(delta.dtype), _ptr(weight), _ptr(out), tokens, hidden, float(eps), float(mult),
                                                  partials, partial_stride, self._stream()), "norm_add")
         return residual if out is None else out
+
+    def norm_add_norm(self, residual: torch.Tensor, delta: torch.Tensor, delta_weight: torch.Tensor, delta_eps: float, weight: torch.Tensor, eps: float,
+                      out_dtype: torch.dtype, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """``residual += delta * rsqrt(mean(delta^2) + delta_eps) * delta_weight`` in place, then ``residual * rsqrt(mean(residual^2) +
+        eps) * weight`` in ``out_dtype``; float32 throughout.  ``delta`` is [T, H] or float32 partial sums [S, T, H], added first to
+        last.  ``rows``: nothing is changed and only those rows are worked."""
+        self._check("residual", residual, torch.float32)
+        if residual.dim() != 2:
+            raise KernelError("norm_add_norm: residual must be [T, H]")
+        tokens, hidden = residual.shape
+        if hidden > 16352:
+            raise KernelError(f"norm_add_norm: rows of {hidden} are beyond the kernel (16,352 at most)")
+        self._check("delta_weight", delta_weight, torch.float32, (hidden,))
+        self._check("weight", weight, torch.float32, (hidden,))
+        partials, partial_stride = 1, 0
+        if delta.dim() == 3:
+            partials, partial_stride = delta.shape[0], tokens * hidden
+            self._check("delta", delta, torch.float32, (partials, tokens, hidden))
+        else:
+            self._check("delta", delta, None, (tokens, hidden))
+        count = tokens
+        if rows is not None:
+            self._check("rows", rows, torch.int32)
+            count = rows.shape[0]
+        out = torch.empty((count, hidden), dtype=out_dtype, device=self.device)
+        self._launched(self._core.velox_norm_add_norm(_ptr(residual), _ptr(delta), _code(delta.dtype), _ptr(delta_weight), float(delta_eps), _ptr(weight), float(eps),
+                                                      _ptr(rows), _ptr(out), _code(out_dtype), count, hidden, partials, partial_stride, self._stream()), "norm_add_norm")
+        return out
+
+    def poly_norm(self, x: torch.Tensor, coefficients: torch.Tensor, eps: float) -> torch.Tensor:
+        """``a N(x) + b N(x^2) + c N(x^3) + e`` per row, ``N(y) = y * rsqrt(mean(y^2) + eps)``; ``coefficients`` = (a, b, c, e), float32 on the
+        device; float32 arithmetic with one rounding."""
+        self._check("x", x)
+        if x.dim() != 2:
+            raise KernelError("poly_norm: rows are [T, F]")
+        self._check("coefficients", coefficients, torch.float32, (4,))
+        out = torch.empty_like(x)
+        self._launched(self._core.velox_poly_norm(_ptr(x), _ptr(out), _ptr(coefficients), x.shape[0], x.shape[1], float(eps), _code(x.dtype), self._stream()), "poly_norm")
+        return out
 
     def qk_norm_write(self, qkv, num_heads, num_kv_heads, dim, vdim, cached_dim, q_norm, k_norm, whole, eps, q_temp, positions, first_values, mix_weight,
                       slot_mapping, k_cache, v_cache, block_size, write_kv=True) -> torch.Tensor:
@@ -969,13 +1016,17 @@ class HipOps:
         return out
 
     def rotate_pad_write(self, qkv, num_heads, num_kv_heads, dim, vdim, cached_dim, positions, cos, sin, slot_mapping, k_cache, v_cache, block_size, write_kv=True,
-                         interleaved=False):
+                         interleaved=False, post_norm_eps: float = 0.0, values_are_keys: bool = False):
         """Rotates the first ``2 * cos.shape[1]`` channels of every q and k head of ``qkv`` [T, heads * dim + kv_heads * (dim + vdim)]
         (channel i with i + half, or 2i with 2i + 1 when ``interleaved``), writes k and v into the pages at ``cached_dim`` channels a head (zeros in the padding)
-        and returns q as [T, heads * cached_dim]."""
+        and returns q as [T, heads * cached_dim].  ``post_norm_eps`` > 0: every q and k head is divided by its root mean square
+        behind the rotation.  ``values_are_keys``: the rows hold no values ([T, (heads + kv_heads) * dim]); a head's values are its
+        keys as they stand in the row."""
         self._check("qkv", qkv)
         tokens = qkv.shape[0]
-        width = num_heads * dim + num_kv_heads * (dim + vdim)
+        if values_are_keys and vdim != dim:
+            raise KernelError(f"rotate_pad_write: values that are the keys have their size, not {vdim} beside {dim}")
+        width = num_heads * dim + num_kv_heads * (dim + (0 if values_are_keys else vdim))
         if qkv.dim() != 2 or qkv.shape[1] != width:
             raise KernelError(f"rotate_pad_write: qkv must be [T, {width}], got {tuple(qkv.shape)}")
         if dim > cached_dim or vdim > cached_dim:
@@ -998,7 +1049,8 @@ class HipOps:
         q = torch.empty((tokens, num_heads * cached_dim), dtype=qkv.dtype, device=self.device)
         status = self._core.velox_rotate_pad_write(_ptr(qkv), width, _ptr(q), _ptr(positions), _ptr(cos), _ptr(sin), half, _ptr(slot_mapping) if write_kv else _P(0),
                                                    _ptr(k_cache) if write_kv else _P(0), _ptr(v_cache) if write_kv else _P(0), tokens, num_heads, num_kv_heads,
-                                                   dim, vdim, cached_dim, int(block_size), int(bool(write_kv)), _code(qkv.dtype), int(bool(interleaved)), self._stream())
+                                                   dim, vdim, cached_dim, int(block_size), int(bool(write_kv)), _code(qkv.dtype), int(bool(interleaved)), float(post_norm_eps),
+                                                   int(bool(values_are_keys)), self._stream())
         self._launched(status, "rotate_pad_write")
         return q
 
@@ -1032,17 +1084,70 @@ class HipOps:
         self._launched(status, "recurrence_prepare")
         return qk, decay, beta
 
+    def removal_prepare(self, main, r_at, k_at, a_at, low_at, rank, heads, dim, a_bias, w2, w0, decay_scale):
+        """What the generalized delta rule reads of a row of ``main`` (read vectors, keys and removal logits of ``heads * dim``
+        columns each at ``r_at``, ``k_at``, ``a_at``; the decay map's inner row of ``rank`` columns at ``low_at``), all float32:
+        ``vectors`` [T, heads, 3, dim] = r, u, sigmoid(a + a_bias) * u with the unit key u = k / n; ``decay`` [T, heads * dim] =
+        ``exp(-decay_scale sigmoid(w0 + w2 tanh(inner)))``; ``lengths`` [T, heads] = n = sqrt(sum(k^2) + 1e-6)."""
+        self._check("main", main)
+        size = heads * dim
+        if main.dim() != 2 or max(r_at, k_at, a_at) + size > main.shape[1] or low_at + rank > main.shape[1] or min(r_at, k_at, a_at, low_at) < 0:
+            raise KernelError("removal_prepare: the columns do not lie within the rows")
+        if not 1 <= rank <= 8192:
+            raise KernelError(f"removal_prepare: an inner size of {rank} is beyond the kernel (8,192 at most)")
+        tokens = main.shape[0]
+        self._check("a_bias", a_bias, torch.float32, (size,))
+        self._check("w0", w0, torch.float32, (size,))
+        self._check("w2", w2, main.dtype, (size, rank))
+        vectors = torch.empty((tokens, heads, 3, dim), dtype=torch.float32, device=self.device)
+        decay = torch.empty((tokens, size), dtype=torch.float32, device=self.device)
+        lengths = torch.empty((tokens, heads), dtype=torch.float32, device=self.device)
+        self._launched(self._core.velox_removal_prepare(_ptr(main), _code(main.dtype), main.shape[1], int(r_at), int(k_at), int(a_at), int(low_at), int(rank), int(heads),
+                                                        int(dim), _ptr(a_bias), _ptr(w2), _ptr(w0), float(decay_scale), _ptr(vectors), _ptr(decay), _ptr(lengths),
+                                                        tokens, self._stream()), "removal_prepare")
+        return vectors, decay, lengths
+
+    def gated_scan(self, projected, width, gate_bias, input_bias, shift, state, slots, cu_q, max_q_len):
+        """``projected`` [T, 3 * width] = z, u, g of every token; per channel and sequence, from ``state[slot]`` ([slots, width] float32, written
+        back): ``S <- (1 - z) S + z c`` with ``z = sigmoid(z + gate_bias)``, ``u += input_bias`` and ``c = u + shift`` (u >= 0) or ``sigmoid(u)``.
+        Returns ``S * silu(g)``, [T, width] in the rows' dtype."""
+        self._check("projected", projected)
+        tokens = projected.shape[0]
+        if projected.dim() != 2 or projected.shape[1] != 3 * width:
+            raise KernelError(f"gated_scan: rows of {3 * width} columns expected, got {tuple(projected.shape)}")
+        self._check("gate_bias", gate_bias, torch.float32, (width,))
+        self._check("input_bias", input_bias, torch.float32, (width,))
+        self._check("state", state, torch.float32)
+        if state.dim() != 2 or state.shape[1] != width:
+            raise KernelError(f"gated_scan: the state must be [slots, {width}], got {tuple(state.shape)}")
+        self._check("slots", slots, torch.int32)
+        self._check("cu_q", cu_q, torch.int32, (slots.shape[0] + 1,))
+        if not 1 <= max_q_len <= tokens:
+            raise KernelError(f"gated_scan: max_q_len={max_q_len} outside [1, {tokens}]")
+        out = torch.empty((tokens, width), dtype=projected.dtype, device=self.device)
+        elems = int(self._core.velox_gated_scan_scratch_elems(slots.shape[0], int(max_q_len), int(width)))
+        scratch = torch.empty(elems, dtype=torch.float32, device=self.device) if elems else None
+        self._launched(self._core.velox_gated_scan(_ptr(projected), _code(projected.dtype), int(width), _ptr(gate_bias), _ptr(input_bias), float(shift), _ptr(state),
+                                                   _ptr(slots), _ptr(cu_q), _ptr(out), _ptr(scratch), slots.shape[0], int(max_q_len), self._stream()), "gated_scan")
+        return out
+
     def linear_scan_supports(self, dim: int, vdim: int) -> None:
         """Raises if the scan kernel cannot hold a column of a ``dim x vdim`` state in one wave."""
         if self._core.velox_linear_scan_lanes(int(dim)) > 64:
             raise KernelError(f"linear_scan: key heads of {dim} channels are beyond the kernel (512 at most)")
 
-    def linear_scan(self, qk, v_source, v_at, decay, beta, state, slots, cu_q, max_q_len, heads, kv_heads, dim, vdim, delta):
+    _SCAN_RULES = {"additive": 0, "delta": 1, "removal": 2}
+
+    def linear_scan(self, qk, v_source, v_at, decay, beta, state, slots, cu_q, max_q_len, heads, kv_heads, dim, vdim, rule):
         """Per sequence and head, token by token from ``state[slot, head]`` ([dim, vdim] float32), which is written back:
-        ``S <- g S`` (rows); ``u = beta (v - S^T k)`` (``delta``) or ``u = v``; ``S <- S + k u^T``; ``o = S^T q``.  ``decay`` is
-        [T, heads] or [T, heads * dim].  Returns float32 [T, heads * vdim]."""
+        ``S <- g S`` (rows); ``u = beta (v - S^T k)`` (rule ``"delta"``) or ``u = v`` (``"additive"``); ``S <- S + k u^T``; ``o = S^T q``.
+        Rule ``"removal"``: ``qk`` holds a third vector ``b`` per head and token, and ``S <- g S - b (k^T S) + k (beta v)^T`` with both
+        terms on the old state.  ``decay`` is [T, heads] or [T, heads * dim].  Returns float32 [T, heads * vdim]."""
+        if rule not in self._SCAN_RULES:
+            raise KernelError(f"linear_scan: rule {rule!r} is not implemented ({', '.join(self._SCAN_RULES)})")
+        delta = rule != "additive"
         tokens = qk.shape[0]
-        self._check("qk", qk, torch.float32, (tokens, kv_heads, 2, dim), align=16)
+        self._check("qk", qk, torch.float32, (tokens, kv_heads, 3 if rule == "removal" else 2, dim), align=16)
         self._check("v_source", v_source)
         if v_source.dim() != 2 or v_source.shape[0] != tokens or v_at + heads * vdim > v_source.shape[1]:
             raise KernelError("linear_scan: the values do not lie within their source")
@@ -1052,7 +1157,7 @@ class HipOps:
         per_channel = tuple(decay.shape) == (tokens, heads * dim)
         if delta:
             if beta is None:
-                raise KernelError("linear_scan: the delta rule needs beta")
+                raise KernelError(f"linear_scan: the {rule} rule needs beta")
             self._check("beta", beta, torch.float32, (tokens, heads))
         self._check("state", state, torch.float32)
         if state.dim() != 4 or tuple(state.shape[1:]) != (heads, dim, vdim):
@@ -1063,23 +1168,26 @@ class HipOps:
         out = torch.empty((tokens, heads * vdim), dtype=torch.float32, device=self.device)
         status = self._core.velox_linear_scan(_ptr(qk), _ptr(v_source), _code(v_source.dtype), v_source.shape[1], int(v_at), _ptr(decay), int(per_channel),
                                               _ptr(beta) if delta else _P(0), _ptr(state), _ptr(slots), _ptr(cu_q), _ptr(out), slots.shape[0], int(max_q_len), int(heads),
-                                              int(kv_heads), int(dim), int(vdim), int(bool(delta)), self._stream())
+                                              int(kv_heads), int(dim), int(vdim), self._SCAN_RULES[rule], self._stream())
         self._launched(status, "linear_scan")
         return out
 
     def gated_head_norm(self, read, weight, eps, gate_source, gate_at, gate_kind, heads, vdim, out_dtype):
         """``read`` float32 [T, heads * vdim]: every head divided by its root mean square (``eps`` inside the root), times
-        ``weight`` [vdim], times ``silu(z)`` or ``sigmoid(z)`` of the gate's columns; [T, heads * vdim] in ``out_dtype``."""
+        ``weight`` ([vdim], shared by the heads, or [heads * vdim]), times ``silu(z)`` or ``sigmoid(z)`` of the gate's columns;
+        [T, heads * vdim] in ``out_dtype``."""
         tokens = read.shape[0]
         self._check("read", read, torch.float32, (tokens, heads * vdim))
-        self._check("weight", weight, torch.float32, (vdim,))
+        self._check("weight", weight, torch.float32, (weight.numel(),))
+        if weight.numel() not in (vdim, heads * vdim):
+            raise KernelError(f"gated_head_norm: the weight has {vdim} or {heads * vdim} entries, got {weight.numel()}")
         self._check("gate_source", gate_source)
         if gate_source.dim() != 2 or gate_source.shape[0] != tokens or gate_at + heads * vdim > gate_source.shape[1] or gate_kind not in ("silu", "sigmoid"):
             raise KernelError("gated_head_norm: the gate's columns do not lie within its source, or its kind is unknown")
         out = torch.empty((tokens, heads * vdim), dtype=out_dtype, device=self.device)
         status = self._core.velox_gated_head_norm(_ptr(read), _ptr(weight), float(eps), _ptr(gate_source), _code(gate_source.dtype), gate_source.shape[1],
                                                   int(gate_at), 0 if gate_kind == "silu" else 1, _ptr(out), _code(out_dtype), tokens, int(heads), int(vdim),
-                                                  self._stream())
+                                                  int(weight.numel() != vdim), self._stream())
         self._launched(status, "gated_head_norm")
         return out
 
@@ -1311,7 +1419,8 @@ class HipOps:
         shift)`` with ``g = min(gate, limit)``, ``u = clamp(up, -limit, limit)``.  ``identity_experts``: choices from
         ``num_experts`` on are experts without tensors whose result is ``weight[t, k] x[t]``; the plan leaves them out and
         the last kernel adds them in their turn.  ``output_norm`` (an ``OutputNormSink``): the last kernel norms the sum in
-        float32 and adds it to the sink's residual; what comes back is then a ``ResidualCopy`` of the updated residual.
+        float32 and adds it to the sink's residual; what comes back is then a ``ResidualCopy`` of the updated residual, or, when
+        the sink names the norm that follows, a ``ReadyInput`` with that norm's result.
         ``ungated`` (``"relu2"``): the units have no gate branch, ``W_down act(W_up x)``; ``gate_up_weight`` is then [E * F, H]."""
         alpha, limit, shift = (float(v) for v in unit)
         if ungated is not None and ungated not in self._ACTIVATION_CODES:
@@ -1369,16 +1478,26 @@ class HipOps:
         if output_norm is not None:
             self._check("residual", output_norm.residual, torch.float32, (tokens, hidden))
             self._check("norm weight", output_norm.weight, torch.float32, (hidden,))
-            copy = torch.empty((tokens, hidden), dtype=out_dtype, device=self.device) if out_dtype != torch.float32 else None
+            following = output_norm.following.deferred_form() if output_norm.following is not None else None
+            copy = torch.empty((tokens, hidden), dtype=out_dtype, device=self.device) if out_dtype != torch.float32 or following is not None else None
+            if following is not None:
+                self._check("next norm weight", following[0], torch.float32, (hidden,))
             status = self._core.velox_routed_combine_norm(_ptr(y), _ptr(plan), _ptr(shared), tokens, top, num_experts, hidden, _code(out_dtype),
                                                           _ptr(identity_input), _ptr(weight), int(bool(scale_rows)), _ptr(output_norm.residual),
-                                                          _ptr(output_norm.weight), float(output_norm.eps), float(output_norm.mult), _ptr(copy), self._stream())
+                                                          _ptr(output_norm.weight), float(output_norm.eps), float(output_norm.mult), _ptr(copy),
+                                                          _ptr(following[0]) if following is not None else _P(0), float(following[1]) if following is not None else 0.0,
+                                                          self._stream())
+            if status == 0 and following is not None:
+                return ReadyInput(copy, output_norm.following)
             if status == 0:
                 return ResidualCopy(output_norm.residual if copy is None else copy)
             if status != -1:
                 self._launched(status, "routed_combine_norm")
             # (a row too long for the fused kernel's registers: the two kernels one after the other)
             out = self._routed_combine(y, plan, shared, tokens, top, num_experts, hidden, out_dtype, identity_input, weight, scale_rows)
+            if following is not None:
+                self.norm_add(output_norm.residual, out, output_norm.weight, output_norm.eps, output_norm.mult, torch.float32)
+                return ReadyInput(self.add_rmsnorm(output_norm.residual, None, following[0], following[1], out_dtype), output_norm.following)
             return ResidualCopy(self.norm_add(output_norm.residual, out, output_norm.weight, output_norm.eps, output_norm.mult, out_dtype))
         out = torch.empty((tokens, hidden), dtype=out_dtype, device=self.device)
         self._launched(self._core.velox_routed_combine(_ptr(y), _ptr(plan), _ptr(shared), _ptr(out), tokens, top, num_experts, hidden, _code(out_dtype),

@@ -264,16 +264,36 @@ class ResidualCopy:
 
 
 @dataclass
+class NormedDelta:
+    """A sub-layer's output whose OWN norm is still to be taken before the residual gets it: ``residual += norm(y)``.
+    Handed on in a delta's place; the norm that reads the residual next takes both norms and the add in one kernel."""
+
+    y: torch.Tensor  # [T, H] or float32 partial sums [S, T, H]
+    norm: "Norm"
+
+
+@dataclass
+class ReadyInput:
+    """What a sub-layer hands on when its last kernel has added its normed output to the residual AND taken the next
+    norm: ``x`` is that norm's result, [T, H] in the run dtype.  It can only go to the norm it was made for."""
+
+    x: torch.Tensor
+    norm: "Norm"
+
+
+@dataclass
 class OutputNormSink:
     """Where a sub-layer whose last kernel can norm its own output may put it: ``residual += mult * output *
     rsqrt(mean(output^2) + eps) * weight``.  A feed-forward that sets ``accepts_output_norm = True`` takes ``output_norm=``
     in ``forward`` and returns either its output as always, or, when it has done the norm and the add itself, a
-    ``ResidualCopy`` of the updated residual."""
+    ``ResidualCopy`` of the updated residual; or, when ``following`` names the norm that reads the residual next (one
+    that has a ``deferred_form``), a ``ReadyInput`` with that norm's result."""
 
     residual: torch.Tensor
     weight: torch.Tensor
     eps: float
     mult: float
+    following: Optional["Norm"] = None
 
 
 class Mixer(Part):
@@ -307,7 +327,8 @@ class Norm(Part):
         """``residual`` [T, H] float32.
 
         ``delta`` is [T, H] or float32 partial sums [S, T, H], which are added first to last, or a ``SumOf`` two such
-        terms, or a ``DeferredNorm`` made for this very norm (then the residual is up to date and the ``DeferredNorm`` itself is what comes back).
+        terms, or a ``DeferredNorm`` made for this very norm (then the residual is up to date and the ``DeferredNorm`` itself is what comes back),
+        or a ``NormedDelta`` (the delta passes a norm of its own first) or a ``ReadyInput`` made for this norm (its tensor comes back).
         With ``rows`` None: ``residual += delta`` in place (delta may be None) and the
         normalised residual comes back in the run dtype, [T, H].  With ``rows`` (int32
         [R]): nothing is changed and ``normalise(residual[rows] + delta[rows])`` comes back.

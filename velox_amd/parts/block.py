@@ -9,6 +9,10 @@ norm's kernel, so each block hands its feed-forward output on to whoever normali
 read the residual stream itself and only their outputs are normed, so nothing is pending between blocks; what is handed
 on is the updated residual in the run dtype (``ResidualCopy``), which the norm's kernel writes beside the float32 sum.
 
+``SandwichBlock`` (not in the reference): ``h = h + norm1b(mixer(norm1(h))); h = h + norm2b(ff(norm2(h)))``, a norm
+before and one after each sub-layer.  The norm behind a sub-layer, the residual sum and the norm before the next
+sub-layer are one kernel: the output travels as a ``NormedDelta``.
+
 ``ParallelBlock`` (not in the reference): ``n = norm(h); h = h + (mixer(n) + ff(n))``, one norm that both
 sub-layers read.  It hands both outputs on as a ``SumOf``, which the next norm's kernel adds up in float32.
 
@@ -21,7 +25,9 @@ from typing import Optional, Tuple
 
 import torch
 
-from .base import Block, FeedForward, Mixer, Norm, OutputNormSink, Part, ResidualCopy, ResidualSink, StreamUpdate, SumOf, register_arrangement
+from .base import (
+    Block, FeedForward, Mixer, Norm, NormedDelta, OutputNormSink, Part, PartSpec, ResidualCopy, ResidualSink, StreamUpdate, SumOf, make_part, register_arrangement,
+)
 
 
 class PreNormBlock(Block):
@@ -141,6 +147,49 @@ class OutputNormBlock(Block):
 
 
 register_arrangement("output_norm", OutputNormBlock)
+
+
+class SandwichBlock(Block):
+    def __init__(self, prefix: str, mixer: Mixer, feed_forward: FeedForward, mixer_norm: Norm, ff_norm: Norm, output_norm: Optional[PartSpec] = None,
+                 output_norm_prefixes: Tuple[str, str] = ("mixer_output_norm.", "feed_forward_output_norm.")) -> None:
+        """``output_norm``: the kind and constants of the two norms behind the sub-layers (a kind with a ``deferred_form``);
+        their tensors stand under the block's prefix and ``output_norm_prefixes``."""
+        super().__init__(prefix)
+        if output_norm is None:
+            raise ValueError("a sandwich block needs output_norm, the kind of the norms behind its sub-layers")
+        self.mixer = mixer
+        self.feed_forward = feed_forward
+        self.mixer_norm = mixer_norm
+        self.ff_norm = ff_norm
+        self.mixer_out_norm, self.ff_out_norm = (make_part("norm", output_norm.kind, prefix=prefix + below, **output_norm.kwargs()) for below in output_norm_prefixes)
+        self.has_feed_forward = type(feed_forward).__name__ != "NoFeedForward"
+
+    def children(self) -> Tuple[Part, ...]:
+        if not self.has_feed_forward:
+            return (self.mixer_norm, self.mixer, self.mixer_out_norm)  # (the norms of the other sub-layer do not exist)
+        return (self.mixer_norm, self.mixer, self.mixer_out_norm, self.ff_norm, self.feed_forward, self.ff_out_norm)
+
+    def input_norm(self) -> Optional[Norm]:
+        return self.mixer_norm
+
+    def forward(self, residual: torch.Tensor, pending, ctx, cache, owns_cache: bool, next_norm: Optional[Norm] = None):
+        normed = self.mixer_norm.forward(residual, pending, ctx)
+        pending = NormedDelta(self.mixer.forward(normed, ctx, cache, owns_cache), self.mixer_out_norm)
+        if not self.has_feed_forward:
+            return pending
+        normed = self.ff_norm.forward(residual, pending, ctx)
+        form = self.ff_out_norm.deferred_form()
+        if form is not None and getattr(self.feed_forward, "accepts_output_norm", False):
+            following = next_norm if next_norm is not None and next_norm.deferred_form() is not None else None
+            out = self.feed_forward.forward(normed, ctx, output_norm=OutputNormSink(residual, form[0], form[1], 1.0, following))
+            if not isinstance(out, torch.Tensor):
+                return out  # (the experts' last kernel has done the rest)
+        else:
+            out = self.feed_forward.forward(normed, ctx)
+        return NormedDelta(out, self.ff_out_norm)
+
+
+register_arrangement("sandwich", SandwichBlock)
 
 
 class HyperConnectionBlock(Block):

@@ -10,7 +10,11 @@ Beside ``parts.attention`` and ``parts.normed_attention`` this mixer has
 * a rotation of the first ``rotary_dim`` channels of each query and key head only (the rest passes), in either layout of
   the position encoding: channel ``i`` with ``i + rotary_dim / 2`` or channel ``2i`` with ``2i + 1``;
 * its own sizes for query/key heads (``dim``) and value heads (``vdim``), a scale from the configuration, a sliding
-  window (``window``: a query at ``i`` sees ``j`` with ``0 <= i - j < window``; pages behind it are given back).
+  window (``window``: a query at ``i`` sees ``j`` with ``0 <= i - j < window``; pages behind it are given back);
+* ``post_norm_eps``: queries and keys are divided by their root mean square per head BEHIND the rotation (no weight);
+* ``values_are_keys``: there is no value product, a key head's values are its keys as the projection left them, before
+  rotation and norm (the cache still holds both: what is written as a key is no longer what is written as a value);
+* ``sink_score``: one more key in every softmax, of that score and without a value (0: one is added to the denominator).
 
 How it meets the kernels: as for ``NormedAttentionMixer`` the paged cache holds heads of ``D = ceil16(max(dim, vdim))``
 channels with zeros in the padding, the queries are written at that size by the kernel that rotates them and writes the
@@ -29,7 +33,8 @@ from .base import CompositeNeed, Mixer, Param, PositionEncoding, StateNeed, fuse
 class ConvAttentionMixer(Mixer):
     def __init__(self, prefix: str, hidden_size: int, num_heads: int, num_kv_heads: int, dim: int, vdim: int, scale: float,
                  window: Optional[int] = None, conv_taps: int = 0, qkv_bias: bool = True, out_bias: bool = True,
-                 position: Optional[PositionEncoding] = None, names: Tuple[Tuple[str, str], ...] = ()) -> None:
+                 position: Optional[PositionEncoding] = None, names: Tuple[Tuple[str, str], ...] = (), post_norm_eps: Optional[float] = None,
+                 values_are_keys: bool = False, sink_score: Optional[float] = None) -> None:
         """``conv_taps``: columns of the convolution's weights (0 or 1 column less than 2: 0 = no convolution);
         ``names``: pairs (tensor, name below the prefix) that replace the default names ``q``, ``k``, ``v``, ``o``; a
         bias is the tensor's name with ``.b`` added, a convolution's weights with ``.conv``."""
@@ -42,6 +47,14 @@ class ConvAttentionMixer(Mixer):
             raise ValueError(f"window={window} must be at least 1")
         if conv_taps < 0:
             raise ValueError("conv_taps must not be negative")
+        if values_are_keys and (int(vdim) != int(dim) or conv_taps):
+            raise ValueError("values that are the keys have the keys' size and come without a convolution")
+        if post_norm_eps is not None and not float(post_norm_eps) > 0:
+            raise ValueError("post_norm_eps must be positive")
+        self.post_norm_eps = float(post_norm_eps) if post_norm_eps is not None else None
+        self.values_are_keys = bool(values_are_keys)
+        self.sink_score = float(sink_score) if sink_score is not None else None
+        self.sinks: Optional[torch.Tensor] = None  # float32 [heads]
         self.interleaved = getattr(position, "layout", "halves") == "interleaved"
         self.hidden_size = int(hidden_size)
         self.num_heads = int(num_heads)
@@ -61,7 +74,7 @@ class ConvAttentionMixer(Mixer):
         self.names.update(dict(names))
         self.q_size = self.num_heads * self.dim
         self.k_size = self.num_kv_heads * self.dim
-        self.v_size = self.num_kv_heads * self.vdim
+        self.v_size = 0 if self.values_are_keys else self.num_kv_heads * self.vdim
         self.channels = self.q_size + self.k_size + self.v_size
         self.qkv_weight: Optional[torch.Tensor] = None
         self.qkv_bias_vec: Optional[torch.Tensor] = None
@@ -72,12 +85,14 @@ class ConvAttentionMixer(Mixer):
 
     def params(self) -> Dict[str, Param]:
         h, n = self.hidden_size, self.names
-        sizes = (self.q_size, self.k_size, self.v_size)
-        out = {"qkv_weight": fused_rows((n["q"], n["k"], n["v"]), tuple((s, h) for s in sizes))}
+        sources, sizes = (n["q"], n["k"], n["v"]), (self.q_size, self.k_size, self.v_size)
+        if self.values_are_keys:
+            sources, sizes = sources[:2], sizes[:2]
+        out = {"qkv_weight": fused_rows(sources, tuple((s, h) for s in sizes))}
         if self.qkv_bias:
-            out["qkv_bias_vec"] = fused_rows((n["q"] + ".b", n["k"] + ".b", n["v"] + ".b"), tuple((s,) for s in sizes), role="vector")
+            out["qkv_bias_vec"] = fused_rows(tuple(s + ".b" for s in sources), tuple((s,) for s in sizes), role="vector")
         if self.conv_taps:
-            out["conv_weight"] = fused_rows((n["q"] + ".conv", n["k"] + ".conv", n["v"] + ".conv"), tuple((s, self.conv_taps) for s in sizes), role="vector")
+            out["conv_weight"] = fused_rows(tuple(s + ".conv" for s in sources), tuple((s, self.conv_taps) for s in sizes), role="vector")
         out["o_weight"] = single(n["o"], (h, self.num_heads * self.vdim))
         if self.out_bias:
             out["o_bias_vec"] = single(n["o"] + ".b", (h,), role="vector")
@@ -90,6 +105,8 @@ class ConvAttentionMixer(Mixer):
         return CompositeNeed((pages, StateNeed((("conv_tail", (self.conv_taps - 1, self.channels), None),))))
 
     def finalize(self, device, dtype) -> None:
+        if self.sink_score is not None:
+            self.sinks = torch.full((self.num_heads,), self.sink_score, dtype=torch.float32, device=device)
         self.refresh_derived()
 
     def refresh_derived(self) -> None:
@@ -138,6 +155,8 @@ class ConvAttentionMixer(Mixer):
             qkv, self.num_heads, self.num_kv_heads, self.dim, self.vdim, self.cached_dim, ctx.positions, cos, sin,
             meta.slot_mapping, pages.tensors["k"], pages.tensors["v"], pages.block_size, write_kv=owns_cache,
             **({"interleaved": True} if self.interleaved else {}),
+            **({"post_norm_eps": self.post_norm_eps} if self.post_norm_eps is not None else {}),
+            **({"values_are_keys": True} if self.values_are_keys else {}),
         )
         attn = ops.paged_attention(
             q, self.num_heads, self.num_kv_heads, self.cached_dim,
@@ -146,6 +165,7 @@ class ConvAttentionMixer(Mixer):
             ctx.max_q_len, meta.max_kv_len, self.scale, self.window,
             ctx.all_decode, ctx.workspace,
             decode_prefix=getattr(ctx, "decode_prefix", 0), portions_max_kv_len=getattr(meta, "max_kv_len_of_portions", 0) or None,
+            **({"sinks": self.sinks} if self.sinks is not None else {}),
         )
         return ops.linear(attn, self.operand("o_padded" if self.o_padded is not None else "o_weight"), self.o_bias_vec if self.out_bias else None, ctx.dtype)
 

@@ -73,14 +73,20 @@ register_part("feed_forward", "gated_mlp", GatedMLP)
 
 class PlainMLP(FeedForward):
     """``W_down act(W_up x)`` without a gate branch and without biases; ``act`` is ``relu2`` (the square of the rectified
-    value).  The activation is float32 with one rounding at the store."""
+    value) or ``poly_norm``: with four learned numbers ``(a, b, c, e)``, ``a N(z) + b N(z^2) + c N(z^3) + e``, powers element
+    by element and ``N(y) = y / sqrt(mean(y^2) + norm_eps)`` over a token's whole row (so it needs the whole row and is a
+    kernel of its own between the products).  The activation is float32 with one rounding at the store."""
 
     def __init__(self, prefix: str, hidden_size: int, intermediate_size: int, activation: str = "relu2",
-                 names: Tuple[str, str] = ("up_proj.weight", "down_proj.weight")) -> None:
+                 names: Tuple[str, str] = ("up_proj.weight", "down_proj.weight"), norm_eps: float = 1e-6, coefficients_name: str = "act") -> None:
+        """``norm_eps``, ``coefficients_name`` (of the tensor of four numbers): for ``poly_norm`` only."""
         super().__init__(prefix)
-        if activation not in UNGATED_ACTIVATIONS:
-            raise ValueError(f"activation {activation!r} is not implemented ({', '.join(UNGATED_ACTIVATIONS)})")
+        if activation not in UNGATED_ACTIVATIONS + ("poly_norm",):
+            raise ValueError(f"activation {activation!r} is not implemented ({', '.join(UNGATED_ACTIVATIONS + ('poly_norm',))})")
         self.activation = activation
+        self.norm_eps = float(norm_eps)
+        self.coefficients_name = coefficients_name
+        self.coefficients: Optional[torch.Tensor] = None
         self.names = tuple(names)
         self.hidden_size = int(hidden_size)
         self.intermediate_size = int(intermediate_size)
@@ -89,7 +95,10 @@ class PlainMLP(FeedForward):
 
     def params(self) -> Dict[str, Param]:
         h, i = self.hidden_size, self.intermediate_size
-        return {"up_weight": single(self.names[0], (i, h)), "down_weight": single(self.names[1], (h, i))}
+        out = {"up_weight": single(self.names[0], (i, h)), "down_weight": single(self.names[1], (h, i))}
+        if self.activation == "poly_norm":
+            out["coefficients"] = single(self.coefficients_name, (4,), role="vector", init="one_plus_normal")
+        return out
 
     def prepare_kernels(self, ops) -> None:
         self.prepare_weight(ops, "up_weight")
@@ -97,7 +106,10 @@ class PlainMLP(FeedForward):
 
     def forward(self, x, ctx, sink=None):
         ops = ctx.ops
-        act = ops.linear_act(x, self.operand("up_weight"), ctx.dtype, self.activation)
+        if self.activation == "poly_norm":
+            act = ops.poly_norm(ops.linear(x, self.operand("up_weight"), None, ctx.dtype), self.coefficients, self.norm_eps)
+        else:
+            act = ops.linear_act(x, self.operand("up_weight"), ctx.dtype, self.activation)
         return ops.linear(act, self.operand("down_weight"), None, ctx.dtype, partials_ok=True)
 
 

@@ -33,9 +33,22 @@ halves of the low-rank maps and one for their second halves (a block-diagonal we
 cost one product together), the convolution, ``recurrence_prepare`` (unit vectors, decay, beta), ``linear_scan`` (the
 recurrence itself, token by token, a sequence's portion in order from its slot's state), ``gated_head_norm``, the output
 product.
+
+``GeneralDeltaMixer`` is the generalized delta rule: what is removed from the state and what is written to it are set
+apart.  Per head, with a decay ``w_t`` and a removal rate ``a_t`` per key channel, a read vector ``r_t``, a key ``k_t`` and its unit
+vector ``u_t = k_t / sqrt(sum(k_t^2) + 1e-6)``:
+
+    ``S <- diag(w_t) S - (a_t * u_t) (u_t^T S) + k_t v_t^T``  (both terms on the old state);  ``o_t = S^T r_t``
+
+with ``w_t = exp(-c sigmoid(W_w2 tanh(W_w1 x) + w0))``, ``a_t = sigmoid(W_a x + b_a)``, the read-out of each head divided by its root mean
+square, times a weight for every channel of all heads, times ``sigmoid(W_g x)``, then the output product.  Its kernels: one
+product for everything that reads ``x`` (``[r; k; v; a; g; w1]``), ``removal_prepare`` (unit vectors and lengths of the keys, removal
+vectors, the second half of the low-rank decay map and the decay itself, all float32), ``linear_scan`` with the same lanes
+and staging as above, ``gated_head_norm``, the output product.
 """
 from __future__ import annotations
 
+import math
 from typing import Dict, Optional, Tuple
 
 import torch
@@ -202,7 +215,7 @@ class LinearRecurrenceMixer(Mixer):
             main if self.rule == "delta" else None, self.beta_at or 0,
         )
         read = ops.linear_scan(qk, qkv, v_at, decay, beta, cache.tensors["state"], ctx.slots, ctx.cu_q, ctx.max_q_len,
-                               heads, kv_heads, dim, vdim, self.rule == "delta")
+                               heads, kv_heads, dim, vdim, self.rule)
         if self.gate == "silu":
             gate_source, gate_at, gate_kind = main, self.g_at, "silu"
         else:
@@ -212,3 +225,64 @@ class LinearRecurrenceMixer(Mixer):
 
 
 register_part("mixer", "linear_recurrence", LinearRecurrenceMixer)
+
+
+class GeneralDeltaMixer(Mixer):
+    def __init__(self, prefix: str, hidden_size: int, num_heads: int, dim: int, vdim: int, norm_eps: float, decay_rank: int, decay_scale: float = math.exp(-0.5),
+                 names: Tuple[Tuple[str, str], ...] = ()) -> None:
+        """``decay_rank``: the inner size of the decay's low-rank map (rows of ``w1``); ``decay_scale``: the constant ``c``;
+        ``names``: pairs (tensor, name below the prefix) that replace the default names."""
+        super().__init__(prefix)
+        if min(int(num_heads), int(dim), int(vdim), int(decay_rank)) < 1 or not float(decay_scale) > 0 or not float(norm_eps) > 0:
+            raise ValueError("heads, dim, vdim, decay_rank, decay_scale and norm_eps must be positive")
+        self.hidden_size = int(hidden_size)
+        self.num_heads, self.dim, self.vdim = int(num_heads), int(dim), int(vdim)
+        self.norm_eps = float(norm_eps)
+        self.decay_rank, self.decay_scale = int(decay_rank), float(decay_scale)
+        self.names = {n: n for n in ("r", "k", "v", "a", "g", "w1", "w2", "w0", "norm", "o")}
+        self.names.update({"a_bias": "a.b"})
+        self.names.update(dict(names))
+        self.k_size, self.v_size = self.num_heads * self.dim, self.num_heads * self.vdim
+        # columns of the first product
+        self.r_at, self.k_at, self.v_at = 0, self.k_size, 2 * self.k_size
+        self.a_at = self.v_at + self.v_size
+        self.g_at = self.a_at + self.k_size
+        self.low_at = self.g_at + self.v_size
+        self.main_weight = self.w2_weight = self.w0 = self.a_bias = self.norm_weight = self.o_weight = None
+
+    def params(self) -> Dict[str, Param]:
+        h, n = self.hidden_size, self.names
+        rows = ((n["r"], self.k_size), (n["k"], self.k_size), (n["v"], self.v_size), (n["a"], self.k_size), (n["g"], self.v_size), (n["w1"], self.decay_rank))
+        return {
+            "main_weight": fused_rows(tuple(r[0] for r in rows), tuple((r[1], h) for r in rows)),
+            "a_bias": single(n["a_bias"], (self.k_size,), role="vector"),
+            "w2_weight": single(n["w2"], (self.k_size, self.decay_rank), product=False),  # (read by ``removal_prepare``)
+            "w0": single(n["w0"], (self.k_size,), role="vector"),
+            "norm_weight": single(n["norm"], (self.v_size,), role="vector", init="one_plus_normal"),
+            "o_weight": single(n["o"], (h, self.v_size)),
+        }
+
+    def cache_need(self):
+        return StateNeed((("state", (self.num_heads, self.dim, self.vdim), torch.float32),))
+
+    def prepare_kernels(self, ops) -> None:
+        self.prepare_weight(ops, "main_weight")
+        self.prepare_weight(ops, "o_weight")
+        check = getattr(ops, "linear_scan_supports", None)
+        if check is not None:
+            check(self.dim, self.vdim)
+
+    def forward(self, x, ctx, cache, owns_cache: bool = True):
+        if not owns_cache:
+            raise RuntimeError("a recurrent mixer cannot read another entry's state: every run of it advances a state of its own")
+        ops = ctx.ops
+        main = ops.linear(x, self.operand("main_weight"), None, ctx.dtype)
+        vectors, decay, lengths = ops.removal_prepare(main, self.r_at, self.k_at, self.a_at, self.low_at, self.decay_rank, self.num_heads, self.dim,
+                                                      self.a_bias, self.w2_weight, self.w0, self.decay_scale)
+        read = ops.linear_scan(vectors, main, self.v_at, decay, lengths, cache.tensors["state"], ctx.slots, ctx.cu_q, ctx.max_q_len,
+                               self.num_heads, self.num_heads, self.dim, self.vdim, "removal")
+        y = ops.gated_head_norm(read, self.norm_weight, self.norm_eps, main, self.g_at, "sigmoid", self.num_heads, self.vdim, ctx.dtype)
+        return ops.linear(y, self.operand("o_weight"), None, ctx.dtype, partials_ok=True)
+
+
+register_part("mixer", "general_delta", GeneralDeltaMixer)

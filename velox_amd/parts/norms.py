@@ -13,7 +13,7 @@ from typing import Dict, Optional
 
 import torch
 
-from .base import DeferredNorm, Norm, Param, ResidualCopy, ScaledSum, StreamUpdate, register_part, single
+from .base import DeferredNorm, Norm, NormedDelta, Param, ReadyInput, ResidualCopy, ScaledSum, StreamUpdate, register_part, single
 
 
 class RMSNorm(Norm):
@@ -39,6 +39,15 @@ class RMSNorm(Norm):
             if delta.norm is not self or rows is not None:
                 raise ValueError("a DeferredNorm can only go to the norm it was made for, on all rows")
             return delta
+        if isinstance(delta, ReadyInput):
+            if delta.norm is not self or rows is not None:
+                raise ValueError("a ReadyInput can only go to the norm it was made for, on all rows")
+            return delta.x
+        if isinstance(delta, NormedDelta):
+            form = delta.norm.deferred_form()
+            if form is None:
+                raise ValueError(f"{type(delta.norm).__name__} cannot norm a sub-layer's output inside the next norm's kernel")
+            return ctx.ops.norm_add_norm(residual, delta.y, form[0], form[1], self.weight, self.eps, ctx.dtype, rows=rows)
         if isinstance(delta, ResidualCopy):
             delta = None  # (the block before has added everything itself)
         if rows is None:
