@@ -16,6 +16,9 @@ over the steps in which all of them decode, ``..._frac``: that step's share of t
 ``e2e_b<B>_p512_g256``: generated tokens / wall time with the prompts' time included, which is how
 the reference's ``benchmark.py:204`` counts).
 
+``--design kedanex`` measures the Kedanex design (a norm on both sides of every sub-layer, the generalized delta rule, a gated recurrence per
+channel, window attention whose values are the keys, PolyNorm, experts) beside Gosulorn with one stream (the closest recurrent mixers) and
+Tiverax with the same experts.
 ``--design lelutar`` measures the Lelutar design (norms without statistics, a hashed table of token pairs beside the embedding, grouped-query
 attention with two head sizes beside attention over a latent with a sink and a gate per head, ungated experts chosen among the best groups)
 beside Tiverax with the same experts and the dense decoder with the same heads.
@@ -332,6 +335,27 @@ def lelutar_config(size: dict) -> dict:
             "embedding": {"scale": size["width"] ** 0.5, "bigram": {"buckets": size["buckets"], "mul_prev": 1000003, "mul_cur": 998244353 % 65536}}, "layers": layers}
 
 
+# Layer sizes for --design kedanex: eight layers, twice (the generalized delta rule with a dense feed-forward, a gated recurrence,
+# attention over a sliding window, the generalized delta rule, these three with experts); the last layer runs the weights of
+# layer 3 again.  Beside it: Gosulorn at the same width with one stream, and Tiverax with the same experts in every layer.
+KEDANEX_SIZES = {
+    "2k": dict(width=2048, delta_heads=32, delta_dim=64, rank=64, gru_width=3072, heads=16, kv_heads=4, dim=128, window=1024, ff=8448, experts=16, top=2, expert_ff=1408),
+    "4k": dict(width=4096, delta_heads=64, delta_dim=64, rank=128, gru_width=6144, heads=32, kv_heads=8, dim=128, window=2048, ff=16512, experts=32, top=4, expert_ff=1408),
+}
+
+
+def kedanex_config(size: dict) -> dict:
+    delta = {"heads": size["delta_heads"], "dim": size["delta_dim"], "w1_rank": size["rank"]}
+    attention = {"heads": size["heads"], "kv_heads": size["kv_heads"], "dim": size["dim"], "vdim": size["dim"], "scale": size["dim"] ** -0.5,
+                 "mask": {"size": size["window"]}, "rot": {"dims": size["dim"], "base": 1e6}}
+    dense = {"kind": "dense", "ff": size["ff"]}
+    routed = {"kind": "moe", "router": {"experts": size["experts"], "top": size["top"]}, "expert": {"ff": size["expert_ff"]}}
+    order = (("general_delta", delta, dense), ("mingru", {"width": size["gru_width"]}, routed), ("attention", attention, routed), ("general_delta", delta, routed))
+    layers = [{"type": kind, "mixer": mixer, "mlp": mlp} for kind, mixer, mlp in order * 2]
+    layers[7]["weights_of"] = 3
+    return {"architecture": "Kedanex", "vocab": DESIGN_VOCAB, "width": size["width"], "norm": {"eps": 1e-6}, "layers": layers}
+
+
 def tiverax_all_routed(size: dict) -> dict:
     """Tiverax at the width of ``size`` with the same experts per layer and per token (no shared expert, no dense layers)."""
     config = tiverax_config(dict(TIVERAX_SIZES["2k" if size["width"] == 2048 else "4k"], experts=size["experts"], top=size["top"], expert_ff=size["expert_ff"]))
@@ -348,6 +372,9 @@ def designs_at(design: str, name: str):
     if design == "gosulorn":
         size = GOSULORN_SIZES[name]
         return (("gosulorn", gosulorn_config(size)), ("qwen2", qwen2_like(dict(size, rot_dim=0))))
+    if design == "kedanex":
+        size = KEDANEX_SIZES[name]
+        return (("kedanex", kedanex_config(size)), ("gosulorn", gosulorn_config(dict(GOSULORN_SIZES[name], streams=1))), ("tiverax", tiverax_all_routed(size)))
     if design == "lelutar":
         size = LELUTAR_SIZES[name]
         dense = dict(width=size["width"], heads=size["heads"], kv_heads=size["kv_heads"], dim=size["dim"], rot_dim=0, ff=size["top"] * size["expert_ff"])
@@ -401,7 +428,7 @@ def main() -> int:
     parser.add_argument("--shape", default="7b", choices=sorted(SHAPES), help="layer sizes: the headline is 7b; 1.5b and 32b are the reference's other two")
     parser.add_argument("--far", action="store_true",
                         help="further sizes under `points`: decode at batch 1 and 8 behind 32,256 tokens, a prefill of 8,192 tokens, and a decode step of a true float32 run (batch 8)")
-    parser.add_argument("--design", default=None, choices=["tiverax", "dipisun", "gosulorn", "lelutar"],
+    parser.add_argument("--design", default=None, choices=["tiverax", "dipisun", "gosulorn", "lelutar", "kedanex"],
                         help="instead of the headline: prefill and decode of this design at real layer sizes beside the framework's closest models of equal size")
     parser.add_argument("--only", default="", help="with --design: which of the models that are measured side by side (names with commas between them; default: all)")
     parser.add_argument("--sizes", default="2k,4k", help="with --design: which of the sizes (2k, 4k = the models' widths)")
@@ -415,7 +442,7 @@ def main() -> int:
         points = design_points(args)
         first = args.sizes.split(",")[0]
         head = points.get(f"{args.design}_{first}") or next(iter(points.values()))
-        sizes = {"tiverax": TIVERAX_SIZES, "dipisun": DIPISUN_SIZES, "gosulorn": GOSULORN_SIZES, "lelutar": LELUTAR_SIZES}[args.design]
+        sizes = {"tiverax": TIVERAX_SIZES, "dipisun": DIPISUN_SIZES, "gosulorn": GOSULORN_SIZES, "lelutar": LELUTAR_SIZES, "kedanex": KEDANEX_SIZES}[args.design]
         print(json.dumps({
             "metric": "decode_tokens_per_second", "value": head["decode_tok_s"], "unit": "tok/s", "n_gpus": 1, "steps": args.steps,
             "warmup": args.warmup, "ms_per_step": head["decode_ms"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None,

@@ -543,7 +543,8 @@ struct RemovalArgs {
 
 template <typename T>
 __global__ void __launch_bounds__(256) removal_prepare_kernel(const RemovalArgs a) {
-  extern __shared__ float inner[];  // [group, rank], behind the tanh
+  extern __shared__ float4_t inner_pieces[];
+  float* inner = reinterpret_cast<float*>(inner_pieces);  // [group, rank], behind the tanh
   const int h = blockIdx.x, t0 = blockIdx.y * a.group;
   const int count = a.tokens - t0 < a.group ? a.tokens - t0 : a.group;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -584,17 +585,22 @@ __global__ void __launch_bounds__(256) removal_prepare_kernel(const RemovalArgs 
       x[j] = inner + (j0 + j < count ? j0 + j : count - 1) * rank;  // (a place beyond the group follows the last token and is not stored)
     }
     if (vec) {
-      for (int m = 0; m < rank; m += 8) {
+      for (int m = 0; m < rank; m += 8) {  // (16-byte pieces of w2's row and of the inner rows, which start at multiples of 32 bytes)
         const float4_t raw = *reinterpret_cast<const float4_t*>(w + m);
+        float wide[8];
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
           const unsigned bits = __float_as_uint(raw[e]);
-          const float lo = __uint_as_float(bits << 16), hi = __uint_as_float(bits & 0xffff0000u);
+          wide[2 * e] = __uint_as_float(bits << 16);
+          wide[2 * e + 1] = __uint_as_float(bits & 0xffff0000u);
+        }
 #pragma unroll
-          for (int j = 0; j < REMOVAL_TOKENS; ++j) {
-            z[j] += lo * x[j][m + 2 * e];
-            z[j] += hi * x[j][m + 2 * e + 1];
-          }
+        for (int j = 0; j < REMOVAL_TOKENS; ++j) {
+          const float4_t first = *reinterpret_cast<const float4_t*>(x[j] + m), second = *reinterpret_cast<const float4_t*>(x[j] + m + 4);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) z[j] += wide[e] * first[e];
+#pragma unroll
+          for (int e = 0; e < 4; ++e) z[j] += wide[4 + e] * second[e];
         }
       }
     } else {
