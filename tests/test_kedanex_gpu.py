@@ -118,6 +118,57 @@ def test_generalized_delta_rule_kernels(ops, dtype, heads, dim, vdim, rank):
     assert not torch.equal(states[0], kept)
 
 
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("heads,dim,vdim,rank", [(2, 64, 64, 16), (1, 128, 48, 24), (3, 16, 20, 5), (2, 32, 7, 33), (1, 48, 48, 1), (5, 80, 80, 64), (1, 96, 33, 8), (1, 112, 16, 3)])
+def test_chunks_of_tokens_equal_the_token_by_token_kernels(ops, dtype, heads, dim, vdim, rank):
+    """Long and short portions beside single tokens (chunks that are full, partly filled, of one token), strong and weak decays,
+    keys that come back unchanged, against the plain reference; then a loud first token that must still be read at the end
+    of a long portion, whole and in pieces that end inside and at a chunk's border."""
+    ref, dt = TorchOps(), DTYPES[dtype]
+    ks, vs = heads * dim, heads * vdim
+    width = 3 * ks + 2 * vs + rank
+    at = (0, ks, 2 * ks, 2 * ks + vs, 3 * ks + 2 * vs)
+    w2 = (torch.randn(ks, rank) * 2 / math.sqrt(rank)).to(dt).cuda()
+    a_bias, w0 = torch.randn(ks).cuda() * 2, torch.randn(ks).cuda() * 3  # (decays from 0.545 to 1, removal rates from 0 to 1)
+    states = [torch.randn(5, heads, dim, vdim).cuda() * 0.3]
+    states.append(states[0].clone())
+    kept = states[0].clone()
+    for lengths, slots in (((100, 1, 16, 33), (3, 0, 2, 1)), ((17,), (2,)), ((1, 48, 15), (1, 3, 0)), ((300, 2), (0, 3))):
+        cu, slot = ints([0] + list(np.cumsum(lengths))), ints(slots)
+        main = torch.randn(sum(lengths), width)
+        main[3::4, ks:2 * ks] = main[2::4, ks:2 * ks][: main[3::4].shape[0]]  # (every fourth key is the one before it)
+        main = main.to(dt).cuda()
+        got = ops.removal_scan(main, *at, rank, heads, dim, vdim, a_bias, w2, w0, math.exp(-0.5), states[0], slot, cu, max(lengths), chunked=True)
+        want = ref.removal_scan(main, *at, rank, heads, dim, vdim, a_bias, w2, w0, math.exp(-0.5), states[1], slot, cu, max(lengths))
+        near(got, want, 3e-5, "read-out")
+        near(states[0], states[1], 3e-5, "state")
+    assert torch.equal(states[0][4], kept[4])  # (a slot nobody holds is left alone)
+    # a loud first token behind decays near 1 and removal rates near 0
+    n = 500
+    main = torch.randn(n, width)
+    main[:, at[4]:] *= 0.2
+    main[0, at[2]:at[2] + vs] *= 300.0
+    main = main.to(dt).cuda()
+    slow = torch.full((ks,), -8.0).cuda()
+
+    def run(cuts, rows, **kw):
+        state, outs, here = torch.zeros(2, heads, dim, vdim).cuda(), [], 0
+        for c in cuts:
+            outs.append(ops.removal_scan(rows[here:here + c].clone(), *at, rank, heads, dim, vdim, slow, w2 * 0.1, slow, math.exp(-0.5), state, ints([1]), ints([0, c]), c, **kw))
+            here += c
+        return torch.cat(outs), state
+
+    whole, state = run((n,), main)
+    assert torch.equal(whole, run((n,), main)[0])
+    for cuts, kw in (((n,), dict(chunked=False)), ((1, 2, 300, 17, 180), {}), ((16, 32, 47, 405), {}), ((15, 33, 452), dict(chunked=True))):
+        pieces, piece_state = run(cuts, main, **kw)
+        near(pieces, whole, 3e-5, f"pieces {cuts}")
+        near(piece_state, state, 3e-5, f"state {cuts}")
+    quiet = main.clone()
+    quiet[0, at[2]:at[2] + vs] = 0.0
+    assert float((run((n,), quiet)[0][-1] - whole[-1]).abs().max()) > 0.2 * float(whole[-1].abs().max())
+
+
 @pytest.mark.parametrize("heads,dim,vdim", [(2, 64, 64), (1, 128, 128), (3, 32, 48), (2, 12, 12), (1, 256, 16), (1, 72, 40)])
 def test_a_long_portion_equals_its_pieces_and_its_first_token_is_kept(ops, heads, dim, vdim):
     """600 tokens in one step, in pieces (one of a single token, one of two) and against the plain loop; with decays close

@@ -238,6 +238,10 @@ class TorchOps:
         z = torch.tanh(main[:, low_at:low_at + rank].float()) @ w2.float().T + w0
         return torch.stack([r.view(t, heads, dim), u, removal], 2).contiguous(), torch.exp(-decay_scale * torch.sigmoid(z)), lengths
 
+    def removal_scan(self, main, r_at, k_at, v_at, a_at, low_at, rank, heads, dim, vdim, a_bias, w2, w0, decay_scale, state, slots, cu_q, max_q_len):
+        vectors, decay, lengths = self.removal_prepare(main, r_at, k_at, a_at, low_at, rank, heads, dim, a_bias, w2, w0, decay_scale)
+        return self.linear_scan(vectors, main, v_at, decay, lengths, state, slots, cu_q, max_q_len, heads, heads, dim, vdim, "removal")
+
     def gated_scan(self, projected, width, gate_bias, input_bias, shift, state, slots, cu_q, max_q_len):
         """``S <- (1 - z) S + z c`` per channel from ``state[slot]``, which is written back; -> ``S * silu(g)``."""
         z = torch.sigmoid(projected[:, :width].float() + gate_bias)

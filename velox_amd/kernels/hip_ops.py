@@ -176,6 +176,10 @@ class HipOps:
         c.velox_gated_scan_scratch_elems.restype = ctypes.c_longlong
         c.velox_norm_add_norm.argtypes = [_P, _P, _I, _P, _F, _P, _F, _P, _P, _I, _I, _I, _I, ctypes.c_longlong, _P]
         c.velox_poly_norm.argtypes = [_P, _P, _P, _I, _I, _F, _I, _P]
+        c.velox_removal_chunk_scan.argtypes = [_P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I, _P, _P, _P, _F, _P, _P, _P, _P, _P, _I, _I, _P]
+        c.velox_removal_chunk_scan.restype = _I
+        c.velox_removal_chunk_scratch_elems.argtypes = [_I, _I, _I, _I, _I, _I]
+        c.velox_removal_chunk_scratch_elems.restype = ctypes.c_longlong
         for fn in (c.velox_removal_prepare, c.velox_gated_scan, c.velox_norm_add_norm, c.velox_poly_norm):
             fn.restype = _I
         c.velox_embed_bigram.argtypes = [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _P, _P, _P, _P, _P]
@@ -1106,6 +1110,46 @@ class HipOps:
                                                         int(dim), _ptr(a_bias), _ptr(w2), _ptr(w0), float(decay_scale), _ptr(vectors), _ptr(decay), _ptr(lengths),
                                                         tokens, self._stream()), "removal_prepare")
         return vectors, decay, lengths
+
+    REMOVAL_CHUNK_TOKENS = 32  # portions at least this long go through the chunked kernels where the sizes are theirs
+
+    def removal_scan(self, main, r_at, k_at, v_at, a_at, low_at, rank, heads, dim, vdim, a_bias, w2, w0, decay_scale, state, slots, cu_q, max_q_len,
+                     chunked: Optional[bool] = None):
+        """The generalized delta rule from the rows of its input product (columns as for ``removal_prepare``, values of ``heads * vdim``
+        columns at ``v_at``) and ``state`` [slots, heads, dim, vdim], which is written back; float32 read-outs [T, heads * vdim].  Steps with a
+        long portion are worked in chunks of 16 tokens on the matrix cores (heads of a multiple of 16 channels, 128 at most, and
+        decays whose product over a chunk keeps away from underflow), all others token by token; ``chunked`` decides it for a
+        test."""
+        tokens = main.shape[0]
+        scratch_elems = 0
+        if chunked is not False and max_q_len >= (1 if chunked else self.REMOVAL_CHUNK_TOKENS) and 16 * decay_scale < 13:
+            scratch_elems = int(self._core.velox_removal_chunk_scratch_elems(tokens, slots.shape[0], int(heads), int(dim), int(vdim), int(rank)))
+        if scratch_elems == 0:
+            if chunked:
+                raise KernelError(f"removal_scan: heads of {dim} channels with an inner size of {rank} are not the chunked kernels'")
+            vectors, decay, lengths = self.removal_prepare(main, r_at, k_at, a_at, low_at, rank, heads, dim, a_bias, w2, w0, decay_scale)
+            return self.linear_scan(vectors, main, v_at, decay, lengths, state, slots, cu_q, max_q_len, heads, heads, dim, vdim, "removal")
+        self._check("main", main)
+        size = heads * dim
+        if (main.dim() != 2 or max(r_at, k_at, a_at) + size > main.shape[1] or low_at + rank > main.shape[1] or v_at + heads * vdim > main.shape[1]
+                or min(r_at, k_at, v_at, a_at, low_at) < 0):
+            raise KernelError("removal_scan: the columns do not lie within the rows")
+        self._check("a_bias", a_bias, torch.float32, (size,))
+        self._check("w0", w0, torch.float32, (size,))
+        self._check("w2", w2, main.dtype, (size, rank))
+        self._check("state", state, torch.float32)
+        if state.dim() != 4 or tuple(state.shape[1:]) != (heads, dim, vdim):
+            raise KernelError(f"removal_scan: the state must be [slots, {heads}, {dim}, {vdim}], got {tuple(state.shape)}")
+        self._check("slots", slots, torch.int32)
+        self._check("cu_q", cu_q, torch.int32, (slots.shape[0] + 1,))
+        if not 1 <= max_q_len <= tokens:
+            raise KernelError(f"removal_scan: max_q_len={max_q_len} outside [1, {tokens}]")
+        out = torch.empty((tokens, heads * vdim), dtype=torch.float32, device=self.device)
+        scratch = torch.empty(scratch_elems, dtype=torch.float32, device=self.device)
+        self._launched(self._core.velox_removal_chunk_scan(_ptr(main), _code(main.dtype), main.shape[1], int(r_at), int(k_at), int(v_at), int(a_at), int(low_at), int(rank),
+                                                           int(heads), int(dim), int(vdim), _ptr(a_bias), _ptr(w2), _ptr(w0), float(decay_scale), _ptr(scratch), _ptr(state),
+                                                           _ptr(slots), _ptr(cu_q), _ptr(out), slots.shape[0], int(max_q_len), self._stream()), "removal_scan")
+        return out
 
     def gated_scan(self, projected, width, gate_bias, input_bias, shift, state, slots, cu_q, max_q_len):
         """``projected`` [T, 3 * width] = z, u, g of every token; per channel and sequence, from ``state[slot]`` ([slots, width] float32, written

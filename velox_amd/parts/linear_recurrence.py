@@ -42,9 +42,11 @@ vector ``u_t = k_t / sqrt(sum(k_t^2) + 1e-6)``:
 
 with ``w_t = exp(-c sigmoid(W_w2 tanh(W_w1 x) + w0))``, ``a_t = sigmoid(W_a x + b_a)``, the read-out of each head divided by its root mean
 square, times a weight for every channel of all heads, times ``sigmoid(W_g x)``, then the output product.  Its kernels: one
-product for everything that reads ``x`` (``[r; k; v; a; g; w1]``), ``removal_prepare`` (unit vectors and lengths of the keys, removal
-vectors, the second half of the low-rank decay map and the decay itself, all float32), ``linear_scan`` with the same lanes
-and staging as above, ``gated_head_norm``, the output product.
+product for everything that reads ``x`` (``[r; k; v; a; g; w1]``), ``removal_scan``, ``gated_head_norm``, the output product.  ``removal_scan`` is
+two kernels: for steps of single tokens and short portions ``removal_prepare`` (unit vectors and lengths of the keys, removal
+vectors, the second half of the low-rank decay map and the decay itself, all float32) and ``linear_scan`` with the same lanes and
+staging as above; for long portions chunks of 16 tokens on the float32 matrix instructions (everything that does not touch the
+state for all chunks at once, then a chain of chunks).
 """
 from __future__ import annotations
 
@@ -277,10 +279,8 @@ class GeneralDeltaMixer(Mixer):
             raise RuntimeError("a recurrent mixer cannot read another entry's state: every run of it advances a state of its own")
         ops = ctx.ops
         main = ops.linear(x, self.operand("main_weight"), None, ctx.dtype)
-        vectors, decay, lengths = ops.removal_prepare(main, self.r_at, self.k_at, self.a_at, self.low_at, self.decay_rank, self.num_heads, self.dim,
-                                                      self.a_bias, self.w2_weight, self.w0, self.decay_scale)
-        read = ops.linear_scan(vectors, main, self.v_at, decay, lengths, cache.tensors["state"], ctx.slots, ctx.cu_q, ctx.max_q_len,
-                               self.num_heads, self.num_heads, self.dim, self.vdim, "removal")
+        read = ops.removal_scan(main, self.r_at, self.k_at, self.v_at, self.a_at, self.low_at, self.decay_rank, self.num_heads, self.dim, self.vdim,
+                                self.a_bias, self.w2_weight, self.w0, self.decay_scale, cache.tensors["state"], ctx.slots, ctx.cu_q, ctx.max_q_len)
         y = ops.gated_head_norm(read, self.norm_weight, self.norm_eps, main, self.g_at, "sigmoid", self.num_heads, self.vdim, ctx.dtype)
         return ops.linear(y, self.operand("o_weight"), None, ctx.dtype, partials_ok=True)
 
