@@ -37,17 +37,17 @@ struct RemovalChunkArgs {
   float* out;  // [T, heads * vdim]
 };
 
-// A chunk and head in `scratch`, in floats: U' | R' | -B | K (each 16 * dim), P_16 (dim), Dv | Ov (each 16 * columns).  U' and R' as
-// [dim / 16][16 tokens][16 channels], B and K as [dim][16 tokens], Dv and Ov as [columns][16 tokens]: what a wave reads of one
+// A chunk and head in `scratch`, in floats: U' | R' | -B | K (each 16 * dim), P_16 (dim), Dv | Ov | V (each 16 * columns).  U' and R' as
+// [dim / 16][16 tokens][16 channels], B and K as [dim][16 tokens], Dv, Ov and V as [columns][16 tokens]: what a wave reads of one
 // of them is one contiguous kilobyte, 16 bytes a lane.
 __host__ __device__ __forceinline__ int removal_columns(int vdim) { return (vdim + 15) / 16 * 16; }
-__host__ __device__ __forceinline__ size_t removal_record(int dim, int vdim) { return (size_t)65 * dim + 32 * removal_columns(vdim); }
+__host__ __device__ __forceinline__ size_t removal_record(int dim, int vdim) { return (size_t)65 * dim + 48 * removal_columns(vdim); }
 // the first record of a sequence: sequences' chunks never overlap, because floor((a + n) / 16) + 1 >= floor(a / 16) + ceil(n / 16)
 __device__ __forceinline__ int removal_first_chunk(int first_token, int sequence) { return first_token / CHUNK + sequence; }
 
 __device__ __forceinline__ float removal_sigmoid(float z) { return 1.f / (1.f + expf(-z)); }
 __device__ __forceinline__ float4_t mfma4(float a, float b, float4_t c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
-__device__ __forceinline__ float4_t lds4(const float* p) { return *reinterpret_cast<const float4_t*>(p); }
+__device__ __forceinline__ float4_t four(const float* p) { return *reinterpret_cast<const float4_t*>(p); }
 
 template <typename T>
 __global__ void __launch_bounds__(256) removal_chunk_prepare_kernel(const RemovalChunkArgs a) {
@@ -69,29 +69,42 @@ __global__ void __launch_bounds__(256) removal_chunk_prepare_kernel(const Remova
   float* small = inner + CHUNK * inner_row;
   const T* rows = (const T*)a.main + (size_t)t0 * a.ld;
 
+  // a wave takes four tokens and a lane two channels of each (dim <= 128): all of a wave's loads are asked for before the first
+  // is used (tokens beyond the portion: zeros, with decays of 1)
+  float r[4][2], k[4][2], al[4][2];
+#pragma unroll
+  for (int q = 0; q < 4; ++q) {
+    const int j = wave + 4 * q;
+    const T* mine = rows + (size_t)j * a.ld + (size_t)h * dim;
+#pragma unroll
+    for (int p = 0; p < 2; ++p) {
+      const int c = lane + 64 * p;
+      const bool there = j < count && c < dim;
+      r[q][p] = there ? to_f32(mine[a.r_at + c]) : 0.f;
+      k[q][p] = there ? to_f32(mine[a.k_at + c]) : 0.f;
+      al[q][p] = there ? to_f32(mine[a.a_at + c]) : 0.f;
+    }
+  }
+  const float bias[2] = {lane < dim ? a.a_bias[(size_t)h * dim + lane] : 0.f, lane + 64 < dim ? a.a_bias[(size_t)h * dim + lane + 64] : 0.f};
+#pragma unroll 4
   for (int i = tid; i < CHUNK * padded_rank; i += 256) {
     const int j = i / padded_rank, m = i - j * padded_rank;
     inner[j * inner_row + m] = j < count && m < rank ? tanhf(to_f32(rows[(size_t)j * a.ld + a.low_at + m])) : 0.f;
   }
-  const float* bias = a.a_bias + (size_t)h * dim;
-  for (int j = wave; j < CHUNK; j += 4) {  // (tokens beyond the portion: zeros, with decays of 1)
-    const T* mine = rows + (size_t)j * a.ld + (size_t)h * dim;
-    float s = 0.f;
-    if (j < count)
-      for (int c = lane; c < dim; c += 64) { const float v = to_f32(mine[a.k_at + c]); s += v * v; }
-    const float inv = 1.f / sqrtf(wave_sum(s) + 1e-6f);
-    for (int c = lane; c < dim; c += 64) {
-      float r = 0.f, k = 0.f, u = 0.f, removal = 0.f;
-      if (j < count) {
-        r = to_f32(mine[a.r_at + c]);
-        k = to_f32(mine[a.k_at + c]);
-        u = k * inv;
-        removal = removal_sigmoid(to_f32(mine[a.a_at + c]) + bias[c]) * u;
+#pragma unroll
+  for (int q = 0; q < 4; ++q) {
+    const int j = wave + 4 * q;
+    const float inv = 1.f / sqrtf(wave_sum(k[q][0] * k[q][0] + k[q][1] * k[q][1]) + 1e-6f);
+#pragma unroll
+    for (int p = 0; p < 2; ++p) {
+      const int c = lane + 64 * p;
+      if (c < dim) {
+        const float u = k[q][p] * inv;
+        matrix[0][j * row + c] = u;
+        matrix[1][j * row + c] = r[q][p];
+        matrix[2][j * row + c] = removal_sigmoid(al[q][p] + bias[p]) * u;
+        matrix[3][j * row + c] = k[q][p];
       }
-      matrix[0][j * row + c] = u;
-      matrix[1][j * row + c] = r;
-      matrix[2][j * row + c] = removal;
-      matrix[3][j * row + c] = k;
     }
   }
   __syncthreads();
@@ -101,10 +114,21 @@ __global__ void __launch_bounds__(256) removal_chunk_prepare_kernel(const Remova
     const size_t channel = (size_t)h * dim + tile * 16;
     const T* w = (const T*)a.w2 + (channel + n) * rank;
     float4_t z = {0.f, 0.f, 0.f, 0.f};
-    for (int m = 4 * g; m < padded_rank; m += 16) {
-      const float4_t x = lds4(inner + n * inner_row + m);
+    if (rank % 16 == 0 && ((uintptr_t)a.w2 & 15) == 0) {  // (then four neighbours of a row are one access)
+#pragma unroll 4
+      for (int m = 4 * g; m < padded_rank; m += 16) {
+        float y[4];
+        load4<T>(w, 0, m, rank, true, true, y);
+        const float4_t x = four(inner + n * inner_row + m);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) z = mfma4(m + e < rank ? to_f32(w[m + e]) : 0.f, x[e], z);
+        for (int e = 0; e < 4; ++e) z = mfma4(y[e], x[e], z);
+      }
+    } else {
+      for (int m = 4 * g; m < padded_rank; m += 16) {
+        const float4_t x = four(inner + n * inner_row + m);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) z = mfma4(m + e < rank ? to_f32(w[m + e]) : 0.f, x[e], z);
+      }
     }
     float4_t dec;
 #pragma unroll
@@ -145,7 +169,7 @@ __global__ void __launch_bounds__(256) removal_chunk_prepare_kernel(const Remova
     const float* right = matrix[(wave & 1) ? 2 : 3] + n * row;
     float4_t m = {0.f, 0.f, 0.f, 0.f};
     for (int c = 4 * g; c < dim; c += 16) {
-      const float4_t x = lds4(left + c), y = lds4(right + c);
+      const float4_t x = four(left + c), y = four(right + c);
 #pragma unroll
       for (int e = 0; e < 4; ++e) m = mfma4(x[e], y[e], m);
     }
@@ -171,7 +195,7 @@ __global__ void __launch_bounds__(256) removal_chunk_prepare_kernel(const Remova
       float v = t == n ? 1.f : 0.f;
 #pragma unroll
       for (int q = 0; q < (t + 3) / 4; ++q) {
-        const float4_t m = lds4(M2 + t * CHUNK_STRIDE + 4 * q);
+        const float4_t m = four(M2 + t * CHUNK_STRIDE + 4 * q);
 #pragma unroll
         for (int e = 0; e < 4; ++e)
           if (4 * q + e < t) v -= m[e] * x[4 * q + e];
@@ -185,7 +209,7 @@ __global__ void __launch_bounds__(256) removal_chunk_prepare_kernel(const Remova
   }
   __syncthreads();
   if (wave < 2) {  // M4 T and T M1
-    const float4_t x = lds4((wave == 0 ? M4 : inverse) + n * CHUNK_STRIDE + 4 * g);
+    const float4_t x = four((wave == 0 ? M4 : inverse) + n * CHUNK_STRIDE + 4 * g);
     const float* y = (wave == 0 ? inverse : M1) + 4 * g * CHUNK_STRIDE + n;
     float4_t m = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -195,7 +219,7 @@ __global__ void __launch_bounds__(256) removal_chunk_prepare_kernel(const Remova
     for (int i = 0; i < 4; ++i) to[(4 * g + i) * CHUNK_STRIDE + n] = m[i];
   }
   __syncthreads();
-  const float4_t t4 = lds4(inverse + n * CHUNK_STRIDE + 4 * g), m4t = lds4(M4T + n * CHUNK_STRIDE + 4 * g);
+  const float4_t t4 = four(inverse + n * CHUNK_STRIDE + 4 * g), m4t = four(M4T + n * CHUNK_STRIDE + 4 * g);
   for (int tile = wave; tile < dim / 16; tile += 4) {  // U' and R', 16 channels at a time
     float4_t up = {0.f, 0.f, 0.f, 0.f}, rp;
 #pragma unroll
@@ -213,7 +237,7 @@ __global__ void __launch_bounds__(256) removal_chunk_prepare_kernel(const Remova
       to[16 * dim + (4 * g + i) * 16] = rp[i];
     }
   }
-  const float4_t m3 = lds4(M3 + n * CHUNK_STRIDE + 4 * g), m4 = lds4(M4 + n * CHUNK_STRIDE + 4 * g), tm1 = lds4(TM1 + n * CHUNK_STRIDE + 4 * g);
+  const float4_t m3 = four(M3 + n * CHUNK_STRIDE + 4 * g), m4 = four(M4 + n * CHUNK_STRIDE + 4 * g), tm1 = four(TM1 + n * CHUNK_STRIDE + 4 * g);
   const int columns = removal_columns(a.vdim);
   float* record_d = record + 65 * dim;
   for (int tile = wave; tile < columns / 16; tile += 4) {  // Dv and Ov, 16 columns of values at a time
@@ -231,97 +255,122 @@ __global__ void __launch_bounds__(256) removal_chunk_prepare_kernel(const Remova
     for (int e = 0; e < 4; ++e) ov = mfma4(-m4[e], dv[e], ov);
     *reinterpret_cast<float4_t*>(record_d + (size_t)column * CHUNK + 4 * g) = dv;
     *reinterpret_cast<float4_t*>(record_d + (size_t)(columns + column) * CHUNK + 4 * g) = ov;
+    *reinterpret_cast<float4_t*>(record_d + (size_t)(2 * columns + column) * CHUNK + 4 * g) = v;
   }
 }
 
 // What a wave reads of one chunk, in registers: loaded SCAN_AHEAD chunks before it is worked.
+template <int WAVES>
 struct RemovalOperands {
-  float4_t up, rp, nb, k, p, dv;
-  float v[4];
+  static constexpr int READS = WAVES >= 4 ? 1 : (4 + WAVES - 1) / WAVES;  // read-outs of a chunk that a lane finishes
+  float4_t up, rp, nb, k, p, dv, v;
+  float ov[READS];
 };
 #define SCAN_AHEAD 4
 
-template <typename T, int WAVES>
-__global__ void __launch_bounds__(64 * WAVES) removal_chunk_scan_kernel(const RemovalChunkArgs a) {
+// (at most 256 registers a wave: the matrix instructions then keep the state in ordinary registers)
+template <int WAVES>
+__global__ void __launch_bounds__(64 * WAVES, 2) removal_chunk_scan_kernel(const RemovalChunkArgs a) {
   __shared__ float4_t parts[2][2][WAVES][64];  // [buffer][D, O][wave][lane]
-  const int tile = blockIdx.x, h = blockIdx.y, b = blockIdx.z;
+  // (heads lie along the grid's first dimension in both kernels: with a multiple of 8 heads the workgroups that read a record run
+  // on the XCD that wrote it and share it in that XCD's L2)
+  const int h = blockIdx.x, tile = blockIdx.y, b = blockIdx.z;
   const int lo = a.cu_q[b], hi = a.cu_q[b + 1];
   if (hi <= lo) return;  // (the whole workgroup)
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int n = lane & 15, g = lane >> 4;
   constexpr int dim = 16 * WAVES;
+  constexpr int READS = RemovalOperands<WAVES>::READS;
   const int vdim = a.vdim, columns = removal_columns(vdim);
   const int column = tile * 16 + n;
   const bool live = column < vdim;
-  const int col = live ? column : vdim - 1;
   const int chunks = (hi - lo + CHUNK - 1) / CHUNK;
   const size_t stride = (size_t)a.heads * removal_record(dim, vdim);  // between a sequence's records of this head
-  const float* records = a.scratch + ((size_t)removal_first_chunk(lo, b) * a.heads + h) * removal_record(dim, vdim);
-  const T* values = (const T*)a.main + (size_t)lo * a.ld + a.v_at + (size_t)h * vdim + col;
-  const int last_row = hi - lo - 1;
-
-  auto load = [&](int c, RemovalOperands& o) {
-    const float* record = records + (size_t)c * stride;
-    const int at = wave * 256 + n * 16 + 4 * g;
-    o.up = lds4(record + at);
-    o.rp = lds4(record + 16 * dim + at);
-    o.nb = lds4(record + 32 * dim + at);
-    o.k = lds4(record + 48 * dim + at);
-    o.p = lds4(record + 64 * dim + wave * 16 + 4 * g);
-    o.dv = lds4(record + 65 * dim + (size_t)column * CHUNK + 4 * g);
+  // a lane's places in a record, in floats (the record's own address is the same for the whole wave and moves from chunk to chunk)
+  const uint32_t rows_at = wave * 256 + n * 16 + 4 * g, decays_at = 64 * dim + wave * 16 + 4 * g, column_at = 65 * dim + column * CHUNK + 4 * g;
+  uint32_t reads_at[READS];
 #pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const int t = c * CHUNK + 4 * g + e;  // (rows beyond the portion follow its last one: their keys are zero)
-      o.v[e] = to_f32(values[(size_t)(t < last_row ? t : last_row) * a.ld]);
-    }
+  for (int q = 0; q < READS; ++q) {
+    const int i = (tid + q * 64 * WAVES) & 255;  // a read-out's place in the order in which the parts lie in LDS
+    reads_at[q] = 65 * dim + (columns + tile * 16 + ((i >> 2) & 15)) * CHUNK + (i >> 6) * 4 + (i & 3);
+  }
+  const float* next = a.scratch + ((size_t)removal_first_chunk(lo, b) * a.heads + h) * removal_record(dim, vdim);
+  int asked = 0;  // chunks asked for so far
+  auto load = [&](RemovalOperands<WAVES>& o) {
+    const float* record = next;
+    o.up = four(record + rows_at);
+    o.rp = four(record + 16 * dim + rows_at);
+    o.nb = four(record + 32 * dim + rows_at);
+    o.k = four(record + 48 * dim + rows_at);
+    o.p = four(record + decays_at);
+    o.dv = four(record + column_at);
+    o.v = four(record + 32 * columns + column_at);
+#pragma unroll
+    for (int q = 0; q < READS; ++q) o.ov[q] = record[reads_at[q]];
+    ++asked;
+    if (asked < chunks) next += stride;  // (beyond the last chunk the last one is asked for again)
   };
 
-  float* S = a.state + (((size_t)a.slots[b] * a.heads + h) * dim + wave * 16 + 4 * g) * vdim + col;
+  float* S = a.state + (((size_t)a.slots[b] * a.heads + h) * dim + wave * 16 + 4 * g) * vdim + (live ? column : vdim - 1);
   float4_t z;
 #pragma unroll
   for (int i = 0; i < 4; ++i) z[i] = S[(size_t)i * vdim];
 
-  RemovalOperands ops[SCAN_AHEAD];
+  const size_t out_row = (size_t)a.heads * vdim;
+  float* out = a.out + (size_t)lo * out_row + (size_t)h * vdim + tile * 16;
+  int left = hi - lo;  // tokens from the current chunk on
+
+  auto work = [&](int buffer, const RemovalOperands<WAVES>& o) {
+    float4_t d = {0.f, 0.f, 0.f, 0.f}, read = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-  for (int c = 0; c < SCAN_AHEAD; ++c)
-    if (c < chunks) load(c, ops[c]);
-  for (int c0 = 0; c0 < chunks; c0 += SCAN_AHEAD) {
+    for (int e = 0; e < 4; ++e) {
+      d = mfma4(o.up[e], z[e], d);
+      read = mfma4(o.rp[e], z[e], read);
+    }
+    parts[buffer][0][wave][lane] = d;
+    parts[buffer][1][wave][lane] = read;
 #pragma unroll
-    for (int j = 0; j < SCAN_AHEAD; ++j) {
-      const int c = c0 + j;
-      if (c >= chunks) break;  // (the same for the whole workgroup)
-      RemovalOperands& o = ops[j];
-      float4_t d = {0.f, 0.f, 0.f, 0.f}, read = {0.f, 0.f, 0.f, 0.f};
+    for (int e = 0; e < 4; ++e) z = mfma4(o.k[e], o.v[e], z);
+    __syncthreads();  // (one a chunk: a buffer is written again behind the next chunk's barrier)
+    d = o.dv;
 #pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        d = mfma4(o.up[e], z[e], d);
-        read = mfma4(o.rp[e], z[e], read);
-      }
-      parts[j & 1][0][wave][lane] = d;
-      parts[j & 1][1][wave][lane] = read;
+    for (int w = 0; w < WAVES; ++w) d += parts[buffer][0][w][lane];
 #pragma unroll
-      for (int e = 0; e < 4; ++e) z = mfma4(o.k[e], o.v[e], z);
-      __syncthreads();  // (one a chunk: a buffer is written again behind the next chunk's barrier)
-      d = o.dv;
+    for (int e = 0; e < 4; ++e) z = mfma4(o.nb[e], d[e], z);
+    z *= o.p;
+    // the chunk's read-outs: 256 of them over the workgroup's lanes
+    const float* sums = reinterpret_cast<const float*>(parts[buffer][1]);
 #pragma unroll
-      for (int w = 0; w < WAVES; ++w) d += parts[j & 1][0][w][lane];
-#pragma unroll
-      for (int e = 0; e < 4; ++e) z = mfma4(o.nb[e], d[e], z);
-      z *= o.p;
-      // the chunk's read-outs: 256 of them over the workgroup's lanes
-      const float* sums = reinterpret_cast<const float*>(parts[j & 1][1]);
-      const float* ov = records + (size_t)c * stride + 65 * dim + (size_t)(columns + tile * 16) * CHUNK;
-      for (int i = tid; i < 256; i += 64 * WAVES) {
-        const int t = (i >> 6) * 4 + (i & 3), e = (i >> 2) & 15;  // (the order in which the parts lie in LDS)
-        float v = ov[e * CHUNK + t];
+    for (int q = 0; q < READS; ++q) {
+      const int i = tid + q * 64 * WAVES;
+      if (i < 256) {
+        const int t = (i >> 6) * 4 + (i & 3), e = (i >> 2) & 15;
+        float v = o.ov[q];
 #pragma unroll
         for (int w = 0; w < WAVES; ++w) v += sums[w * 256 + i];
-        const int token = c * CHUNK + t;
-        if (token <= last_row && tile * 16 + e < vdim) a.out[((size_t)(lo + token) * a.heads + h) * vdim + tile * 16 + e] = v;
+        if (t < left && tile * 16 + e < vdim) out[t * out_row + e] = v;
       }
-      if (c + SCAN_AHEAD < chunks) load(c + SCAN_AHEAD, o);
+    }
+    left -= CHUNK;
+    out += CHUNK * out_row;
+  };
+
+  // Loads are asked for whether or not there is a chunk that far ahead (then the last one's again): the same number of them lies
+  // between a chunk's loads and its work on every path, so that waiting for the one does not wait for the others.
+  RemovalOperands<WAVES> ops[SCAN_AHEAD];
+#pragma unroll
+  for (int j = 0; j < SCAN_AHEAD; ++j) load(ops[j]);
+  int c = 0;
+  for (; c + SCAN_AHEAD <= chunks; c += SCAN_AHEAD) {
+#pragma unroll
+    for (int j = 0; j < SCAN_AHEAD; ++j) {
+      work(j & 1, ops[j]);
+      load(ops[j]);
     }
   }
+#pragma unroll
+  for (int j = 0; j < SCAN_AHEAD - 1; ++j)
+    if (c + j < chunks) work(j & 1, ops[j]);  // (the same for the whole workgroup)
   if (live) {
 #pragma unroll
     for (int i = 0; i < 4; ++i) S[(size_t)i * vdim] = z[i];
@@ -343,16 +392,16 @@ template <typename T>
 static void removal_chunk_launch(const RemovalChunkArgs& a, int num_seqs, int max_q_len, hipStream_t stream) {
   const int chunks = (max_q_len + CHUNK - 1) / CHUNK;
   removal_chunk_prepare_kernel<T><<<dim3(a.heads, chunks, num_seqs), 256, removal_prepare_lds(a.dim, a.rank), stream>>>(a);
-  const dim3 grid(removal_columns(a.vdim) / 16, a.heads, num_seqs);
+  const dim3 grid(a.heads, removal_columns(a.vdim) / 16, num_seqs);
   switch (a.dim / 16) {
-    case 1: removal_chunk_scan_kernel<T, 1><<<grid, 64, 0, stream>>>(a); break;
-    case 2: removal_chunk_scan_kernel<T, 2><<<grid, 128, 0, stream>>>(a); break;
-    case 3: removal_chunk_scan_kernel<T, 3><<<grid, 192, 0, stream>>>(a); break;
-    case 4: removal_chunk_scan_kernel<T, 4><<<grid, 256, 0, stream>>>(a); break;
-    case 5: removal_chunk_scan_kernel<T, 5><<<grid, 320, 0, stream>>>(a); break;
-    case 6: removal_chunk_scan_kernel<T, 6><<<grid, 384, 0, stream>>>(a); break;
-    case 7: removal_chunk_scan_kernel<T, 7><<<grid, 448, 0, stream>>>(a); break;
-    default: removal_chunk_scan_kernel<T, 8><<<grid, 512, 0, stream>>>(a); break;
+    case 1: removal_chunk_scan_kernel<1><<<grid, 64, 0, stream>>>(a); break;
+    case 2: removal_chunk_scan_kernel<2><<<grid, 128, 0, stream>>>(a); break;
+    case 3: removal_chunk_scan_kernel<3><<<grid, 192, 0, stream>>>(a); break;
+    case 4: removal_chunk_scan_kernel<4><<<grid, 256, 0, stream>>>(a); break;
+    case 5: removal_chunk_scan_kernel<5><<<grid, 320, 0, stream>>>(a); break;
+    case 6: removal_chunk_scan_kernel<6><<<grid, 384, 0, stream>>>(a); break;
+    case 7: removal_chunk_scan_kernel<7><<<grid, 448, 0, stream>>>(a); break;
+    default: removal_chunk_scan_kernel<8><<<grid, 512, 0, stream>>>(a); break;
   }
 }
 
