@@ -1,4 +1,4 @@
-// gated_scan: a recurrence on every channel by itself, S_t = (1 - z_t) S_(t-1) + z_t c_t, whose gates read only the current token.
+// gated_scan: a recurrence on every channel by itself, S_t = (1 - z_t) S_(t-1) + z_t c_t, with gates that do not depend on the state.
 //   A row of `proj` holds z, u and g, `width` channels each:  z = sigmoid(proj_z + bias_z);  u = proj_u + bias_u;
 //   c = u + shift (u >= 0) or sigmoid(u) (u < 0);  out[t] = S_t * silu(g).  The state is float32 [slots, width].
 // Everything between a load and a store is float32.

@@ -9,11 +9,11 @@ of its own.  Three types of mixer, each with any of the feed-forwards:
     the generalized delta rule: a matrix per head with a decay and a removal rate per key channel, which removes what
     it holds along the key's direction and writes the key itself (``parts.linear_recurrence.GeneralDeltaMixer``).
 ``mingru``
-    a gated recurrence on every channel by itself whose gates read only the current token (``parts.gated_recurrence``).
+    a gated recurrence on every channel by itself with gates that do not depend on the state (``parts.gated_recurrence``).
 ``attention``
     grouped-query softmax attention over a sliding window whose values are the keys as projected, with a rotation of the
     first ``rot.dims`` channels, queries and keys divided by their root mean square behind the rotation, the score scale of
-    the configuration and one added to the softmax's denominator (``parts.conv_attention``).
+    the configuration and a silent key of score 0 in every softmax (``parts.conv_attention``).
 
 The feed-forward is ``W_down polynorm(W_up h)`` (``dense``), a mixture of gated SiLU experts whose weights are the softmax over the
 chosen logits (``moe``), or absent.

@@ -1,5 +1,5 @@
-"""Recurrences that work on every channel by itself: ``S_t = (1 - z_t) S_(t-1) + z_t c_t``, gates that read only the current
-token (a minimal gated recurrent unit).
+"""Recurrences that work on every channel by itself: ``S_t = (1 - z_t) S_(t-1) + z_t c_t``, with gates that do not
+depend on the state (a minimal gated recurrent unit).
 
 ``z = sigmoid(W_z x + b_z)`` and ``u = W_x x + b_x``, both of ``width`` channels; the candidate ``c`` is ``u + shift`` where ``u >= 0`` and
 ``sigmoid(u)`` where ``u < 0`` (continuous at 0 for a shift of 1/2, and positive everywhere); the output is
