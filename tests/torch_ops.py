@@ -146,13 +146,15 @@ class TorchOps:
             act = 0.5 * gate * (1.0 + torch.tanh(0.7978845608028654 * (gate + 0.044715 * gate * gate * gate)))
         elif activation == "silu":
             act = gate * torch.sigmoid(gate)
+        elif activation == "relu":
+            act = torch.relu(gate)
         else:
             raise ValueError(activation)
         return (act * up).to(gate_up.dtype)
 
     # -- short convolution, recurrences -------------------------------------------------------
-    def short_conv(self, x, channels, weight, tail, slots, cu_q, max_q_len, activation="none", update_state=True):
-        """``x`` [T, >= channels]: the first ``channels`` columns pass ``y_t = sum_j w[:, j] u_(t - taps + 1 + j)`` per sequence,
+    def short_conv(self, x, channels, weight, tail, slots, cu_q, max_q_len, activation="none", update_state=True, first=0, bias=None):
+        """``x`` [T, >= first + channels]: ``channels`` columns from ``first`` on pass ``y_t = sum_j w[:, j] u_(t - taps + 1 + j)`` per sequence,
         the inputs before a portion's start come from ``tail[slot]`` ([taps - 1, channels], oldest first), which is then
         brought up to date.  Returns [T, channels] in x's dtype."""
         taps = weight.shape[1]
@@ -160,11 +162,13 @@ class TorchOps:
         bounds = cu_q.tolist()
         for b, slot in enumerate(slots.tolist()):
             lo, hi = bounds[b], bounds[b + 1]
-            u = x[lo:hi, :channels].float()
+            u = x[lo:hi, first:first + channels].float()
             if taps > 1:
                 before = tail[slot].float() if tail is not None else torch.zeros((taps - 1, channels), device=x.device)
                 u = torch.cat([before, u], 0)
             y = sum(weight[:, j].float() * u[j:j + hi - lo] for j in range(taps))
+            if bias is not None:
+                y = y + bias
             if activation == "silu":
                 y = y * torch.sigmoid(y)
             out[lo:hi] = y.to(x.dtype)
@@ -288,6 +292,33 @@ class TorchOps:
             state[slot] = s
         return out.view(t, heads * vdim)
 
+    def state_space_scan(self, xbc, step_source, step_at, dt_bias, rate, skip, state, slots, cu_q, max_q_len, heads, groups, size, vdim):
+        """``xbc`` [T, heads * vdim + 2 * groups * size] = x, B, C; ``d = softplus(dt + dt_bias)``; per head, from ``state[slot, head]``
+        ([size, vdim] float32), which is written back: ``S <- exp(-rate d) S + d B x^T``, ``y = S^T C + skip x``.  float32 [T, heads * vdim]."""
+        t = xbc.shape[0]
+        inner, gn = heads * vdim, groups * size
+        x = xbc[:, :inner].float().view(t, heads, vdim)
+        b, c = (xbc[:, at:at + gn].float().view(t, groups, size).repeat_interleave(heads // groups, 1) for at in (inner, inner + gn))
+        step = torch.nn.functional.softplus(step_source[:, step_at:step_at + heads].float() + dt_bias, threshold=60.0)
+        decay = torch.exp(-rate * step)
+        out = torch.empty((t, heads, vdim), dtype=torch.float32, device=xbc.device)
+        bounds = cu_q.tolist()
+        for n, slot in enumerate(slots.tolist()):
+            s = state[slot].clone()
+            for i in range(bounds[n], bounds[n + 1]):
+                s = decay[i][:, None, None] * s + (step[i][:, None] * b[i])[:, :, None] * x[i][:, None, :]
+                out[i] = (s * c[i][:, :, None]).sum(1) + skip[:, None] * x[i]
+            state[slot] = s
+        return out.view(t, inner)
+
+    def gated_group_norm(self, read, gate_source, gate_at, weight, eps, groups, out_dtype):
+        """``y = read * silu(gate)``; each of ``groups`` equal parts of a row over its root mean square, times ``weight``."""
+        t, width = read.shape
+        z = gate_source[:, gate_at:gate_at + width].float()
+        y = (read * (z * torch.sigmoid(z))).view(t, groups, width // groups)
+        y = y / torch.sqrt((y * y).mean(-1, keepdim=True) + eps)
+        return (y.view(t, width) * weight).to(out_dtype)
+
     def gated_head_norm(self, read, weight, eps, gate_source, gate_at, gate_kind, heads, vdim, out_dtype):
         t = read.shape[0]
         o = read.view(t, heads, vdim)
@@ -298,8 +329,17 @@ class TorchOps:
 
     @staticmethod
     def _one_delta(delta):
-        from velox_amd.parts.base import SumOf
+        from velox_amd.parts.base import NormedSum, SumOf
 
+        def whole(y):
+            return y.float().sum(0) if y.dim() == 3 else y.float()
+
+        if isinstance(delta, NormedSum):
+            total = 0.0
+            for y, weight, scale in zip(delta.terms, delta.weights, delta.scales):
+                y = whole(y)
+                total = total + scale * (y / torch.sqrt((y * y).mean(-1, keepdim=True) + delta.eps) * weight)
+            return total if delta.plain is None else total + whole(delta.plain)
         if isinstance(delta, SumOf):
             first = delta.first.float().sum(0) if delta.first.dim() == 3 else delta.first.float()
             return first + delta.second.float()
@@ -323,6 +363,27 @@ class TorchOps:
             x = x + delta[rows.long()].float()
         var = (x * x).sum(-1, keepdim=True) / x.shape[-1]
         return (x * torch.rsqrt(var + eps) * weight.float()).to(out_dtype)
+
+    def normed_sum_norm(self, residual, delta, weight, eps, out_dtype, rows=None):
+        if rows is None:
+            return self.add_rmsnorm(residual, delta, weight, eps, out_dtype)
+        return self.add_rmsnorm_rows(residual, delta, rows, weight, eps, out_dtype)
+
+    def join_rows(self, residual, delta, start, out_dtype):
+        """``[residual + delta ; start]`` in ``out_dtype``, [T, 2 H]; the residual is cleared."""
+        delta = self._one_delta(delta)
+        if delta is not None and delta.dim() == 3:
+            delta = delta.float().sum(0)
+        x = residual if delta is None else residual + delta.float()
+        out = torch.cat([x.to(out_dtype), start.to(out_dtype)], dim=-1)
+        residual.zero_()
+        return out
+
+    def kept_copy(self, x, dtype):
+        return x.to(dtype).clone()
+
+    def softcap_(self, x, cap, scale=1.0):
+        return x.mul_(scale).div_(cap).tanh_().mul_(cap)
 
     def add_sinusoid(self, hidden, positions, frequencies):
         """hidden[t, 2i] += sin(p_t f_i), hidden[t, 2i + 1] += cos(p_t f_i), in place."""
@@ -568,9 +629,11 @@ class TorchOps:
 
     # -- attention over the paged cache -------------------------------------------------
     def paged_attention(self, qkv, num_heads, num_kv_heads, head_dim, k_cache, v_cache, block_size, block_tables, cu_q, kv_lens, max_q_len, max_kv_len, scale, window, all_decode, workspace, splits=None, decode_prefix=0, portions_max_kv_len=None,
-                        distance_bias=None, sinks=None):
+                        distance_bias=None, sinks=None, keep_first=0, softcap=None, gate=None):
         """``distance_bias``: float32 [heads, L]; the score of a key ``n`` behind the query gets column ``min(n, L - 1)``.
-        ``sinks``: float32 [heads]; ``exp(sinks[h])`` joins the denominator of every row of head ``h``."""
+        ``sinks``: float32 [heads]; ``exp(sinks[h])`` joins the denominator of every row of head ``h``.  ``keep_first``: tokens that a
+        window keeps.  ``softcap``: the scaled score becomes ``softcap * tanh(s / softcap)``.  ``gate = (source, first column, channels
+        per head or 0)``: a head's output times ``sigmoid`` of its columns (of its one column)."""
         t = qkv.shape[0]
         group = num_heads // num_kv_heads
         q_all = qkv[:, : num_heads * head_dim].view(t, num_heads, head_dim)
@@ -589,10 +652,12 @@ class TorchOps:
             q_pos = ctx + torch.arange(q_len, device=qkv.device)
             keep = q_pos[:, None] >= index[None, :]
             if window is not None:
-                keep &= index[None, :] > q_pos[:, None] - window
+                keep &= (index[None, :] > q_pos[:, None] - window) | (index[None, :] < keep_first)
             for h in range(num_heads):
                 kv = h // group
                 scores = (q_all[lo:hi, h].float() @ keys[:, kv].T) * scale
+                if softcap is not None:
+                    scores = softcap * torch.tanh(scores / softcap)
                 if distance_bias is not None:
                     behind = (q_pos[:, None] - index[None, :]).clamp(min=0, max=distance_bias.shape[1] - 1)
                     scores = scores + distance_bias[h].float()[behind]
@@ -604,6 +669,12 @@ class TorchOps:
                     denom = denom + torch.exp(sinks[h].float() - m)
                 p = p.to(qkv.dtype).float()  # the kernel rounds p to the value dtype for the second product
                 out[lo:hi, h] = (p @ values[:, kv]) / denom
+        if gate is not None:
+            source, at, channels = gate
+            if channels == 0:
+                out *= torch.sigmoid(source[:, at:at + num_heads].float())[:, :, None]
+            else:
+                out[:, :, :channels] *= torch.sigmoid(source[:, at:at + num_heads * channels].float()).view(t, num_heads, channels)
         return out.to(qkv.dtype).view(t, num_heads * head_dim)
 
     # -- sampling -----------------------------------------------------------------------

@@ -5,7 +5,8 @@ or nothing).  Entries with equal paged needs form a *group*: one pool of pages, 
 allocator, one block table per request; page ``p`` of a group addresses page ``p`` of
 every entry in it (the reference has exactly one such group for all layers,
 ``src/paged_kv_cache.py:51-55``).  A group whose need has a window gives pages back as soon
-as every key in them lies behind the window of all queries still to come.  Entries with
+as every key in them lies behind the window of all queries still to come, except those that
+hold the first tokens a need keeps (``PagedNeed.keep_first``).  Entries with
 a ``StateNeed`` get one row per request in fixed-size tensors, indexed by the request's
 *slot* (the reference's ``seq_index``, ``engine/scheduler.py:58,113-129``); slot rows are zeroed
 when a request takes the slot.  An entry may state several needs at once (``CompositeNeed``: pages
@@ -94,6 +95,10 @@ class PageGroup:
             return 0
         first_key = max(0, num_computed - self.need.window + 1)
         return first_key // self.page_size
+
+    def kept_pages(self) -> int:
+        """Leading table entries that hold tokens every query reads, however far behind its window."""
+        return self.table_entries_for(self.need.keep_first) if self.need.window is not None else 0
 
 
 class StateSlots:
@@ -332,7 +337,7 @@ class CacheManager:
         for index, group in enumerate(self.groups):
             first = min(group.first_needed_page(num_computed), len(seq.tables[index]))
             table = seq.tables[index]
-            for position in range(seq.released[index], first):
+            for position in range(max(seq.released[index], group.kept_pages()), first):
                 if table[position] != NULL_PAGE:
                     group.allocator.drop(table[position])
                     table[position] = NULL_PAGE

@@ -39,6 +39,34 @@ constexpr int D = VELOX_HEAD_DIM;
 #define VELOX_ATTN_BIAS 0
 #endif
 constexpr bool BIASED = VELOX_ATTN_BIAS != 0;
+
+// Further builds, each a flag of its own; without it the part of `Extras` that it reads is ignored and the code is what it is
+// without it:
+//   VELOX_ATTN_KEEP  a window keeps the first keys of the sequence: key n is seen iff n <= position and (n > position - window
+//                    or n < keep_first).  The tiles that hold the kept keys come before the window's, unless the two meet.
+//   VELOX_ATTN_CAP   scores pass softcap * tanh(score / softcap) behind the scale (and before a bias)
+//   VELOX_ATTN_GATE  a head's output is multiplied by sigmoid(gate), one number per head or one per channel, where its row
+//                    is finished: in the kernels' last lines, or in the merge when its keys are split
+#ifndef VELOX_ATTN_KEEP
+#define VELOX_ATTN_KEEP 0
+#endif
+#ifndef VELOX_ATTN_CAP
+#define VELOX_ATTN_CAP 0
+#endif
+#ifndef VELOX_ATTN_GATE
+#define VELOX_ATTN_GATE 0
+#endif
+constexpr bool KEEPS = VELOX_ATTN_KEEP != 0, CAPPED = VELOX_ATTN_CAP != 0, GATED = VELOX_ATTN_GATE != 0;
+
+struct Extras {
+  int keep_first;       // keys every query sees, whatever its window
+  float softcap;
+  const void* gate;     // rows of the run's type, one per token like the output's, gate_stride elements apart
+  int gate_stride;
+  int gate_channels;    // 0: a row holds one number per head; else this many per head (channels beyond are not multiplied)
+  int gate_by_four;     // four neighbouring channels of a head can be read with one aligned access
+};
+
 static_assert(D % 16 == 0 && D >= 16 && D <= 256, "head size must be a multiple of 16 between 16 and 256");
 
 template <typename T> struct Frag;
@@ -136,7 +164,78 @@ template <> struct Softmax<bf16_t> {
   static __device__ __forceinline__ float exp_of(float x) { return __builtin_amdgcn_exp2f(x); }
 };
 
+// A score behind the cap, in the exponent's unit: cap * tanh(x / cap).
+template <typename T> struct Cap {
+  float in, out;
+  __device__ __forceinline__ Cap(float scale, float cap) : in(scale / cap), out(cap * Softmax<T>::SCALE) {}
+  __device__ __forceinline__ float operator()(float raw) const {
+    const float x = raw * in;
+    if constexpr (sizeof(T) == 4) return out * tanhf(x);
+    // 1 - 2 / (e^2x + 1) with the hardware's exponential and reciprocal; either end goes to its limit
+    const float e = __builtin_amdgcn_exp2f(x * 2.88539008177792681472f);
+    return out * (1.f - 2.f * __builtin_amdgcn_rcpf(e + 1.f));
+  }
+};
+
+// The gate's factor of channels c .. c + 3 of a head in a token's row.
+template <typename T> __device__ __forceinline__ float4_t gate_of(const Extras& x, size_t token, int head, int c) {
+  const T* row = (const T*)x.gate + token * x.gate_stride;
+  auto sigmoid = [](float z) { return 1.f / (1.f + expf(-z)); };
+  if (x.gate_channels == 0) {
+    const float one = sigmoid(to_f32(row[head]));
+    return float4_t{one, one, one, one};
+  }
+  float4_t out = float4_t{1.f, 1.f, 1.f, 1.f};
+  const T* from = row + (size_t)head * x.gate_channels + c;
+  if (x.gate_by_four && c + 4 <= x.gate_channels) {
+    const Frag<T> f = load_frag<T>(from);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      if constexpr (sizeof(T) == 4) out[j] = sigmoid(f.v[j]);
+      else out[j] = sigmoid(__uint_as_float(((uint32_t)(uint16_t)f.v[j]) << 16));
+    }
+  } else {
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (c + j < x.gate_channels) out[j] = sigmoid(to_f32(from[j]));
+  }
+  return out;
+}
+
+// Where the tiles of keys of a row block lie.  Without kept keys tile t starts at key n_begin + t * BN.  With a window and kept
+// keys the first `kept_tiles` tiles are those of keys 0 .. keep_first - 1 and the window's follow; when the two meet there is
+// one run of tiles from key 0.  Page ids are kept in one array, the kept tiles' first.
+struct KeyTiles {
+  int n_begin, kept_tiles, kept_end, kept_pages;
+  template <int BN> __device__ __forceinline__ static KeyTiles of(int first_visible, int window, int keep_first, int page_shift) {
+    KeyTiles k{0, 0, 0, 0};
+    if (window > 0) k.n_begin = (first_visible < 0 ? 0 : first_visible) / BN * BN;
+    if constexpr (KEEPS) {
+      if (k.n_begin > 0) {
+        k.kept_tiles = (keep_first + BN - 1) / BN;
+        if (k.n_begin <= k.kept_tiles * BN) {
+          k.n_begin = 0;
+          k.kept_tiles = 0;
+        }
+        k.kept_end = k.kept_tiles * BN;
+        k.kept_pages = (k.kept_end + (1 << page_shift) - 1) >> page_shift;
+      }
+    }
+    return k;
+  }
+  template <int BN> __device__ __forceinline__ int first_key(int tile) const {
+    if constexpr (KEEPS) return tile < kept_tiles ? tile * BN : n_begin + (tile - kept_tiles) * BN;
+    return n_begin + tile * BN;
+  }
+  // place of key n's page id in the array, `first_page` being the window part's first page there
+  __device__ __forceinline__ int id_at(int n, int page_shift, int first_page) const {
+    if constexpr (KEEPS) return (n >> page_shift) + (n < kept_end ? 0 : kept_pages - first_page);
+    return (n >> page_shift) - first_page;
+  }
+};
+
 constexpr int PREFILL_PAGE_IDS = 2048;
+constexpr int KEPT_PAGE_IDS = 1024;  // of them, the most that kept keys may take (checked by the launcher)
 // two waves per SIMD hide each other's waits; up to head size 128 the registers allow it without spilling, and the
 // compiler is held to it (left alone it takes more registers than one wave per SIMD's worth buys back)
 constexpr int GENERAL_MIN_WAVES = D <= 128 ? 2 : 1;
@@ -153,7 +252,7 @@ __global__ void __launch_bounds__(64 * WAVES * KSPLIT) __attribute__((amdgpu_wav
     const int* __restrict__ block_tables, int table_width, const int* __restrict__ cu_q, const int* __restrict__ kv_lens,
     T* __restrict__ out, float* __restrict__ part_o, float* __restrict__ part_lse,
     int nh, int nkv, int page_shift, float scale, int window, int splits, int total_tokens, const float* __restrict__ bias_table, int bias_len,
-    const float* __restrict__ sinks) {
+    const float* __restrict__ sinks, const Extras extras) {
   typedef Block<T> B;
   typedef typename B::Operand Operand;
   constexpr int KB = B::KB;
@@ -220,13 +319,9 @@ __global__ void __launch_bounds__(64 * WAVES * KSPLIT) __attribute__((amdgpu_wav
   const int last_tok = last_row / group;
   int n_end = ctx + last_tok + 1;
   if (n_end > kv_len) n_end = kv_len;
-  int n_begin = 0;
-  if (window > 0) {
-    n_begin = ctx + first_tok - window + 1;
-    if (n_begin < 0) n_begin = 0;
-    n_begin = n_begin / BN * BN;
-  }
-  const int tiles_total = (n_end - n_begin + BN - 1) / BN;
+  const KeyTiles keys = KeyTiles::of<BN>(ctx + first_tok - window + 1, window, extras.keep_first, page_shift);
+  const int n_begin = keys.n_begin;
+  const int tiles_total = keys.kept_tiles + (n_end - n_begin + BN - 1) / BN;
   const int tiles_per_split = (tiles_total + splits - 1) / splits;
   const int tile_lo = split * tiles_per_split;
   int tile_hi = tile_lo + tiles_per_split;
@@ -250,18 +345,23 @@ __global__ void __launch_bounds__(64 * WAVES * KSPLIT) __attribute__((amdgpu_wav
   // Page ids of the keys this workgroup visits are kept in LDS, a window of PREFILL_PAGE_IDS pages at a time (the tile
   // loop moves the window on when the next tile would leave it); zeros go to the padding columns of the K tile.
   const int* table = block_tables + (size_t)b * table_width;
-  const int last_key = n_begin + tile_hi * BN < kv_len ? n_begin + tile_hi * BN : kv_len;
+  const int keys_end = keys.first_key<BN>(tile_hi - 1) + BN;
+  const int last_key = keys_end < kv_len ? keys_end : kv_len;
   const int last_page = tile_hi > tile_lo ? (last_key - 1) >> page_shift : -1;
-  int first_page = (n_begin + tile_lo * BN) >> page_shift;  // first page of the window
+  const int kept_pages = KEEPS ? keys.kept_pages : 0;
+  int first_page = keys.first_key<BN>(tile_lo > keys.kept_tiles ? tile_lo : keys.kept_tiles) >> page_shift;  // first page of the window
   auto load_page_ids = [&]() {
     const int num_pages = last_page - first_page + 1;
-    for (int p = threadIdx.x; p < num_pages && p < PREFILL_PAGE_IDS; p += SETW * KSPLIT) page_ids[p] = table[first_page + p];
+    for (int p = threadIdx.x; p < num_pages && p < PREFILL_PAGE_IDS - kept_pages; p += SETW * KSPLIT) page_ids[kept_pages + p] = table[first_page + p];
   };
+  if constexpr (KEEPS) {
+    for (int p = threadIdx.x; p < kept_pages && p < KEPT_PAGE_IDS; p += SETW * KSPLIT) page_ids[p] = table[p];
+  }
   load_page_ids();
   if constexpr (DP > D) {
     for (int e = tid; e < BN * (DP - D); e += SETW) k_tile[(e / (DP - D)) * KS + D + e % (DP - D)] = from_f32<T>(0.f);
   }
-  auto page_of = [&](int n) -> size_t { return (size_t)page_ids[(n >> page_shift) - first_page]; };
+  auto page_of = [&](int n) -> size_t { return (size_t)page_ids[keys.id_at(n, page_shift, first_page)]; };
 
   Operand qf[CT][NQB];
   float m_i[CT], l_i[CT];
@@ -280,7 +380,8 @@ __global__ void __launch_bounds__(64 * WAVES * KSPLIT) __attribute__((amdgpu_wav
     for (int c = 0; c < NC; ++c) acc_o[ct][c] = float4_t{0.f, 0.f, 0.f, 0.f};
   }
   const float scale_eff = scale * Softmax<T>::SCALE;
-  const float scale_used = BIASED ? 1.f : scale_eff;  // (with a bias the scores are scaled where it is added)
+  const float scale_used = BIASED || CAPPED ? 1.f : scale_eff;  // (with a cap or a bias the scores are scaled where it is applied)
+  const Cap<T> cap(scale, CAPPED ? extras.softcap : 1.f);
 
   // ---- staging: global -> registers (issued a tile ahead) -> LDS; what does not change from tile to tile is computed once
   constexpr int VPR = D / VEC;              // vectors per key row of K
@@ -377,22 +478,23 @@ __global__ void __launch_bounds__(64 * WAVES * KSPLIT) __attribute__((amdgpu_wav
   __syncthreads();  // page ids are in place
   // iteration `it` covers tiles tile_lo + it * KSPLIT .. + KSPLIT - 1, one per set (the last iteration may leave a set without one)
   const int iterations = tile_hi > tile_lo ? (tile_hi - tile_lo + KSPLIT - 1) / KSPLIT : 0;
-  if (tile_lo + set < tile_hi) fetch(n_begin + (tile_lo + set) * BN);
+  if (tile_lo + set < tile_hi) fetch(keys.first_key<BN>(tile_lo + set));
   for (int it = 0; it < iterations; ++it) {
     const int tile = tile_lo + it * KSPLIT + set;
     const bool have_tile = KSPLIT == 1 || tile < tile_hi;
-    const int n0 = n_begin + tile * BN;
+    const int n0 = keys.first_key<BN>(tile);
     __syncthreads();  // the previous tile has been read by every wave
     if (have_tile) commit(n0);
     __syncthreads();
     if (it + 1 < iterations) {
-      const int next_first = n_begin + (tile_lo + (it + 1) * KSPLIT) * BN;  // first key of the next iteration's tiles
-      if (((next_first + KSPLIT * BN - 1) >> page_shift) - first_page >= PREFILL_PAGE_IDS) {  // the same for every thread
-        first_page = next_first >> page_shift;
+      const int next_tile = tile_lo + (it + 1) * KSPLIT;  // first of the next iteration's tiles
+      const int next_last = keys.first_key<BN>(next_tile + KSPLIT - 1) + BN - 1;
+      if ((next_last >> page_shift) - first_page >= PREFILL_PAGE_IDS - kept_pages) {  // the same for every thread
+        first_page = keys.first_key<BN>(next_tile > keys.kept_tiles ? next_tile : keys.kept_tiles) >> page_shift;
         load_page_ids();
         __syncthreads();
       }
-      if (tile + KSPLIT < tile_hi) fetch(n0 + KSPLIT * BN);  // in flight while this tile is computed
+      if (tile + KSPLIT < tile_hi) fetch(keys.first_key<BN>(tile + KSPLIT));  // in flight while this tile is computed
     }
     if (!have_tile || n0 > wave_last_pos) continue;  // nothing this wave may read; it still took part in the staging
 
@@ -427,7 +529,15 @@ __global__ void __launch_bounds__(64 * WAVES * KSPLIT) __attribute__((amdgpu_wav
       }
     }
     // ---- scale, mask (only where the tile crosses a row's limits), running maximum ----------
-    const bool whole = n0 + BN <= kv_len && n0 + BN - 1 <= wave_first_pos && (window <= 0 || n0 > wave_last_pos - window);
+    const bool whole = n0 + BN <= kv_len && n0 + BN - 1 <= wave_first_pos && (window <= 0 || n0 > wave_last_pos - window || (KEEPS && n0 + BN <= extras.keep_first));
+    if constexpr (CAPPED) {
+#pragma unroll
+      for (int ct = 0; ct < CT; ++ct)
+#pragma unroll
+        for (int t = 0; t < NT; ++t)
+#pragma unroll
+          for (int j = 0; j < 4; ++j) s[ct][t][j] = cap(s[ct][t][j]);
+    }
     if constexpr (BIASED) {
       // the scores take their final form here (scaled, in the exponent's unit, bias added); a tile that lies wholly
       // in the last column's reach gets one number per row
@@ -440,7 +550,7 @@ __global__ void __launch_bounds__(64 * WAVES * KSPLIT) __attribute__((amdgpu_wav
 #pragma unroll
           for (int t = 0; t < NT; ++t)
 #pragma unroll
-            for (int j = 0; j < 4; ++j) s[ct][t][j] = fmaf(s[ct][t][j], scale_eff, c);
+            for (int j = 0; j < 4; ++j) s[ct][t][j] = fmaf(s[ct][t][j], CAPPED ? 1.f : scale_eff, c);
         } else {
 #pragma unroll
           for (int t = 0; t < NT; ++t)
@@ -448,7 +558,7 @@ __global__ void __launch_bounds__(64 * WAVES * KSPLIT) __attribute__((amdgpu_wav
             for (int j = 0; j < 4; ++j) {
               int d = d0 - (16 * t + 4 * g + j);
               d = d < 0 ? 0 : (d > bias_len - 1 ? bias_len - 1 : d);
-              s[ct][t][j] = fmaf(s[ct][t][j], scale_eff, tab[d] * Softmax<T>::SCALE);
+              s[ct][t][j] = fmaf(s[ct][t][j], CAPPED ? 1.f : scale_eff, tab[d] * Softmax<T>::SCALE);
             }
         }
       }
@@ -470,7 +580,7 @@ __global__ void __launch_bounds__(64 * WAVES * KSPLIT) __attribute__((amdgpu_wav
 #pragma unroll
           for (int j = 0; j < 4; ++j) {
             const int n = n0 + 16 * t + 4 * g + j;
-            const bool keep = row_ok[ct] && n < kv_len && n <= pos[ct] && (window <= 0 || n > pos[ct] - window);
+            const bool keep = row_ok[ct] && n < kv_len && n <= pos[ct] && (window <= 0 || n > pos[ct] - window || (KEEPS && n < extras.keep_first));
             s[ct][t][j] = keep ? s[ct][t][j] : -INFINITY;
             mx = fmaxf(mx, s[ct][t][j]);
           }
@@ -570,8 +680,10 @@ __global__ void __launch_bounds__(64 * WAVES * KSPLIT) __attribute__((amdgpu_wav
       T* dst = out + (token * nh + head[ct]) * D + 4 * g;
 #pragma unroll
       for (int c = 0; c < NC; ++c) {
+        float4_t o = acc_o[ct][c] * inv;
+        if constexpr (GATED) o = o * gate_of<T>(extras, token, head[ct], 16 * c + 4 * g);
 #pragma unroll
-        for (int j = 0; j < 4; ++j) dst[16 * c + j] = from_f32<T>(acc_o[ct][c][j] * inv);
+        for (int j = 0; j < 4; ++j) dst[16 * c + j] = from_f32<T>(o[j]);
       }
     } else {
       const size_t slot = ((size_t)split * total_tokens + token) * nh + head[ct];
@@ -614,7 +726,7 @@ __global__ void __launch_bounds__(64 * WAVES * KSPLIT) __attribute__((amdgpu_wav
     const int* __restrict__ block_tables, int table_width, const int* __restrict__ cu_q, const int* __restrict__ kv_lens,
     bf16_t* __restrict__ out, float* __restrict__ part_o, float* __restrict__ part_lse,
     int nh, int nkv, int page_shift, float scale, int window, int splits, int total_tokens, const float* __restrict__ bias_table, int bias_len,
-    const float* __restrict__ sinks) {
+    const float* __restrict__ sinks, const Extras extras) {
   typedef bf16_t T;
   typedef Block<T> B;
   typedef typename B::Operand Operand;
@@ -672,13 +784,9 @@ __global__ void __launch_bounds__(64 * WAVES * KSPLIT) __attribute__((amdgpu_wav
   const int last_tok = last_row / group;
   int n_end = ctx + last_tok + 1;
   if (n_end > kv_len) n_end = kv_len;
-  int n_begin = 0;
-  if (window > 0) {
-    n_begin = ctx + first_tok - window + 1;
-    if (n_begin < 0) n_begin = 0;
-    n_begin = n_begin / BN * BN;
-  }
-  const int tiles_total = (n_end - n_begin + BN - 1) / BN;
+  const KeyTiles keys = KeyTiles::of<BN>(ctx + first_tok - window + 1, window, extras.keep_first, page_shift);
+  const int n_begin = keys.n_begin;
+  const int tiles_total = keys.kept_tiles + (n_end - n_begin + BN - 1) / BN;
   const int tiles_per_split = (tiles_total + splits - 1) / splits;
   const int tile_lo = split * tiles_per_split;
   int tile_hi = tile_lo + tiles_per_split;
@@ -700,15 +808,20 @@ __global__ void __launch_bounds__(64 * WAVES * KSPLIT) __attribute__((amdgpu_wav
 
   // page ids of the keys this workgroup visits, a window of PREFILL_PAGE_IDS pages at a time
   const int* table = block_tables + (size_t)b * table_width;
-  const int last_key = n_begin + tile_hi * BN < kv_len ? n_begin + tile_hi * BN : kv_len;
+  const int keys_end = keys.first_key<BN>(tile_hi - 1) + BN;
+  const int last_key = keys_end < kv_len ? keys_end : kv_len;
   const int last_page = tile_hi > tile_lo ? (last_key - 1) >> page_shift : -1;
-  int first_page = (n_begin + tile_lo * BN) >> page_shift;
+  const int kept_pages = KEEPS ? keys.kept_pages : 0;
+  int first_page = keys.first_key<BN>(tile_lo > keys.kept_tiles ? tile_lo : keys.kept_tiles) >> page_shift;
   auto load_page_ids = [&]() {
     const int num_pages = last_page - first_page + 1;
-    for (int p = threadIdx.x; p < num_pages && p < PREFILL_PAGE_IDS; p += SETW * KSPLIT) page_ids[p] = table[first_page + p];
+    for (int p = threadIdx.x; p < num_pages && p < PREFILL_PAGE_IDS - kept_pages; p += SETW * KSPLIT) page_ids[kept_pages + p] = table[first_page + p];
   };
+  if constexpr (KEEPS) {
+    for (int p = threadIdx.x; p < kept_pages && p < KEPT_PAGE_IDS; p += SETW * KSPLIT) page_ids[p] = table[p];
+  }
   load_page_ids();
-  auto page_of = [&](int n) -> size_t { return (size_t)page_ids[(n >> page_shift) - first_page]; };
+  auto page_of = [&](int n) -> size_t { return (size_t)page_ids[keys.id_at(n, page_shift, first_page)]; };
 
   Operand qf[CT][NQB];
   float m_i[CT], l_i[CT];
@@ -725,7 +838,8 @@ __global__ void __launch_bounds__(64 * WAVES * KSPLIT) __attribute__((amdgpu_wav
     for (int c = 0; c < NC; ++c) acc_o[ct][c] = float4_t{0.f, 0.f, 0.f, 0.f};
   }
   const float scale_eff = scale * Softmax<T>::SCALE;
-  const float scale_used = BIASED ? 1.f : scale_eff;  // (with a bias the scores are scaled where it is added)
+  const float scale_used = BIASED || CAPPED ? 1.f : scale_eff;  // (with a cap or a bias the scores are scaled where it is applied)
+  const Cap<T> cap(scale, CAPPED ? extras.softcap : 1.f);
 
   // ---- what each lane asks for: load instruction q = wave + WAVES * m of a tile fills bytes [1024 q, 1024 q + 1024) of
   // the K part (or the V^T part) of a buffer; lane l's 16 bytes are piece s = 64 q + l of the tile
@@ -763,7 +877,7 @@ __global__ void __launch_bounds__(64 * WAVES * KSPLIT) __attribute__((amdgpu_wav
       size_t k_page[LPW];
 #pragma unroll
       for (int m = 0; m < LPW; ++m)
-        k_page[m] = (size_t)__builtin_amdgcn_readfirstlane(page_ids[((n0 + KEYS_PER_LOAD * (wave + WAVES * m)) >> page_shift) - window_first]);
+        k_page[m] = (size_t)__builtin_amdgcn_readfirstlane(page_ids[keys.id_at(n0 + KEYS_PER_LOAD * (wave + WAVES * m), page_shift, window_first)]);
 #pragma unroll
       for (int m = 0; m < LPW; ++m) {
         const int key0 = n0 + KEYS_PER_LOAD * (wave + WAVES * m);
@@ -810,27 +924,28 @@ __global__ void __launch_bounds__(64 * WAVES * KSPLIT) __attribute__((amdgpu_wav
   __syncthreads();  // page ids are in place
   // round `it` covers tiles tile_lo + it * KSPLIT .. + KSPLIT - 1, one per set (the last round may leave a set without one)
   const int rounds = tile_hi > tile_lo ? (tile_hi - tile_lo + KSPLIT - 1) / KSPLIT : 0;
-  if (tile_lo + set < tile_hi) issue(n_begin + (tile_lo + set) * BN, 0);
+  if (tile_lo + set < tile_hi) issue(keys.first_key<BN>(tile_lo + set), 0);
   int buffer = 0;
   for (int it = 0; it < rounds; ++it, buffer ^= 1) {
     const int tile = tile_lo + it * KSPLIT + set;
     const bool have_tile = KSPLIT == 1 || tile < tile_hi;
-    const int n0 = n_begin + tile * BN;
+    const int n0 = keys.first_key<BN>(tile);
     wait_for_loads<0>();                  // this wave's pieces of the tile have landed
     __syncthreads();                      // everybody's have, and everybody is done with the other buffer
     if (it + 1 < rounds) {
-      const int next_first = n_begin + (tile_lo + (it + 1) * KSPLIT) * BN;  // first key of the next round's tiles
-      if (((next_first + KSPLIT * BN - 1) >> page_shift) - first_page >= PREFILL_PAGE_IDS) {  // the same for every thread
-        first_page = next_first >> page_shift;
+      const int next_tile = tile_lo + (it + 1) * KSPLIT;  // first of the next round's tiles
+      const int next_last = keys.first_key<BN>(next_tile + KSPLIT - 1) + BN - 1;
+      if ((next_last >> page_shift) - first_page >= PREFILL_PAGE_IDS - kept_pages) {  // the same for every thread
+        first_page = keys.first_key<BN>(next_tile > keys.kept_tiles ? next_tile : keys.kept_tiles) >> page_shift;
         __syncthreads();
         load_page_ids();
         __syncthreads();
       }
-      if (tile + KSPLIT < tile_hi) issue(n0 + KSPLIT * BN, buffer ^ 1);
+      if (tile + KSPLIT < tile_hi) issue(keys.first_key<BN>(tile + KSPLIT), buffer ^ 1);
     }
     // the sequence's last tile, if it is one of this round's and the sequence ends inside a piece of eight keys (the same
     // answer for every thread; once per sequence and workgroup): what follows the last key in that piece is zeroed in LDS
-    const int last_tile = (kv_len - 1 - n_begin) / BN;
+    const int last_tile = keys.kept_tiles + (kv_len - 1 - n_begin) / BN;
     if ((kv_len & 7) != 0 && last_tile >= tile_lo + it * KSPLIT && last_tile < tile_lo + (it + 1) * KSPLIT && last_tile < tile_hi) {
       if (tile == last_tile) {
         const int piece = (kv_len - n0) >> 3, valid = (kv_len - n0) & 7;
@@ -865,7 +980,15 @@ __global__ void __launch_bounds__(64 * WAVES * KSPLIT) __attribute__((amdgpu_wav
         for (int ct = 0; ct < CT; ++ct) s[ct][t] = B::mma(kf[cb], qf[ct][cb], s[ct][t]);
     }
     // ---- scale, mask (only where the tile crosses a row's limits), running maximum ----------
-    const bool whole = n0 + BN <= kv_len && n0 + BN - 1 <= wave_first_pos && (window <= 0 || n0 > wave_last_pos - window);
+    const bool whole = n0 + BN <= kv_len && n0 + BN - 1 <= wave_first_pos && (window <= 0 || n0 > wave_last_pos - window || (KEEPS && n0 + BN <= extras.keep_first));
+    if constexpr (CAPPED) {
+#pragma unroll
+      for (int ct = 0; ct < CT; ++ct)
+#pragma unroll
+        for (int t = 0; t < NT; ++t)
+#pragma unroll
+          for (int j = 0; j < 4; ++j) s[ct][t][j] = cap(s[ct][t][j]);
+    }
     if constexpr (BIASED) {
 #pragma unroll
       for (int ct = 0; ct < CT; ++ct) {
@@ -876,7 +999,7 @@ __global__ void __launch_bounds__(64 * WAVES * KSPLIT) __attribute__((amdgpu_wav
 #pragma unroll
           for (int t = 0; t < NT; ++t)
 #pragma unroll
-            for (int j = 0; j < 4; ++j) s[ct][t][j] = fmaf(s[ct][t][j], scale_eff, c);
+            for (int j = 0; j < 4; ++j) s[ct][t][j] = fmaf(s[ct][t][j], CAPPED ? 1.f : scale_eff, c);
         } else {
 #pragma unroll
           for (int t = 0; t < NT; ++t)
@@ -884,7 +1007,7 @@ __global__ void __launch_bounds__(64 * WAVES * KSPLIT) __attribute__((amdgpu_wav
             for (int j = 0; j < 4; ++j) {
               int d = d0 - (32 * (t >> 1) + 8 * g + 4 * (t & 1) + j);
               d = d < 0 ? 0 : (d > bias_len - 1 ? bias_len - 1 : d);
-              s[ct][t][j] = fmaf(s[ct][t][j], scale_eff, tab[d] * Softmax<T>::SCALE);
+              s[ct][t][j] = fmaf(s[ct][t][j], CAPPED ? 1.f : scale_eff, tab[d] * Softmax<T>::SCALE);
             }
         }
       }
@@ -905,7 +1028,7 @@ __global__ void __launch_bounds__(64 * WAVES * KSPLIT) __attribute__((amdgpu_wav
 #pragma unroll
           for (int j = 0; j < 4; ++j) {
             const int n = n0 + 32 * (t >> 1) + 8 * g + 4 * (t & 1) + j;
-            const bool keep = row_ok[ct] && n < kv_len && n <= pos[ct] && (window <= 0 || n > pos[ct] - window);
+            const bool keep = row_ok[ct] && n < kv_len && n <= pos[ct] && (window <= 0 || n > pos[ct] - window || (KEEPS && n < extras.keep_first));
             s[ct][t][j] = keep ? s[ct][t][j] : -INFINITY;
             mx = fmaxf(mx, s[ct][t][j]);
           }
@@ -1016,8 +1139,10 @@ __global__ void __launch_bounds__(64 * WAVES * KSPLIT) __attribute__((amdgpu_wav
       T* dst = out + (token * nh + head[ct]) * D + 4 * g;
 #pragma unroll
       for (int c = 0; c < NC; ++c) {
+        float4_t o = acc_o[ct][c] * inv;
+        if constexpr (GATED) o = o * gate_of<T>(extras, token, head[ct], 16 * c + 4 * g);
 #pragma unroll
-        for (int j = 0; j < 4; ++j) dst[16 * c + j] = from_f32<T>(acc_o[ct][c][j] * inv);
+        for (int j = 0; j < 4; ++j) dst[16 * c + j] = from_f32<T>(o[j]);
       }
     } else {
       const size_t slot = ((size_t)split * total_tokens + token) * nh + head[ct];
@@ -1075,7 +1200,7 @@ __global__ void __launch_bounds__(64 * WAVES) decode_attention_kernel(
     const int* __restrict__ block_tables, int table_width, const int* __restrict__ kv_lens,
     T* __restrict__ out, float* __restrict__ part_o, float* __restrict__ part_lse,
     int nh, int nkv, int page_shift, float scale, int window, int splits, int total_tokens, const float* __restrict__ bias_table, int bias_len,
-    const float* __restrict__ sinks) {
+    const float* __restrict__ sinks, const Extras extras) {
   constexpr int NC = D / 16;
   constexpr int NCW = (NC + WAVES - 1) / WAVES;
   typedef KeyOps<T, sizeof(T) == 2 && D % 32 == 0> KO;
@@ -1095,24 +1220,25 @@ __global__ void __launch_bounds__(64 * WAVES) decode_attention_kernel(
   const bool row_ok = i < group;
   const int head = kvh * group + (row_ok ? i : 0);
 
-  int n_begin = 0;
-  if (window > 0) {
-    n_begin = pos - window + 1;
-    if (n_begin < 0) n_begin = 0;
-    n_begin &= ~15;
-  }
-  const int tiles_total = (kv_len - n_begin + 15) / 16;
+  const KeyTiles keys = KeyTiles::of<16>(pos - window + 1, window, extras.keep_first, page_shift);
+  const int n_begin = keys.n_begin;
+  const int tiles_total = keys.kept_tiles + (kv_len - n_begin + 15) / 16;
   const int per_split = (tiles_total + splits - 1) / splits;
   const int t_lo = split * per_split;
   int t_hi = t_lo + per_split;
   if (t_hi > tiles_total) t_hi = tiles_total;
 
   const int* table = block_tables + (size_t)b * table_width;
-  // page ids of keys [n_begin + 16 t_lo, n_begin + 16 t_hi)
-  const int first_page = (n_begin + 16 * t_lo) >> page_shift;
-  const int last_key = n_begin + 16 * t_hi < kv_len ? n_begin + 16 * t_hi : kv_len;
+  // page ids of the keys of tiles [t_lo, t_hi)
+  const int first_page = keys.first_key<16>(t_lo > keys.kept_tiles ? t_lo : keys.kept_tiles) >> page_shift;
+  const int keys_end = keys.first_key<16>(t_hi - 1) + 16;
+  const int last_key = keys_end < kv_len ? keys_end : kv_len;
   const int num_pages = t_hi > t_lo ? ((last_key - 1) >> page_shift) - first_page + 1 : 0;
-  {
+  if constexpr (KEEPS) {
+    const int kept_pages = keys.kept_pages;
+    for (int p = tid; p < kept_pages && p < KEPT_PAGE_IDS; p += 64 * WAVES) page_ids[p] = table[p];
+    for (int p = tid; p < num_pages && kept_pages + p < DECODE_PAGE_IDS; p += 64 * WAVES) page_ids[kept_pages + p] = table[first_page + p];
+  } else {
     // (each thread's first id without a branch around the load: it is on the way of everything that follows)
     int at = first_page + (tid < num_pages ? tid : 0);
     at = at < table_width ? at : table_width - 1;
@@ -1134,7 +1260,7 @@ __global__ void __launch_bounds__(64 * WAVES) decode_attention_kernel(
   // (the launcher sends a step here only if a split's keys span at most DECODE_PAGE_IDS pages; the clamp keeps a
   // violated promise from reading outside the array)
   auto page_of = [&](int n) -> size_t {
-    const int p = (n >> page_shift) - first_page;
+    const int p = keys.id_at(n, page_shift, first_page);
     return (size_t)page_ids[p < DECODE_PAGE_IDS ? p : DECODE_PAGE_IDS - 1];
   };
 
@@ -1146,8 +1272,9 @@ __global__ void __launch_bounds__(64 * WAVES) decode_attention_kernel(
   // sequence is read from the last valid place instead; its score is masked and its values are zeroed when the
   // tile is used.
   auto load_tile = [&](Tile& tile, int t) {
-    int n_k = n_begin + 16 * t + i;      // the key whose row this lane reads
-    int n_v = n_begin + 16 * t + 4 * g;  // the first of the four keys whose values this lane reads
+    const int n0 = keys.first_key<16>(t);
+    int n_k = n0 + i;      // the key whose row this lane reads
+    int n_v = n0 + 4 * g;  // the first of the four keys whose values this lane reads
     n_k = n_k < kv_len ? n_k : kv_len - 1;
     n_v = n_v < kv_len ? n_v : (kv_len - 1) & ~3;
     const T* kp = k_cache + ((page_of(n_k) * nkv + kvh) * page_size + (n_k & (page_size - 1))) * D + KO::LANE * g;
@@ -1164,14 +1291,18 @@ __global__ void __launch_bounds__(64 * WAVES) decode_attention_kernel(
     }
   };
 
+  // (the scores here are natural logarithms in both run dtypes: a cap whose result is in the exponent's unit is brought back)
+  Cap<T> cap(scale, CAPPED ? extras.softcap : 1.f);
+  cap.out = CAPPED ? extras.softcap : 1.f;
   float m_i = -INFINITY, l_i = 0.f;
   float4_t acc_o[NC];
 #pragma unroll
   for (int c = 0; c < NC; ++c) acc_o[c] = float4_t{0.f, 0.f, 0.f, 0.f};
 
   auto compute_tile = [&](Tile& tile, int t) {
-    if (n_begin + 16 * t + 16 > kv_len) {  // the sequence ends inside this tile (the same for the whole wave)
-      const int valid = kv_len - (n_begin + 16 * t + 4 * g);
+    const int n0 = keys.first_key<16>(t);
+    if (n0 + 16 > kv_len) {  // the sequence ends inside this tile (the same for the whole wave)
+      const int valid = kv_len - (n0 + 4 * g);
 #pragma unroll
       for (int c = 0; c < NC; ++c) mask_frag(tile.v[c], valid);
     }
@@ -1181,14 +1312,16 @@ __global__ void __launch_bounds__(64 * WAVES) decode_attention_kernel(
     float mx = -INFINITY;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
-      const int n = n_begin + 16 * t + 4 * g + j;
-      const bool keep = row_ok && n < kv_len && (window <= 0 || n > pos - window);
+      const int n = n0 + 4 * g + j;
+      const bool keep = row_ok && n < kv_len && (window <= 0 || n > pos - window || (KEEPS && n < extras.keep_first));
+      const float scaled = CAPPED ? cap(s[j]) : s[j] * scale;
       if constexpr (BIASED) {
         int d = pos - n;
         d = d < 0 ? 0 : (d > bias_len - 1 ? bias_len - 1 : d);
-        s[j] = keep ? fmaf(s[j], scale, bias_table[(size_t)head * bias_len + d]) : -INFINITY;
+        const float bias = bias_table[(size_t)head * bias_len + d];
+        s[j] = keep ? (CAPPED ? scaled + bias : fmaf(s[j], scale, bias)) : -INFINITY;
       } else {
-        s[j] = keep ? s[j] * scale : -INFINITY;
+        s[j] = keep ? scaled : -INFINITY;
       }
       mx = fmaxf(mx, s[j]);
     }
@@ -1280,6 +1413,7 @@ __global__ void __launch_bounds__(64 * WAVES) decode_attention_kernel(
     sum = sum * inv;
     if (splits == 1) {
       T* dst = out + ((size_t)b * nh + head) * D + 16 * c + 4 * g;
+      if constexpr (GATED) sum = sum * gate_of<T>(extras, (size_t)b, head, 16 * c + 4 * g);
 #pragma unroll
       for (int j = 0; j < 4; ++j) dst[j] = from_f32<T>(sum[j]);
     } else {
@@ -1293,7 +1427,7 @@ __global__ void __launch_bounds__(64 * WAVES) decode_attention_kernel(
 // to the denominator
 template <typename T>
 __global__ void merge_splits_kernel(const float* __restrict__ part_o, const float* __restrict__ part_lse, T* __restrict__ out,
-                                    int nh, int splits, int total_tokens, int first_token, const float* __restrict__ sinks) {
+                                    int nh, int splits, int total_tokens, int first_token, const float* __restrict__ sinks, const Extras extras) {
   const size_t token = (size_t)blockIdx.x + first_token;  // (the launch covers tokens [first_token, total_tokens))
   const int head = blockIdx.y;
   const size_t stride = (size_t)total_tokens * nh;  // slots per split
@@ -1313,7 +1447,9 @@ __global__ void merge_splits_kernel(const float* __restrict__ part_o, const floa
       acc += w * part_o[slot * D + dd];
       denom += w;
     }
-    out[slot0 * D + dd] = from_f32<T>(acc / (denom > 0.f ? denom : 1.f));
+    float o = acc / (denom > 0.f ? denom : 1.f);
+    if constexpr (GATED) o *= gate_of<T>(extras, token, head, dd & ~3)[dd & 3];
+    out[slot0 * D + dd] = from_f32<T>(o);
   }
 }
 
@@ -1339,12 +1475,12 @@ template <typename T>
 static int launch(const void* qkv, int qkv_stride, const void* k_cache, const void* v_cache, const int* block_tables, int table_width,
                   const int* cu_q, const int* kv_lens, void* out, float* part_o, float* part_lse, int num_seqs, int total_tokens,
                   int max_q_len, int max_kv_len, int nh, int nkv, int page_shift, float scale, int window, int splits, int first_token,
-                  const float* bias_table, int bias_len, const float* sinks, hipStream_t stream) {
+                  const float* bias_table, int bias_len, const float* sinks, const Extras& extras, hipStream_t stream) {
   constexpr int BN = tile_keys<T>();
   const int group = nh / nkv;
   // the streaming kernel keeps the page ids of a split's keys in LDS: they have to fit
   const int keys_per_split = (((max_kv_len + 15) / 16 + splits - 1) / splits) * 16;
-  const bool ids_fit = (keys_per_split >> page_shift) + 2 <= DECODE_PAGE_IDS;
+  const bool ids_fit = (keys_per_split >> page_shift) + 2 + (KEEPS ? ((extras.keep_first + 15) / 16 * 16 >> page_shift) + 1 : 0) <= DECODE_PAGE_IDS;
   if (max_q_len == 1 && total_tokens == num_seqs && first_token == 0 && group <= 16 && page_shift >= 2 && sizeof(T) * D <= 512 && ids_fit) {
     // every sequence decodes one token: the streaming kernel.  Register sets per wave: one being computed, the others
     // in flight.  (For steps with one workgroup per compute unit, twice as many sets and eight waves per workgroup
@@ -1352,10 +1488,10 @@ static int launch(const void* qkv, int qkv_stride, const void* k_cache, const vo
     constexpr int DEPTH = sizeof(T) * D <= 256 ? 3 : 2;
     decode_attention_kernel<T, DEPTH, 4><<<dim3(splits, nkv, num_seqs), 256, 0, stream>>>(
         (const T*)qkv, qkv_stride, (const T*)k_cache, (const T*)v_cache, block_tables, table_width, kv_lens, (T*)out, part_o, part_lse,
-        nh, nkv, page_shift, scale, window, splits, total_tokens, bias_table, bias_len, sinks);
+        nh, nkv, page_shift, scale, window, splits, total_tokens, bias_table, bias_len, sinks, extras);
     int status = (int)hipGetLastError();
     if (status != 0 || splits == 1) return status;
-    merge_splits_kernel<T><<<dim3(total_tokens, nh), D < 64 ? 64 : D, 0, stream>>>(part_o, part_lse, (T*)out, nh, splits, total_tokens, 0, sinks);
+    merge_splits_kernel<T><<<dim3(total_tokens, nh), D < 64 ? 64 : D, 0, stream>>>(part_o, part_lse, (T*)out, nh, splits, total_tokens, 0, sinks, extras);
     return (int)hipGetLastError();
   }
   // The kernel whose tiles reach LDS by direct loads: bfloat16, head sizes 64 and 128, pages of at least 8 tokens.
@@ -1368,16 +1504,16 @@ static int launch(const void* qkv, int qkv_stride, const void* k_cache, const vo
       if (two_sets)
         direct_attention_kernel<2, 4, 2><<<grid, 512, 0, stream>>>(
             (const bf16_t*)qkv, qkv_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, table_width, cu_q, kv_lens, (bf16_t*)out,
-            part_o, part_lse, nh, nkv, page_shift, scale, window, splits, total_tokens, bias_table, bias_len, sinks);
+            part_o, part_lse, nh, nkv, page_shift, scale, window, splits, total_tokens, bias_table, bias_len, sinks, extras);
       else
         direct_attention_kernel<2, 4><<<grid, 256, 0, stream>>>(
             (const bf16_t*)qkv, qkv_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, table_width, cu_q, kv_lens, (bf16_t*)out,
-            part_o, part_lse, nh, nkv, page_shift, scale, window, splits, total_tokens, bias_table, bias_len, sinks);
+            part_o, part_lse, nh, nkv, page_shift, scale, window, splits, total_tokens, bias_table, bias_len, sinks, extras);
     }
     int status = (int)hipGetLastError();
     if (status != 0 || splits == 1) return status;
     merge_splits_kernel<T><<<dim3(total_tokens - first_token, nh), D < 64 ? 64 : D, 0, stream>>>(part_o, part_lse, (T*)out, nh, splits, total_tokens,
-                                                                                                 first_token, sinks);
+                                                                                                 first_token, sinks, extras);
     return (int)hipGetLastError();
   };
   if (direct_ok && portion_kernel_choice >= 2 && max_q_len * group > 64) return launch_direct(portion_kernel_choice == 3);
@@ -1430,39 +1566,41 @@ static int launch(const void* qkv, int qkv_stride, const void* k_cache, const vo
       if (rows >= 256 && workgroups * 4 >= 7LL * compute_units()) {
         paged_attention_kernel<T, BN, 2, 1, 4><<<grid, 256, 0, stream>>>(
             (const T*)qkv, qkv_stride, (const T*)k_cache, (const T*)v_cache, block_tables, table_width, cu_q, kv_lens, (T*)out, part_o,
-            part_lse, nh, nkv, page_shift, scale, window, splits, total_tokens, bias_table, bias_len, sinks);
+            part_lse, nh, nkv, page_shift, scale, window, splits, total_tokens, bias_table, bias_len, sinks, extras);
       } else {
         paged_attention_kernel<T, BN, 1, 1, 8><<<grid, 512, 0, stream>>>(
             (const T*)qkv, qkv_stride, (const T*)k_cache, (const T*)v_cache, block_tables, table_width, cu_q, kv_lens, (T*)out, part_o,
-            part_lse, nh, nkv, page_shift, scale, window, splits, total_tokens, bias_table, bias_len, sinks);
+            part_lse, nh, nkv, page_shift, scale, window, splits, total_tokens, bias_table, bias_len, sinks, extras);
       }
     } else {
       dim3 grid(num_seqs * splits, nkv, (rows + 255) / 256);
       paged_attention_kernel<T, BN, WIDE, 1, 8><<<grid, 512, 0, stream>>>(
           (const T*)qkv, qkv_stride, (const T*)k_cache, (const T*)v_cache, block_tables, table_width, cu_q, kv_lens, (T*)out, part_o,
-          part_lse, nh, nkv, page_shift, scale, window, splits, total_tokens, bias_table, bias_len, sinks);
+          part_lse, nh, nkv, page_shift, scale, window, splits, total_tokens, bias_table, bias_len, sinks, extras);
     }
   } else if (WIDE == 2 && (long long)((rows + 63) / 64) * nkv * num_seqs * splits < 2 * compute_units() && max_kv_len >= 8 * BN) {
     // too few workgroups to fill the GPU and many keys each: two sets of waves share a workgroup's keys
     dim3 grid(num_seqs * splits, nkv, (rows + 63) / 64);
     paged_attention_kernel<T, BN, 1, WIDE><<<grid, 256 * WIDE, 0, stream>>>(
         (const T*)qkv, qkv_stride, (const T*)k_cache, (const T*)v_cache, block_tables, table_width, cu_q, kv_lens, (T*)out, part_o,
-        part_lse, nh, nkv, page_shift, scale, window, splits, total_tokens, bias_table, bias_len, sinks);
+        part_lse, nh, nkv, page_shift, scale, window, splits, total_tokens, bias_table, bias_len, sinks, extras);
   } else {
     dim3 grid(num_seqs * splits, nkv, (rows + 63) / 64);
     paged_attention_kernel<T, BN, 1, 1><<<grid, 256, 0, stream>>>(
         (const T*)qkv, qkv_stride, (const T*)k_cache, (const T*)v_cache, block_tables, table_width, cu_q, kv_lens, (T*)out, part_o,
-        part_lse, nh, nkv, page_shift, scale, window, splits, total_tokens, bias_table, bias_len, sinks);
+        part_lse, nh, nkv, page_shift, scale, window, splits, total_tokens, bias_table, bias_len, sinks, extras);
   }
   int status = (int)hipGetLastError();
   if (status != 0 || splits == 1) return status;
   merge_splits_kernel<T><<<dim3(total_tokens - first_token, nh), D < 64 ? 64 : D, 0, stream>>>(part_o, part_lse, (T*)out, nh, splits, total_tokens,
-                                                                                               first_token, sinks);
+                                                                                               first_token, sinks, extras);
   return (int)hipGetLastError();
 }
 
 extern "C" int velox_attention_head_dim() { return D; }
 extern "C" int velox_attention_biased() { return BIASED ? 1 : 0; }
+// what this library was built with: 1 bias by distance, 2 kept first keys, 4 capped scores, 8 gated outputs
+extern "C" int velox_attention_options() { return (BIASED ? 1 : 0) | (KEEPS ? 2 : 0) | (CAPPED ? 4 : 0) | (GATED ? 8 : 0); }
 
 // part_o: float32 [splits, total_tokens, nh, D]; part_lse: float32 [splits, total_tokens, nh]; both unused when splits == 1.
 // first_token: the sequences given (cu_q holds rows of qkv and out) cover rows [first_token, total_tokens); a launch for
@@ -1471,14 +1609,24 @@ extern "C" int velox_paged_attention(const void* qkv, int qkv_stride, const void
                                      const int* block_tables, int table_width, const int* cu_q, const int* kv_lens, void* out,
                                      float* part_o, float* part_lse, int num_seqs, int total_tokens, int max_q_len, int max_kv_len,
                                      int nh, int nkv, int page_shift, float scale, int window, int splits, int first_token, int dtype,
-                                     const float* bias_table, int bias_len, const float* sinks, hipStream_t stream) {
+                                     const float* bias_table, int bias_len, const float* sinks, int keep_first, float softcap, const void* gate,
+                                     int gate_stride, int gate_channels, hipStream_t stream) {
+  // keep_first: read by a build for kept keys; softcap: by one for capped scores; gate (rows of the queries' type), its stride and
+  // channels per head (0: one number per head): by one for gated outputs; each must be given exactly to the build that reads it.
   // sinks: float32 [nh] or nullptr; exp(sinks[h]) joins the softmax's denominator of every row of head h (no key, no value, not scaled)
   if (num_seqs <= 0 || total_tokens <= 0) return 0;
   if (BIASED ? (bias_table == nullptr || bias_len < 1) : bias_table != nullptr) return -1;  // (the build and the call must agree)
+  if (CAPPED != (softcap > 0.f) || GATED != (gate != nullptr) || (!KEEPS && keep_first != 0) || keep_first < 0) return -1;
+  if (GATED && (gate_channels < 0 || gate_channels > D || gate_stride < nh * (gate_channels > 0 ? gate_channels : 1))) return -1;
+  // (kept keys' pages have a part of the page-id arrays; tiles of 64 keys are the largest)
+  if (KEEPS && (((keep_first + 63) / 64 * 64) >> page_shift) + 1 > KEPT_PAGE_IDS) return -1;
+  const size_t elem = dtype == VELOX_BF16 ? 2 : 4;
+  const Extras extras{keep_first, softcap, gate, gate_stride, gate_channels,
+                      gate_channels % 4 == 0 && gate_stride % 4 == 0 && (uintptr_t)gate % (4 * elem) == 0};
   if (nh % nkv != 0 || splits < 1 || page_shift < 0 || max_kv_len < 1 || first_token < 0 || first_token >= total_tokens) return -1;
   if (dtype == VELOX_BF16)
     return launch<bf16_t>(qkv, qkv_stride, k_cache, v_cache, block_tables, table_width, cu_q, kv_lens, out, part_o, part_lse, num_seqs,
-                          total_tokens, max_q_len, max_kv_len, nh, nkv, page_shift, scale, window, splits, first_token, bias_table, bias_len, sinks, stream);
+                          total_tokens, max_q_len, max_kv_len, nh, nkv, page_shift, scale, window, splits, first_token, bias_table, bias_len, sinks, extras, stream);
   return launch<float>(qkv, qkv_stride, k_cache, v_cache, block_tables, table_width, cu_q, kv_lens, out, part_o, part_lse, num_seqs,
-                       total_tokens, max_q_len, max_kv_len, nh, nkv, page_shift, scale, window, splits, first_token, bias_table, bias_len, sinks, stream);
+                       total_tokens, max_q_len, max_kv_len, nh, nkv, page_shift, scale, window, splits, first_token, bias_table, bias_len, sinks, extras, stream);
 }

@@ -700,6 +700,20 @@ extern "C" int velox_scale(float* x, long long n, float factor, hipStream_t stre
   VELOX_RETURN_LAUNCH_STATUS();
 }
 
+// x[i] = cap * tanh(factor * x[i] / cap), float32, in place.
+__global__ void __launch_bounds__(256) softcap_kernel(float* __restrict__ x, long long n, float in, float cap) {
+  for (long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (long long)gridDim.x * blockDim.x) x[i] = cap * tanhf(x[i] * in);
+}
+
+extern "C" int velox_softcap(float* x, long long n, float factor, float cap, hipStream_t stream) {
+  if (n <= 0) return 0;
+  if (!(cap > 0.f)) return -1;
+  long long blocks = (n + 255) / 256;
+  if (blocks > 4096) blocks = 4096;
+  softcap_kernel<<<(int)blocks, 256, 0, stream>>>(x, n, factor / cap, cap);
+  VELOX_RETURN_LAUNCH_STATUS();
+}
+
 // out[i] = act(x[i]) for a unit without a gate branch (ungated_act in common.h).  float32 arithmetic, one rounding.
 
 template <typename T>

@@ -263,7 +263,8 @@ __global__ void __launch_bounds__(256) plain_attention_kernel(const T* __restric
                                                               const int* __restrict__ block_tables, int table_width, const int* __restrict__ cu_q,
                                                               const int* __restrict__ kv_lens, T* __restrict__ out, int num_seqs, int nh, int nkv, int d,
                                                               int page_shift, float scale, int window, const float* __restrict__ bias_table, int bias_len,
-                                                              const float* __restrict__ sinks) {
+                                                              const float* __restrict__ sinks, int keep_first, float softcap, const T* __restrict__ gate,
+                                                              int gate_stride, int gate_channels) {
   __shared__ float q_s[PLAIN_ATTENTION_MAX_D];
   __shared__ float p_s[256];
   __shared__ float scratch[16];
@@ -287,25 +288,29 @@ __global__ void __launch_bounds__(256) plain_attention_kernel(const T* __restric
   float acc[PLAIN_ATTENTION_MAX_D / 256];
 #pragma unroll
   for (int u = 0; u < PLAIN_ATTENTION_MAX_D / 256; ++u) acc[u] = 0.f;
-  for (int j0 = first; j0 <= last; j0 += 256) {
+  // keys before the window that every query sees: 0 .. kept - 1, worked first; then the window's
+  const int kept = min(keep_first, first);
+  for (int j0 = kept > 0 ? 0 : first; j0 <= last; j0 = j0 < kept && j0 + 256 >= kept ? first : j0 + 256) {
+    const int end = j0 < kept ? kept - 1 : last;  // the last key of this run of keys
     const int j = j0 + tid;
     float s = -INFINITY;
-    if (j <= last) {
+    if (j <= end) {
       const T* key = k_cache + (((size_t)table[j >> page_shift] * nkv + kvh) * page_size + (j & (page_size - 1))) * d;
       float dot = 0.f;
       for (int c = 0; c < d; ++c) dot = fmaf(q_s[c], to_f32(key[c]), dot);
       s = dot * scale;
+      if (softcap > 0.f) s = softcap * tanhf(s / softcap);
       // a bias by distance, float32 [nh, bias_len]: the key n positions behind the query reads column min(n, bias_len - 1)
       if (bias_table) s += bias_table[(size_t)head * bias_len + min(last - j, bias_len - 1)];
     }
     const float new_max = fmaxf(running_max, block_max_256(s, scratch));  // (finite: key j0 is always seen)
-    const float p = j <= last ? expf(s - new_max) : 0.f;
+    const float p = j <= end ? expf(s - new_max) : 0.f;
     p_s[tid] = p;
     const float chunk_sum = block_sum(p, scratch);  // (its barriers also publish p_s)
     const float alpha = expf(running_max - new_max);
     denom = denom * alpha + chunk_sum;
     running_max = new_max;
-    const int count = min(256, last - j0 + 1);
+    const int count = min(256, end - j0 + 1);
 #pragma unroll
     for (int u = 0; u < PLAIN_ATTENTION_MAX_D / 256; ++u) {
       const int c = tid + 256 * u;
@@ -324,22 +329,35 @@ __global__ void __launch_bounds__(256) plain_attention_kernel(const T* __restric
 #pragma unroll
   for (int u = 0; u < PLAIN_ATTENTION_MAX_D / 256; ++u) {
     const int c = tid + 256 * u;
-    if (c < d) out[(size_t)token * nh * d + (size_t)head * d + c] = from_f32<T>(acc[u] / denom);
+    if (c >= d) continue;
+    float o = acc[u] / denom;
+    // a gate on the head's output: one number per head, or one per channel of the first gate_channels
+    if (gate && (gate_channels == 0 || c < gate_channels)) {
+      const float z = to_f32(gate[(size_t)token * gate_stride + (gate_channels == 0 ? head : head * gate_channels + c)]);
+      o *= 1.f / (1.f + expf(-z));
+    }
+    out[(size_t)token * nh * d + (size_t)head * d + c] = from_f32<T>(o);
   }
 }
 
 extern "C" int velox_plain_attention(const void* q, int q_width, const void* k_cache, const void* v_cache, const int* block_tables, int table_width,
                                      const int* cu_q, const int* kv_lens, void* out, int num_seqs, int tokens, int nh, int nkv, int d, int page_shift,
-                                     float scale, int window, int dtype, const float* bias_table, int bias_len, const float* sinks, hipStream_t stream) {
+                                     float scale, int window, int dtype, const float* bias_table, int bias_len, const float* sinks, int keep_first,
+                                     float softcap, const void* gate, int gate_stride, int gate_channels, hipStream_t stream) {
+  // keep_first: keys that every query sees, whatever its window; softcap > 0: scores become softcap * tanh(score / softcap) before the
+  // bias; gate: rows of the queries' type, see attention.hip
   if (tokens <= 0) return 0;
+  if (keep_first < 0 || gate_channels < 0 || gate_channels > d || (gate != nullptr && gate_stride < nh * (gate_channels > 0 ? gate_channels : 1))) return -1;
   if (bias_table != nullptr && bias_len < 1) return -1;
   if (d < 1 || d > PLAIN_ATTENTION_MAX_D || nh < 1 || nkv < 1 || nh % nkv != 0 || nh > 65535 || num_seqs < 1 || nh * d > q_width) return -1;
   dim3 grid(tokens, nh);
   if (dtype == VELOX_BF16)
     plain_attention_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)q, q_width, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, table_width,
-                                                             cu_q, kv_lens, (bf16_t*)out, num_seqs, nh, nkv, d, page_shift, scale, window, bias_table, bias_len, sinks);
+                                                             cu_q, kv_lens, (bf16_t*)out, num_seqs, nh, nkv, d, page_shift, scale, window, bias_table, bias_len, sinks, keep_first, softcap,
+                                                             (const bf16_t*)gate, gate_stride, gate_channels);
   else
     plain_attention_kernel<float><<<grid, 256, 0, stream>>>((const float*)q, q_width, (const float*)k_cache, (const float*)v_cache, block_tables, table_width,
-                                                            cu_q, kv_lens, (float*)out, num_seqs, nh, nkv, d, page_shift, scale, window, bias_table, bias_len, sinks);
+                                                            cu_q, kv_lens, (float*)out, num_seqs, nh, nkv, d, page_shift, scale, window, bias_table, bias_len, sinks, keep_first, softcap, (const float*)gate, gate_stride,
+                                                            gate_channels);
   VELOX_RETURN_LAUNCH_STATUS();
 }

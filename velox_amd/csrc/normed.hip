@@ -6,6 +6,8 @@
 //                   sub-layer's OUTPUT, float32 throughout, one rounding for the copy)
 //   norm_add_norm:  the same with the norm that reads the residual next in the same kernel: a norm behind one sub-layer, the
 //                   residual sum, the norm before the next sub-layer
+//   sum_norm:       the residual plus up to two terms that pass norms of their own and up to two that do not, and the norm that
+//                   reads the sum next, or the sum beside another row for a product over both (join)
 //   poly_norm:      a y1 + b y2 + c y3 + e with y_k = z^k / sqrt(mean(z^2k) + eps) over a row
 //   qk_norm_write:  RMS norm of the queries and of the keys (over the whole projection or per head), the query
 //                   temperature, the blend of the values with an earlier layer's, queries written at the kernels' head
@@ -329,6 +331,221 @@ extern "C" int velox_norm_add_norm(float* residual, const void* y, int y_dtype, 
   NormAddNormArgs a{residual, y, y_weight, weight, rows, out, out_dtype == VELOX_BF16, hidden, partials, (size_t)partial_stride, y_eps, eps};
   if (y_dtype == VELOX_BF16) norm_add_norm_launch<bf16_t>(a, count, stream);
   else norm_add_norm_launch<float>(a, count, stream);
+  VELOX_RETURN_LAUNCH_STATUS();
+}
+
+// ---------------------------------------------------------------------------------------------
+// sum_norm: one workgroup per output row.  r = residual + ((n_0 + n_1) + (p_0 + p_1)) with n_i = scale_i * y_i / sqrt(mean(y_i^2) +
+// term_eps) * w_i and plain terms p_i (each term may be missing, and may come as stacked float32 partial sums, added first to last).
+//   norm:  out = r / sqrt(mean(r^2) + eps) * w; r is written back unless `rows` picks rows.
+//   join (weight == nullptr):  out = [r ; start], rows of 2 * hidden; the residual is cleared.
+// The row stays in registers between the passes (PIECES pieces of four neighbours per lane), or in LDS for rows that are no
+// multiple of four.
+// ---------------------------------------------------------------------------------------------
+struct SumTerm {
+  const void* p;
+  int bf16, partials;
+  size_t stride;        // elements between partial sums
+  const float* weight;  // of the term's own norm (normed terms)
+  float scale;
+};
+struct SumNormArgs {
+  float* residual;
+  SumTerm normed[2], plain[2];
+  int num_normed, num_plain;
+  float term_eps;
+  const int* rows;
+  const float* weight;
+  float eps;
+  const void* start;
+  int start_bf16;
+  void* out;
+  int out_bf16, hidden;
+};
+
+__device__ __forceinline__ float4_t term_piece(const SumTerm& t, size_t at) {
+  float4_t v = float4_t{0.f, 0.f, 0.f, 0.f};
+  for (int p = 0; p < t.partials; ++p) {
+    if (t.bf16) {
+      const Piece4<bf16_t> q = *reinterpret_cast<const Piece4<bf16_t>*>((const bf16_t*)t.p + p * t.stride + at);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) v[j] += q.get(j);
+    } else {
+      v += *reinterpret_cast<const float4_t*>((const float*)t.p + p * t.stride + at);
+    }
+  }
+  return v;
+}
+__device__ __forceinline__ float term_value(const SumTerm& t, size_t at) {
+  float v = 0.f;
+  for (int p = 0; p < t.partials; ++p) v += t.bf16 ? to_f32(((const bf16_t*)t.p)[p * t.stride + at]) : ((const float*)t.p)[p * t.stride + at];
+  return v;
+}
+__device__ __forceinline__ void store_piece(void* out, int out_bf16, size_t at, float4_t o) {
+  if (out_bf16) {
+    short4_t bits;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) bits[j] = bf16_bits(o[j]);
+    *reinterpret_cast<short4_t*>((bf16_t*)out + at) = bits;
+  } else {
+    *reinterpret_cast<float4_t*>((float*)out + at) = o;
+  }
+}
+// both sums over the workgroup at once; `scratch` holds 32 floats that nothing else uses
+__device__ __forceinline__ void block_sum2(float& x, float& y, float* scratch) {
+  const int lane = threadIdx.x & (VELOX_WAVE - 1), wave = threadIdx.x / VELOX_WAVE, waves = (blockDim.x + VELOX_WAVE - 1) / VELOX_WAVE;
+  x = wave_sum(x);
+  y = wave_sum(y);
+  if (lane == 0) { scratch[wave] = x; scratch[16 + wave] = y; }
+  __syncthreads();
+  x = y = 0.f;
+  for (int w = 0; w < waves; ++w) { x += scratch[w]; y += scratch[16 + w]; }
+}
+
+template <int PIECES>
+__global__ void __launch_bounds__(1024) sum_norm_vec_kernel(const SumNormArgs a) {
+  __shared__ float pair_scratch[32];
+  __shared__ float scratch[16];
+  const int H = a.hidden;
+  const size_t src = a.rows ? (size_t)a.rows[blockIdx.x] : (size_t)blockIdx.x;
+  float* res = a.residual + src * H;
+  float4_t y0[PIECES], y1[PIECES], r[PIECES];
+  float s0 = 0.f, s1 = 0.f;
+#pragma unroll
+  for (int c = 0; c < PIECES; ++c) {
+    const int at = (threadIdx.x + c * blockDim.x) * 4;
+    y0[c] = y1[c] = r[c] = float4_t{0.f, 0.f, 0.f, 0.f};
+    if (at < H) {
+      if (a.num_normed > 0) y0[c] = term_piece(a.normed[0], src * H + at);
+      if (a.num_normed > 1) y1[c] = term_piece(a.normed[1], src * H + at);
+      r[c] = *reinterpret_cast<const float4_t*>(res + at);  // (asked for before the reduction: the wait hides behind it)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) { s0 += y0[c][j] * y0[c][j]; s1 += y1[c][j] * y1[c][j]; }
+    }
+  }
+  float f0 = 0.f, f1 = 0.f;
+  if (a.num_normed > 0) {
+    block_sum2(s0, s1, pair_scratch);
+    f0 = 1.f / sqrtf(s0 / (float)H + a.term_eps);
+    f1 = 1.f / sqrtf(s1 / (float)H + a.term_eps);
+  }
+  float sumsq = 0.f;
+#pragma unroll
+  for (int c = 0; c < PIECES; ++c) {
+    const int at = (threadIdx.x + c * blockDim.x) * 4;
+    if (at < H) {
+      float4_t n = float4_t{0.f, 0.f, 0.f, 0.f}, p = n;
+      if (a.num_normed > 0) n = y0[c] * f0 * *reinterpret_cast<const float4_t*>(a.normed[0].weight + at) * a.normed[0].scale;
+      if (a.num_normed > 1) n += y1[c] * f1 * *reinterpret_cast<const float4_t*>(a.normed[1].weight + at) * a.normed[1].scale;
+      if (a.num_plain > 0) p = term_piece(a.plain[0], src * H + at);
+      if (a.num_plain > 1) p += term_piece(a.plain[1], src * H + at);
+      r[c] += n + p;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) sumsq += r[c][j] * r[c][j];
+      if (a.weight == nullptr) {
+        const size_t to = (size_t)blockIdx.x * 2 * H + at;
+        SumTerm start{a.start, a.start_bf16, 1, 0, nullptr, 1.f};
+        store_piece(a.out, a.out_bf16, to, r[c]);
+        store_piece(a.out, a.out_bf16, to + H, term_piece(start, src * H + at));
+        *reinterpret_cast<float4_t*>(res + at) = float4_t{0.f, 0.f, 0.f, 0.f};
+      } else if (!a.rows) {
+        *reinterpret_cast<float4_t*>(res + at) = r[c];
+      }
+    }
+  }
+  if (a.weight == nullptr) return;
+  const float inv = 1.f / sqrtf(block_sum(sumsq, scratch) / (float)H + a.eps);
+#pragma unroll
+  for (int c = 0; c < PIECES; ++c) {
+    const int at = (threadIdx.x + c * blockDim.x) * 4;
+    if (at < H) store_piece(a.out, a.out_bf16, (size_t)blockIdx.x * H + at, r[c] * inv * *reinterpret_cast<const float4_t*>(a.weight + at));
+  }
+}
+
+__global__ void __launch_bounds__(256) sum_norm_kernel(const SumNormArgs a) {
+  extern __shared__ float held_row[];
+  __shared__ float pair_scratch[32];
+  __shared__ float scratch[16];
+  const int H = a.hidden;
+  const size_t src = a.rows ? (size_t)a.rows[blockIdx.x] : (size_t)blockIdx.x;
+  float* res = a.residual + src * H;
+  float f0 = 0.f, f1 = 0.f;
+  if (a.num_normed > 0) {
+    float s0 = 0.f, s1 = 0.f;
+    for (int i = threadIdx.x; i < H; i += 256) {
+      const float v = term_value(a.normed[0], src * H + i);
+      s0 += v * v;
+      if (a.num_normed > 1) { const float w = term_value(a.normed[1], src * H + i); s1 += w * w; }
+    }
+    block_sum2(s0, s1, pair_scratch);
+    f0 = 1.f / sqrtf(s0 / (float)H + a.term_eps);
+    f1 = 1.f / sqrtf(s1 / (float)H + a.term_eps);
+  }
+  float sumsq = 0.f;
+  for (int i = threadIdx.x; i < H; i += 256) {  // (every lane reads back only what it wrote itself)
+    float n = 0.f, p = 0.f;
+    if (a.num_normed > 0) n = term_value(a.normed[0], src * H + i) * f0 * a.normed[0].weight[i] * a.normed[0].scale;
+    if (a.num_normed > 1) n += term_value(a.normed[1], src * H + i) * f1 * a.normed[1].weight[i] * a.normed[1].scale;
+    if (a.num_plain > 0) p = term_value(a.plain[0], src * H + i);
+    if (a.num_plain > 1) p += term_value(a.plain[1], src * H + i);
+    const float r = res[i] + (n + p);
+    sumsq += r * r;
+    if (a.weight == nullptr) {
+      const size_t to = (size_t)blockIdx.x * 2 * H + i;
+      const float other = a.start_bf16 ? to_f32(((const bf16_t*)a.start)[src * H + i]) : ((const float*)a.start)[src * H + i];
+      if (a.out_bf16) { ((bf16_t*)a.out)[to] = (bf16_t)r; ((bf16_t*)a.out)[to + H] = (bf16_t)other; }
+      else { ((float*)a.out)[to] = r; ((float*)a.out)[to + H] = other; }
+      res[i] = 0.f;
+    } else {
+      held_row[i] = r;
+      if (!a.rows) res[i] = r;
+    }
+  }
+  if (a.weight == nullptr) return;
+  const float inv = 1.f / sqrtf(block_sum(sumsq, scratch) / (float)H + a.eps);
+  for (int i = threadIdx.x; i < H; i += 256) {
+    const float o = held_row[i] * inv * a.weight[i];
+    const size_t to = (size_t)blockIdx.x * H + i;
+    if (a.out_bf16) ((bf16_t*)a.out)[to] = (bf16_t)o;
+    else ((float*)a.out)[to] = o;
+  }
+}
+
+// terms: four descriptions of five numbers each as the host passes them, the two normed ones first: address, type, partial sums, elements
+// between those, the address of the norm's weight, and scales[i] for the normed ones.
+extern "C" int velox_sum_norm(float* residual, const long long* terms, const float* scales, int num_normed, int num_plain, float term_eps, const int* rows,
+                              const float* weight, float eps, const void* start, int start_dtype, void* out, int out_dtype, int count, int hidden,
+                              hipStream_t stream) {
+  if (count <= 0) return 0;
+  if (hidden < 1 || hidden > 16384 - 64 || num_normed < 0 || num_normed > 2 || num_plain < 0 || num_plain > 2) return (int)hipErrorInvalidValue;
+  if (weight == nullptr && (start == nullptr || rows != nullptr)) return (int)hipErrorInvalidValue;
+  SumNormArgs a{};
+  uintptr_t addresses = (uintptr_t)residual | (uintptr_t)weight | (uintptr_t)out | (uintptr_t)start;
+  bool whole = hidden % 4 == 0;
+  auto term_of = [&](int i) {
+    const long long* d = terms + 5 * i;
+    SumTerm t{(const void*)(uintptr_t)d[0], d[1] == VELOX_BF16, (int)d[2], (size_t)d[3], (const float*)(uintptr_t)d[4], scales[i]};
+    addresses |= (uintptr_t)t.p | (uintptr_t)t.weight;
+    whole = whole && t.stride % 4 == 0;
+    return t;
+  };
+  for (int i = 0; i < num_normed; ++i) a.normed[i] = term_of(i);
+  for (int i = 0; i < num_plain; ++i) a.plain[i] = term_of(2 + i);
+  a.residual = residual; a.num_normed = num_normed; a.num_plain = num_plain; a.term_eps = term_eps; a.rows = rows; a.weight = weight; a.eps = eps;
+  a.start = start; a.start_bf16 = start_dtype == VELOX_BF16; a.out = out; a.out_bf16 = out_dtype == VELOX_BF16; a.hidden = hidden;
+  if (whole && addresses % 16 == 0) {
+    const int pieces = hidden / 4;
+    // few rows: a lane per piece as long as that is possible (the kernel is a chain of waits); many rows: two pieces a lane
+    int lanes = count <= 64 || pieces <= 256 ? pieces : (pieces + 1) / 2;
+    lanes = (lanes + 63) / 64 * 64;
+    if (lanes > 1024) lanes = 1024;
+    const int per_lane = (pieces + lanes - 1) / lanes;
+    if (per_lane <= 1) sum_norm_vec_kernel<1><<<count, lanes, 0, stream>>>(a);
+    else if (per_lane <= 2) sum_norm_vec_kernel<2><<<count, lanes, 0, stream>>>(a);
+    else sum_norm_vec_kernel<4><<<count, lanes, 0, stream>>>(a);
+  } else {
+    sum_norm_kernel<<<count, 256, (size_t)hidden * sizeof(float), stream>>>(a);
+  }
   VELOX_RETURN_LAUNCH_STATUS();
 }
 

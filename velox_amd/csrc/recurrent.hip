@@ -1,6 +1,6 @@
 // Kernels of the mixers that carry a state of fixed size from token to token, and of the blocks around them, for gfx950:
 //   stream_norm         the residual streams' update (mix matrix, weighted sub-layer output) and the norm of their weighted sum
-//   gated_act_mul       act(gate) * up with the tanh form of GELU or SiLU
+//   gated_act_mul       act(gate) * up with the tanh form of GELU, SiLU or the rectifier
 //   short_conv          causal convolution over a few taps per channel, the inputs before a portion's start from the state slot
 //   rotate_pad_write    partial rotation of q and k, q at the attention kernels' head size, k and v into the paged cache
 //   recurrence_prepare  unit q and k, decay and beta of a linear recurrence, all float32
@@ -248,7 +248,7 @@ extern "C" int velox_embed_copies(const int* ids, const void* table, int table_d
 }
 
 // ---------------------------------------------------------------------------------------------
-// gated_act_mul: out[t, i] = act(gate_up[t, i]) * gate_up[t, I + i]; kind 0: SiLU, 1: the tanh form of GELU.
+// gated_act_mul: out[t, i] = act(gate_up[t, i]) * gate_up[t, I + i]; kind 0: SiLU, 1: the tanh form of GELU, 2: max(z, 0).
 // ---------------------------------------------------------------------------------------------
 __device__ __forceinline__ float gelu_tanh_f32(float z) { return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))); }
 
@@ -258,7 +258,7 @@ __global__ void __launch_bounds__(256) gated_act_mul_kernel(const T* __restrict_
   const T* row = gate_up + t * 2 * (size_t)inter;
   for (int i = blockIdx.x * blockDim.x + threadIdx.x; i < inter; i += gridDim.x * blockDim.x) {
     const float g = to_f32(row[i]), u = to_f32(row[inter + i]);
-    const float act = kind == 1 ? gelu_tanh_f32(g) : g * sigmoid_f32(g);
+    const float act = kind == 1 ? gelu_tanh_f32(g) : kind == 2 ? fmaxf(g, 0.f) : g * sigmoid_f32(g);
     out[t * inter + i] = from_f32<T>(act * u);
   }
 }
@@ -275,7 +275,7 @@ extern "C" int velox_gated_act_mul(const void* gate_up, void* out, int tokens, i
 }
 
 // ---------------------------------------------------------------------------------------------
-// short_conv.  x [T, ld]: the first C columns pass y_t = sum_j w[c, j] u_(t - taps + 1 + j), per sequence; the inputs before a
+// short_conv.  x [T, ld], from the first of C columns on: they pass y_t = sum_j w[c, j] u_(t - taps + 1 + j) (+ bias[c]), per sequence; the inputs before a
 // portion's start are tail[slot] ([taps - 1, C], oldest first; nullptr: zeros).  Grid (channel blocks, token chunks, sequences);
 // a thread owns one channel and walks CONV_CHUNK tokens with the last taps - 1 inputs in registers.
 // The tail is brought up to date by the same thread when a sequence's portion is one chunk at most (decoding), else by
@@ -287,7 +287,7 @@ extern "C" int velox_gated_act_mul(const void* gate_up, void* out, int tokens, i
 template <typename T>
 __global__ void __launch_bounds__(256) short_conv_kernel(const T* __restrict__ x, int ld, int C, const float* __restrict__ w, int taps, T* tail,
                                                          const int* __restrict__ slots, const int* __restrict__ cu_q, T* __restrict__ out, int silu,
-                                                         int update_here) {
+                                                         int update_here, const float* __restrict__ bias) {
   const int c = blockIdx.x * blockDim.x + threadIdx.x;
   const int b = blockIdx.z;
   const int lo = cu_q[b], hi = cu_q[b + 1];
@@ -308,9 +308,10 @@ __global__ void __launch_bounds__(256) short_conv_kernel(const T* __restrict__ x
       else if (my_tail) u[j] = to_f32(my_tail[(size_t)(t - lo + taps - 1) * C]);
     }
   }
+  const float start = bias ? bias[c] : 0.f;
   for (int t = first; t < last; ++t) {
     const float now = to_f32(x[(size_t)t * ld + c]);
-    float y = 0.f;
+    float y = start;
 #pragma unroll
     for (int j = 0; j < CONV_TAPS_MAX; ++j)  // (oldest input first; the last column of the weights meets the current token)
       if (j < taps) y += wj[j] * (j == taps - 1 ? now : u[j]);
@@ -349,7 +350,7 @@ __global__ void __launch_bounds__(256) short_conv_tail_kernel(const T* __restric
 }
 
 extern "C" int velox_short_conv(const void* x, int ld, int channels, const float* w, int taps, void* tail, const int* slots, const int* cu_q, void* out,
-                                int num_seqs, int max_q_len, int dtype, int silu, int update_state, hipStream_t stream) {
+                                int num_seqs, int max_q_len, int dtype, int silu, int update_state, const float* bias, hipStream_t stream) {
   if (num_seqs <= 0 || max_q_len <= 0) return 0;
   if (taps < 1 || taps > CONV_TAPS_MAX || num_seqs > 65535) return (int)hipErrorInvalidValue;
   const int chunks = (max_q_len + CONV_CHUNK - 1) / CONV_CHUNK;
@@ -357,9 +358,9 @@ extern "C" int velox_short_conv(const void* x, int ld, int channels, const float
   const dim3 grid((channels + 255) / 256, chunks, num_seqs);
   const int here = (update_state && chunks == 1) ? 1 : 0;
   if (dtype == VELOX_BF16)
-    short_conv_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)x, ld, channels, w, taps, (bf16_t*)tail, slots, cu_q, (bf16_t*)out, silu, here);
+    short_conv_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)x, ld, channels, w, taps, (bf16_t*)tail, slots, cu_q, (bf16_t*)out, silu, here, bias);
   else
-    short_conv_kernel<float><<<grid, 256, 0, stream>>>((const float*)x, ld, channels, w, taps, (float*)tail, slots, cu_q, (float*)out, silu, here);
+    short_conv_kernel<float><<<grid, 256, 0, stream>>>((const float*)x, ld, channels, w, taps, (float*)tail, slots, cu_q, (float*)out, silu, here, bias);
   if (update_state && !here && tail && taps > 1) {
     const dim3 tail_grid((channels + 255) / 256, num_seqs);
     if (dtype == VELOX_BF16) short_conv_tail_kernel<bf16_t><<<tail_grid, 256, 0, stream>>>((const bf16_t*)x, ld, channels, taps, (bf16_t*)tail, slots, cu_q);

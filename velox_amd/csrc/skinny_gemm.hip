@@ -182,7 +182,7 @@ struct RowScale {
   const float* partial;  // [16][blocks] (row m's sums are contiguous), or null: rows are used as they are
   int blocks;
   float inv_width, eps;
-  int act = 0;  // the gate's activation where a kernel stores act(gate) * up: 0 SiLU, 1 the tanh form of GELU
+  int act = 0;  // the gate's activation where a kernel stores act(gate) * up: 0 SiLU, 1 the tanh form of GELU, 2 max(z, 0)
   int ungated = 0;  // the plain product's epilogue: ungated_act(sum + bias, ungated), 0 = none (see common.h)
 };
 
@@ -292,7 +292,7 @@ __global__ void __launch_bounds__(WAVES * 64) skinny_gemm_kernel(const bf16_t* _
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         const float z = sum[j];
-        const float act = rs.act == 1 ? 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))) : z / (1.f + expf(-z));
+        const float act = rs.act == 1 ? 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))) : rs.act == 2 ? fmaxf(z, 0.f) : z / (1.f + expf(-z));
         sum[j] = act * up[j];
       }
     }
@@ -600,12 +600,12 @@ extern "C" int velox_skinny_residual_norm_bf16(const void* a, const void* w, flo
 // pairs: gate/up tile pairs per wave (1 or 2).
 // a_packed != 0: a is in the lanes' order (see packed_row_offset); out_packed (or null; needs n % 64 == 0): room for
 // n / 64 * 1024 elements, the result once more in that order.  Both only with M <= 16.
-// act: 0 SiLU, 1 the tanh form of GELU (velox_skinny_gemm_glu_bf16 is the same with SiLU).
+// act: 0 SiLU, 1 the tanh form of GELU, 2 the rectifier (velox_skinny_gemm_glu_bf16 is the same with SiLU).
 extern "C" int velox_skinny_gemm_glu_act_bf16(const void* a, const void* w, void* out, int m, int n, int k, int waves, int pairs, int packed,
                                               const float* scale_partial, int scale_blocks, float inv_width, float eps, int a_packed,
                                               void* out_packed, int act, hipStream_t stream) {
   if (m <= 0 || n <= 0) return 0;
-  if (act != 0 && act != 1) return -1;
+  if (act < 0 || act > 2) return -1;
   if (k % 64 != 0 || m > 32 || (scale_partial != nullptr && (m > 16 || scale_blocks > ROW_SCALE_BLOCKS))) return -1;
   if ((a_packed || out_packed != nullptr) && (m > 16 || (out_packed != nullptr && n % 64 != 0))) return -1;
   const RowScale rs{scale_partial, scale_blocks, inv_width, eps, act};

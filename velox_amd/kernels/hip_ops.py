@@ -20,7 +20,7 @@ from typing import Tuple, Dict, Optional
 
 import torch
 
-from ..parts.base import DeferredNorm, ReadyInput, ResidualCopy, ResidualSink, SumOf
+from ..parts.base import DeferredNorm, NormedSum, ReadyInput, ResidualCopy, ResidualSink, SumOf
 from . import build
 
 logger = logging.getLogger(__name__)
@@ -91,7 +91,7 @@ class HipOps:
         if arch != build.ARCH:
             raise KernelError(f"the kernels are built for {build.ARCH}; this GPU is {arch}")
         self._core = ctypes.CDLL(build.ensure_core())
-        self._attention: Dict[Tuple[int, bool], ctypes.CDLL] = {}
+        self._attention: Dict[Tuple[int, str], ctypes.CDLL] = {}
         self._declare_core()
         self.num_cus = torch.cuda.get_device_properties(self.device).multi_processor_count
         self.use_library_gemm = True
@@ -145,7 +145,7 @@ class HipOps:
         c.velox_probe_grid_barrier.restype = _I
         c.velox_latent_rotate_write.argtypes = [_P, _I, _P, _I, _I, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _P, _F, _P, _P, _P, _I, _I, _I, _I, _P, _P, _P]
         c.velox_head_linear.argtypes = [_P, _I, _I, _I, _P, _P, _I, _I, _I, _P, _I, _I, _I, _I, _I, _I, _I, _I, _P]
-        c.velox_plain_attention.argtypes = [_P, _I, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _P, _I, _P, _P]
+        c.velox_plain_attention.argtypes = [_P, _I, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _P, _I, _P, _I, _F, _P, _I, _I, _P]
         c.velox_plain_attention.restype = _I
         c.velox_route_top.argtypes = [_P, _P, _P, _I, _I, _I, _I, _I, _P, _I, _I, _F, _P]
         c.velox_routed_plan_elems.argtypes = [_I, _I]
@@ -164,7 +164,16 @@ class HipOps:
         c.velox_stream_norm.argtypes = [_P, _P, _I, _F, _P, _I, _F, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _P]
         c.velox_embed_copies.argtypes = [_P, _P, _I, _P, _I, _I, _I, _F, _I, _P]
         c.velox_gated_act_mul.argtypes = [_P, _P, _I, _I, _I, _I, _P]
-        c.velox_short_conv.argtypes = [_P, _I, _I, _P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _I, _P]
+        c.velox_short_conv.argtypes = [_P, _I, _I, _P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _I, _P, _P]
+        c.velox_sum_norm.argtypes = [_P, _P, _P, _I, _I, _F, _P, _P, _F, _P, _I, _P, _I, _I, _I, _P]
+        c.velox_softcap.argtypes = [_P, ctypes.c_longlong, _F, _F, _P]
+        c.velox_state_space_scan.argtypes = [_P, _I, _I, _P, _I, _I, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P]
+        c.velox_state_space_scratch_elems.argtypes = [_I, _I, _I, _I, _I]
+        c.velox_state_space_scratch_elems.restype = ctypes.c_longlong
+        c.velox_state_space_max_state.argtypes = []
+        c.velox_gated_group_norm.argtypes = [_P, _P, _I, _I, _I, _P, _F, _P, _I, _I, _I, _I, _P]
+        for fn in (c.velox_sum_norm, c.velox_softcap, c.velox_state_space_scan, c.velox_state_space_max_state, c.velox_gated_group_norm):
+            fn.restype = _I
         c.velox_rotate_pad_write.argtypes = [_P, _I, _P, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _P]
         c.velox_recurrence_prepare.argtypes = [_P, _I, _I, _I, _I, _I, _I, _I, _F, _P, _I, _I, _I, _I, _I, _P, _P, _F, _P, _I, _I, _I, _P, _P, _P, _I, _P]
         c.velox_linear_scan.argtypes = [_P, _P, _I, _I, _I, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P]
@@ -200,22 +209,25 @@ class HipOps:
                    c.velox_penalties_from_counts):
             fn.restype = _I
 
-    def attention_library(self, head_dim: int, biased: bool = False) -> ctypes.CDLL:
-        """The attention kernels for one head size; ``biased``: the build whose scores take a bias by distance."""
-        key = (head_dim, bool(biased))
+    def attention_library(self, head_dim: int, biased: bool = False, kept: bool = False, capped: bool = False, gated: bool = False) -> ctypes.CDLL:
+        """The attention kernels for one head size; ``biased``: the build whose scores take a bias by distance; ``kept``: whose
+        windows keep the first keys; ``capped``: whose scores are capped; ``gated``: whose outputs are gated."""
+        key = (head_dim, build.attention_options(biased, kept, capped, gated))
         lib = self._attention.get(key)
         if lib is None:
-            lib = ctypes.CDLL(build.ensure_attention(head_dim, biased=bool(biased)))
-            lib.velox_paged_attention.argtypes = [_P, _I, _P, _P, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _I, _P, _I, _P, _P]
-            lib.velox_attention_biased.restype = _I
+            lib = ctypes.CDLL(build.ensure_attention(head_dim, biased=bool(biased), kept=bool(kept), capped=bool(capped), gated=bool(gated)))
+            lib.velox_paged_attention.argtypes = [_P, _I, _P, _P, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _I, _P, _I, _P,
+                                                  _I, _F, _P, _I, _I, _P]
+            lib.velox_attention_options.restype = _I
             lib.velox_paged_attention.restype = _I
             lib.velox_attention_head_dim.restype = _I
             lib.velox_attention_portion_kernel.argtypes = [_I]
             lib.velox_attention_portion_kernel.restype = None
             if lib.velox_attention_head_dim() != head_dim:
                 raise KernelError(f"attention library for head_dim={head_dim} reports {lib.velox_attention_head_dim()}")
-            if bool(lib.velox_attention_biased()) != bool(biased):
-                raise KernelError(f"attention library for head_dim={head_dim}: built {'with' if lib.velox_attention_biased() else 'without'} the bias by distance")
+            wanted = sum(bit for bit, on in zip((1, 2, 4, 8), (biased, kept, capped, gated)) if on)
+            if lib.velox_attention_options() != wanted:
+                raise KernelError(f"attention library for head_dim={head_dim}: built with the options {lib.velox_attention_options()}, not {wanted}")
             self._attention[key] = lib
         return lib
 
@@ -584,6 +596,81 @@ class HipOps:
                                                       _ptr(rows), _ptr(out), _code(out_dtype), count, hidden, partials, partial_stride, self._stream()), "norm_add_norm")
         return out
 
+    def _sum_norm(self, what, residual, delta, rows, weight, eps, start, out):
+        """``velox_sum_norm`` on ``delta``: None, a tensor, a ``SumOf`` or a ``NormedSum``."""
+        self._check("residual", residual, torch.float32)
+        if residual.dim() != 2:
+            raise KernelError(f"{what}: residual must be [T, H]")
+        tokens, hidden = residual.shape
+        if hidden > 16320:
+            raise KernelError(f"{what}: rows of {hidden} are beyond the kernel (16,320 at most)")
+        normed, weights, scales, term_eps, plain = (), (), (), 1.0, ()
+        if isinstance(delta, NormedSum):
+            normed, weights, scales, term_eps = delta.terms, delta.weights, delta.scales, delta.eps
+            plain = (delta.plain,) if delta.plain is not None else ()
+        elif isinstance(delta, SumOf):
+            plain = (delta.first, delta.second)
+        elif delta is not None:
+            if not isinstance(delta, torch.Tensor):
+                raise KernelError(f"{what}: a {type(delta).__name__} cannot be added here")
+            plain = (delta,)
+        if len(normed) > 2 or len(normed) != len(weights) or len(normed) != len(scales) or len(plain) > 2:
+            raise KernelError(f"{what}: at most two terms with norms of their own and two without")
+        described = (ctypes.c_longlong * 20)()
+        factors = (ctypes.c_float * 4)()
+        for first, terms in ((0, normed), (2, plain)):
+            for i, term in enumerate(terms):
+                partials, stride = 1, 0
+                if term.dim() == 3:
+                    partials, stride = term.shape[0], tokens * hidden
+                    self._check("partial sums of a term", term, torch.float32, (partials, tokens, hidden))
+                else:
+                    self._check("term", term, None, (tokens, hidden))
+                norm_weight = 0
+                if first == 0:
+                    self._check("weight of a term's norm", weights[i], torch.float32, (hidden,))
+                    norm_weight = weights[i].data_ptr()
+                    factors[i] = float(scales[i])
+                described[5 * (first + i):5 * (first + i) + 5] = [term.data_ptr(), _code(term.dtype), partials, stride, norm_weight]
+        if weight is not None:
+            self._check("weight", weight, torch.float32, (hidden,))
+        count = tokens
+        if rows is not None:
+            self._check("rows", rows, torch.int32)
+            count = rows.shape[0]
+        status = self._core.velox_sum_norm(_ptr(residual), ctypes.cast(described, _P), ctypes.cast(factors, _P), len(normed), len(plain), float(term_eps), _ptr(rows),
+                                           _ptr(weight), float(eps), _ptr(start), _code(start.dtype) if start is not None else 0, _ptr(out), _code(out.dtype),
+                                           count, hidden, self._stream())
+        self._launched(status, what)
+        return out
+
+    def normed_sum_norm(self, residual: torch.Tensor, delta: NormedSum, weight: torch.Tensor, eps: float, out_dtype: torch.dtype,
+                        rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """``residual += delta`` in place (the terms' own norms and all sums in float32), then ``residual * rsqrt(mean(residual^2) + eps) *
+        weight`` in ``out_dtype``.  ``rows``: nothing is changed and only those rows are worked."""
+        count = residual.shape[0] if rows is None else rows.shape[0]
+        out = torch.empty((count, residual.shape[-1]), dtype=out_dtype, device=self.device)
+        return self._sum_norm("normed_sum_norm", residual, delta, rows, weight, eps, None, out)
+
+    def join_rows(self, residual: torch.Tensor, delta, start: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:
+        """``[residual + delta ; start]`` in ``out_dtype``, [T, 2 H], and the residual is cleared (what is made of the joined rows
+        becomes the residual).  ``delta``: None, a tensor (or float32 partial sums), a ``SumOf`` or a ``NormedSum``; ``start`` [T, H]."""
+        self._check("start", start, None, tuple(residual.shape))
+        out = torch.empty((residual.shape[0], 2 * residual.shape[1]), dtype=out_dtype, device=self.device)
+        return self._sum_norm("join_rows", residual, delta, None, None, 1.0, start, out)
+
+    def kept_copy(self, x: torch.Tensor, dtype: torch.dtype) -> torch.Tensor:
+        """A float32 ``[T, H]`` tensor in ``dtype``, in memory of its own."""
+        return torch.mul(x, 1.0) if dtype == torch.float32 else self.add_cast(x, None, dtype)
+
+    def softcap_(self, x: torch.Tensor, cap: float, scale: float = 1.0) -> torch.Tensor:
+        """``x = cap * tanh(scale * x / cap)`` in place, float32."""
+        self._check("x", x, torch.float32)
+        if not cap > 0:
+            raise KernelError(f"softcap: the cap must be positive, got {cap}")
+        self._launched(self._core.velox_softcap(_ptr(x), x.numel(), float(scale), float(cap), self._stream()), "softcap")
+        return x
+
     def poly_norm(self, x: torch.Tensor, coefficients: torch.Tensor, eps: float) -> torch.Tensor:
         """``a N(x) + b N(x^2) + c N(x^3) + e`` per row, ``N(y) = y * rsqrt(mean(y^2) + eps)``; ``coefficients`` = (a, b, c, e), float32 on the
         device; float32 arithmetic with one rounding."""
@@ -598,7 +685,7 @@ class HipOps:
     def qk_norm_write(self, qkv, num_heads, num_kv_heads, dim, vdim, cached_dim, q_norm, k_norm, whole, eps, q_temp, positions, first_values, mix_weight,
                       slot_mapping, k_cache, v_cache, block_size, write_kv=True) -> torch.Tensor:
         """Rows of ``qkv`` hold ``num_heads`` queries and ``num_kv_heads`` keys of ``dim`` channels and ``num_kv_heads`` values
-        of ``vdim``.  Queries and keys pass an RMS norm (``whole``: over all heads at once, weights of that size; else per head
+        of ``vdim`` (and possibly columns of others behind them).  Queries and keys pass an RMS norm (``whole``: over all heads at once, weights of that size; else per head
         with one weight of ``dim``), the queries the temperature ``q_temp = (coef, every)``; values are blended with
         ``first_values = (tensor, first column)`` by ``mix_weight`` (one float32 on the device).  Returns the queries as the
         attention kernels read them, ``[T, num_heads * cached_dim]``; keys and values go into the cache at that head size,
@@ -607,7 +694,9 @@ class HipOps:
             raise KernelError("qk_norm_write: rows are [T, width]")
         tokens, width = qkv.shape
         q_size, k_size, v_size = num_heads * dim, num_kv_heads * dim, num_kv_heads * vdim
-        self._check("qkv", qkv, None, (tokens, q_size + k_size + v_size))
+        self._check("qkv", qkv)
+        if width < q_size + k_size + v_size:
+            raise KernelError(f"qk_norm_write: rows of {width} elements do not hold {q_size} + {k_size} + {v_size}")
         self._check("positions", positions, torch.int32, (tokens,))
         self._check("q_norm", q_norm, torch.float32, (q_size if whole else dim,))
         self._check("k_norm", k_norm, torch.float32, (k_size if whole else dim,))
@@ -831,14 +920,16 @@ class HipOps:
         self._launched(status, "skinny_gemm")
         return out
 
+    _GATED_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "relu": 2}
+
     def linear_gated_act(self, x: torch.Tensor, gate_up_weight: torch.Tensor, out_dtype: torch.dtype, activation: str) -> torch.Tensor:
-        """``act(x Wgate^T) * (x Wup^T)`` for ``W = [Wgate; Wup]`` and ``activation`` ``"silu"`` or ``"gelu_tanh"``: one kernel for
+        """``act(x Wgate^T) * (x Wup^T)`` for ``W = [Wgate; Wup]`` and ``activation`` ``"silu"``, ``"gelu_tanh"`` or ``"relu"``: one kernel for
         decode-sized bfloat16 batches (see ``linear_silu_mul``), else the product followed by the activation's kernel."""
         return self.linear_silu_mul(x, gate_up_weight, out_dtype, activation=activation)
 
     def linear_silu_mul(self, x: torch.Tensor, gate_up_weight: torch.Tensor, out_dtype: torch.dtype, waves: Optional[int] = None, pairs: Optional[int] = None, packed: Optional[torch.Tensor] = None,
                         activation: str = "silu") -> torch.Tensor:
-        """``silu(x Wgate^T) * (x Wup^T)`` for ``W = [Wgate; Wup]`` (``activation="gelu_tanh"``: the tanh form of GELU in SiLU's place).  Decode-sized bfloat16 batches run as one kernel that
+        """``silu(x Wgate^T) * (x Wup^T)`` for ``W = [Wgate; Wup]`` (``activation="gelu_tanh"``: the tanh form of GELU in SiLU's place; ``"relu"``: the rectifier).  Decode-sized bfloat16 batches run as one kernel that
         never writes the [M, 2I] product (up to 16 rows on any weight, 17 .. 64 rows on a registered one); everything else
         is the product followed by the SiLU kernel.  ``waves`` and ``pairs`` override the launch shape the wrapper would
         pick (up to 16 rows: waves per workgroup and gate/up tile pairs per wave; 17 .. 64 rows: ``pairs`` = tile pairs per
@@ -854,8 +945,8 @@ class HipOps:
         two_n = gate_up_weight.shape[0]
         fused = (self.use_skinny_gemm and x.dtype == torch.bfloat16 and gate_up_weight.dtype == torch.bfloat16 and out_dtype == torch.bfloat16
                  and m <= 16 and k % 64 == 0 and two_n % 2 == 0 and x.dim() == 2 and gate_up_weight.shape[1] == k)
-        if activation not in ("silu", "gelu_tanh"):
-            raise KernelError(f"linear_silu_mul: activation {activation!r} is not built ('silu' or 'gelu_tanh')")
+        if activation not in self._GATED_ACTIVATIONS:
+            raise KernelError(f"linear_silu_mul: activation {activation!r} is not built ({', '.join(self._GATED_ACTIVATIONS)})")
         if (not fused and activation == "silu" and deferred is None and self.use_skinny_gemm and x.dim() == 2 and 16 < m <= 64 and k % 64 == 0 and two_n % 2 == 0
                 and x.dtype == torch.bfloat16 and gate_up_weight.dtype == torch.bfloat16 and out_dtype == torch.bfloat16
                 and gate_up_weight.shape[1] == k and packed is not None):
@@ -890,7 +981,7 @@ class HipOps:
         out_packed = self._room_for_packed_rows(m, n)
         status = self._core.velox_skinny_gemm_glu_act_bf16(_ptr(x if x_packed is None else x_packed), _ptr(packed if packed is not None else gate_up_weight), _ptr(out),
                                                            m, n, k, int(waves), int(pairs), 1 if packed is not None else 0, *self._scale_args(deferred),
-                                                           int(x_packed is not None), _ptr(out_packed), 1 if activation == "gelu_tanh" else 0, self._stream())
+                                                           int(x_packed is not None), _ptr(out_packed), self._GATED_ACTIVATIONS[activation], self._stream())
         self._launched(status, "skinny_gemm_glu")
         if out_packed is not None:
             out._velox_packed_rows = (out_packed, out._version)
@@ -976,11 +1067,11 @@ class HipOps:
         return out
 
     def gated_act_mul(self, gate_up: torch.Tensor, activation: str) -> torch.Tensor:
-        """``act(gate) * up`` of ``[T, 2 * I]`` (gate first), ``activation`` ``"silu"`` or ``"gelu_tanh"``; float32 inside."""
+        """``act(gate) * up`` of ``[T, 2 * I]`` (gate first), ``activation`` ``"silu"``, ``"gelu_tanh"`` or ``"relu"``; float32 inside."""
         self._check("gate_up", gate_up)
-        kinds = {"silu": 0, "gelu_tanh": 1}
+        kinds = self._GATED_ACTIVATIONS
         if gate_up.dim() != 2 or gate_up.shape[1] % 2 != 0 or activation not in kinds:
-            raise KernelError("gated_act_mul: expected [T, 2 * intermediate] and 'silu' or 'gelu_tanh'")
+            raise KernelError("gated_act_mul: expected [T, 2 * intermediate] and 'silu', 'gelu_tanh' or 'relu'")
         tokens, inter = gate_up.shape[0], gate_up.shape[1] // 2
         out = torch.empty((tokens, inter), dtype=gate_up.dtype, device=self.device)
         for first in range(0, tokens, 65535):
@@ -989,14 +1080,16 @@ class HipOps:
                                                           _code(gate_up.dtype), kinds[activation], self._stream()), "gated_act_mul")
         return out
 
-    def short_conv(self, x, channels, weight, tail, slots, cu_q, max_q_len, activation="none", update_state=True):
-        """The first ``channels`` columns of ``x`` [T, >= channels] through ``y_t = sum_j w[:, j] u_(t - taps + 1 + j)`` per sequence
-        (``weight`` float32 [channels, taps]); the inputs before a portion's start come from ``tail[slot]`` ([taps - 1, channels],
+    def short_conv(self, x, channels, weight, tail, slots, cu_q, max_q_len, activation="none", update_state=True, first=0, bias=None):
+        """The ``channels`` columns of ``x`` [T, >= first + channels] from column ``first`` on through ``y_t = sum_j w[:, j] u_(t - taps + 1 + j)
+        (+ bias)`` per sequence (``weight`` float32 [channels, taps], ``bias`` float32 [channels]); the inputs before a portion's start come from ``tail[slot]`` ([taps - 1, channels],
         oldest first, the dtype of ``x``; None: zeros), which is brought up to date unless ``update_state`` is false.
         ``activation``: ``"none"`` or ``"silu"``.  Returns [T, channels] in x's dtype."""
         self._check("x", x)
-        if x.dim() != 2 or x.shape[1] < channels:
-            raise KernelError(f"short_conv: x {tuple(x.shape)} has fewer than {channels} columns")
+        if x.dim() != 2 or first < 0 or x.shape[1] < first + channels:
+            raise KernelError(f"short_conv: x {tuple(x.shape)} has fewer than {first} + {channels} columns")
+        if bias is not None:
+            self._check("bias", bias, torch.float32, (channels,))
         if weight.dim() != 2:
             raise KernelError("short_conv: the weights must be [channels, taps]")
         taps = weight.shape[1]
@@ -1014,8 +1107,8 @@ class HipOps:
         if activation not in ("none", "silu"):
             raise KernelError(f"short_conv: activation {activation!r}")
         out = torch.empty((x.shape[0], channels), dtype=x.dtype, device=self.device)
-        status = self._core.velox_short_conv(_ptr(x), x.shape[1], int(channels), _ptr(weight), taps, _ptr(tail), _ptr(slots), _ptr(cu_q), _ptr(out),
-                                             slots.shape[0], int(max_q_len), _code(x.dtype), int(activation == "silu"), int(bool(update_state)), self._stream())
+        status = self._core.velox_short_conv(_P(x.data_ptr() + first * x.element_size()), x.shape[1], int(channels), _ptr(weight), taps, _ptr(tail), _ptr(slots), _ptr(cu_q), _ptr(out),
+                                             slots.shape[0], int(max_q_len), _code(x.dtype), int(activation == "silu"), int(bool(update_state)), _ptr(bias), self._stream())
         self._launched(status, "short_conv")
         return out
 
@@ -1233,6 +1326,63 @@ class HipOps:
                                                   int(gate_at), 0 if gate_kind == "silu" else 1, _ptr(out), _code(out_dtype), tokens, int(heads), int(vdim),
                                                   int(weight.numel() != vdim), self._stream())
         self._launched(status, "gated_head_norm")
+        return out
+
+    def state_space_supports(self, size: int, vdim: int) -> None:
+        """Raises if the kernels cannot hold a head's state of ``size x vdim`` numbers."""
+        if size > self._core.velox_state_space_max_state():
+            raise KernelError(f"state_space_scan: {size} entries per column of a head's state are beyond the kernel ({self._core.velox_state_space_max_state()} at most)")
+
+    STATE_SPACE_CHUNK_TOKENS = 32  # portions at least this long are worked in chunks
+
+    def state_space_scan(self, xbc, step_source, step_at, dt_bias, rate, skip, state, slots, cu_q, max_q_len, heads, groups, size, vdim,
+                         chunked: Optional[bool] = None):
+        """Rows of ``xbc`` hold x (``heads * vdim``), B and C (``groups * size`` each), a token's dt stands in ``step_source`` from column ``step_at``
+        on.  With ``d = softplus(dt + dt_bias)``, per sequence and head from ``state[slot, head]`` ([size, vdim] float32), which is written
+        back: ``S <- exp(-rate d) S + d B x^T``; ``y = S^T C + skip x``.  Float32 [T, heads * vdim].  Steps with a long portion are worked
+        in chunks of 64 tokens on the matrix cores, others token by token; ``chunked`` decides it for a test."""
+        self._check("xbc", xbc)
+        if xbc.dim() != 2 or groups < 1 or heads % groups != 0 or xbc.shape[1] != heads * vdim + 2 * groups * size:
+            raise KernelError(f"state_space_scan: rows of {heads} * {vdim} + 2 * {groups} * {size} columns expected, got {tuple(xbc.shape)}")
+        tokens = xbc.shape[0]
+        self._check("step_source", step_source, xbc.dtype)
+        if step_source.dim() != 2 or step_source.shape[0] != tokens or step_at < 0 or step_at + heads > step_source.shape[1]:
+            raise KernelError("state_space_scan: the step sizes do not lie within their source")
+        for name, t in (("dt_bias", dt_bias), ("rate", rate), ("skip", skip)):
+            self._check(name, t, torch.float32, (heads,))
+        self._check("state", state, torch.float32)
+        if state.dim() != 4 or tuple(state.shape[1:]) != (heads, size, vdim):
+            raise KernelError(f"state_space_scan: the state must be [slots, {heads}, {size}, {vdim}], got {tuple(state.shape)}")
+        self._check("slots", slots, torch.int32)
+        self._check("cu_q", cu_q, torch.int32, (slots.shape[0] + 1,))
+        if not 1 <= max_q_len <= tokens:
+            raise KernelError(f"state_space_scan: max_q_len={max_q_len} outside [1, {tokens}]")
+        self.state_space_supports(size, vdim)
+        out = torch.empty((tokens, heads * vdim), dtype=torch.float32, device=self.device)
+        scratch = None
+        if chunked or (chunked is None and max_q_len >= self.STATE_SPACE_CHUNK_TOKENS):
+            elems = int(self._core.velox_state_space_scratch_elems(tokens, slots.shape[0], int(heads), int(size), int(vdim)))
+            scratch = torch.empty(elems, dtype=torch.float32, device=self.device)
+        self._launched(self._core.velox_state_space_scan(_ptr(xbc), _code(xbc.dtype), xbc.shape[1], _ptr(step_source), step_source.shape[1], int(step_at),
+                                                         _ptr(dt_bias), _ptr(rate), _ptr(skip), _ptr(state), _ptr(slots), _ptr(cu_q), _ptr(out), _ptr(scratch),
+                                                         tokens, slots.shape[0], int(max_q_len), int(heads), int(groups), int(size), int(vdim), self._stream()),
+                       "state_space_scan")
+        return out
+
+    def gated_group_norm(self, read, gate_source, gate_at, weight, eps, groups, out_dtype):
+        """``y = read * silu(z)`` with ``z`` the columns of ``gate_source`` from ``gate_at`` on; each of ``groups`` equal parts of a row divided by its
+        root mean square (``eps`` inside the root), times ``weight``; [T, width] in ``out_dtype``."""
+        self._check("read", read, torch.float32)
+        if read.dim() != 2 or groups < 1 or read.shape[1] % groups != 0:
+            raise KernelError(f"gated_group_norm: rows {tuple(read.shape)} do not fall into {groups} equal parts")
+        tokens, width = read.shape
+        self._check("weight", weight, torch.float32, (width,))
+        self._check("gate_source", gate_source)
+        if gate_source.dim() != 2 or gate_source.shape[0] != tokens or gate_at < 0 or gate_at + width > gate_source.shape[1]:
+            raise KernelError("gated_group_norm: the gate's columns do not lie within its source")
+        out = torch.empty((tokens, width), dtype=out_dtype, device=self.device)
+        self._launched(self._core.velox_gated_group_norm(_ptr(read), _ptr(gate_source), _code(gate_source.dtype), gate_source.shape[1], int(gate_at), _ptr(weight),
+                                                         float(eps), _ptr(out), _code(out_dtype), tokens, width, int(groups), self._stream()), "gated_group_norm")
         return out
 
     # -- rotary + cache write ---------------------------------------------------------------------
@@ -1595,7 +1745,8 @@ class HipOps:
 
     def paged_attention(self, qkv, num_heads, num_kv_heads, head_dim, k_cache, v_cache, block_size, block_tables, cu_q, kv_lens,
                         max_q_len, max_kv_len, scale, window, all_decode, workspace, splits: Optional[int] = None, decode_prefix: int = 0,
-                        portions_max_kv_len: Optional[int] = None, distance_bias: Optional[torch.Tensor] = None, sinks: Optional[torch.Tensor] = None):
+                        portions_max_kv_len: Optional[int] = None, distance_bias: Optional[torch.Tensor] = None, sinks: Optional[torch.Tensor] = None,
+                        keep_first: int = 0, softcap: Optional[float] = None, gate: Optional[Tuple[torch.Tensor, int, int]] = None):
         """Attention of every token of the step over its sequence's keys in the cache.  ``decode_prefix``: how many of the
         first sequences bring exactly one token (the engine puts decoded tokens before portions of prompts).  In a mixed
         step those run through the streaming kernel with their keys split over workgroups, the others through the
@@ -1604,8 +1755,24 @@ class HipOps:
         ``distance_bias``: float32 ``[num_heads, L]``, added to the scaled scores: a key ``n`` positions behind the query reads
         column ``min(n, L - 1)`` of its query head's row (the kernels' build for it is loaded by ``attention_library(d, True)``).
         ``sinks``: float32 ``[num_heads]``; ``exp(sinks[h])`` joins the denominator of every softmax of head ``h`` (a sink has no key
-        and no value and is not scaled)."""
+        and no value and is not scaled).  ``keep_first`` beside a window: so many first tokens of a sequence are seen whatever the
+        window.  ``softcap``: a scaled score ``s`` becomes ``softcap * tanh(s / softcap)`` (before the bias).  ``gate = (source, first column, channels)``:
+        head ``h``'s output times ``sigmoid`` of the source's columns, ``channels`` per head (channels beyond are left alone) or one per head
+        with ``channels`` = 0.  (Each of the three has a build of the kernels: ``attention_library``.)"""
         tokens = qkv.shape[0]
+        keep_first = int(keep_first) if window else 0
+        gate_at, gate_stride, gate_channels = 0, 0, 0
+        if gate is not None:
+            gate, gate_at, gate_channels = gate
+            self._check("gate", gate, qkv.dtype)
+            gate_stride = gate.shape[1] if gate.dim() == 2 else 0
+            if gate.dim() != 2 or gate.shape[0] != tokens or gate_at < 0 or not 0 <= gate_channels <= head_dim or gate_at + num_heads * max(gate_channels, 1) > gate_stride:
+                raise KernelError("paged_attention: the gate's columns do not lie within its source")
+        if keep_first < 0 or (softcap is not None and not softcap > 0):
+            raise KernelError(f"paged_attention: keep_first={keep_first} must not be negative, softcap={softcap} must be positive")
+
+        def gate_rows(first_token: int):
+            return _P(0) if gate is None else _P(gate.data_ptr() + (first_token * gate_stride + gate_at) * gate.element_size())
         if sinks is not None:
             self._check("sinks", sinks, torch.float32, (num_heads,))
         width = qkv.shape[1] if qkv.dim() == 2 else -1  # rows may carry keys and values after the queries
@@ -1647,10 +1814,10 @@ class HipOps:
             status = self._core.velox_plain_attention(_ptr(qkv), width, _ptr(k_cache), _ptr(v_cache), _ptr(block_tables), block_tables.shape[1], _ptr(cu_q),
                                                       _ptr(kv_lens), _ptr(out), num_seqs, tokens, num_heads, num_kv_heads, head_dim,
                                                       block_size.bit_length() - 1, float(scale), int(window or 0), _code(qkv.dtype), _ptr(distance_bias), bias_len,
-                                                      _ptr(sinks), self._stream())
+                                                      _ptr(sinks), keep_first, float(softcap or 0.0), gate_rows(0), gate_stride, int(gate_channels), self._stream())
             self._launched(status, "plain_attention")
             return out
-        lib = self.attention_library(head_dim, distance_bias is not None)
+        lib = self.attention_library(head_dim, distance_bias is not None, kept=keep_first > 0, capped=softcap is not None, gated=gate is not None)
         group = num_heads // num_kv_heads
 
         def launch(first_seq: int, count: int, first_token: int, num_tokens: int, longest: int, decode_only: bool, splits: Optional[int]) -> None:
@@ -1659,9 +1826,11 @@ class HipOps:
             # counts rows from its first sequence and takes the slices.
             row_tiles = (longest * group + 63) // 64
             if splits is None:
-                splits = self.choose_splits(count, num_kv_heads, row_tiles, max_kv_len, decode_only)
+                # (a window bounds the keys a row block walks, however long the sequence)
+                seen = window + keep_first + longest if window else max_kv_len
+                splits = self.choose_splits(count, num_kv_heads, row_tiles, min(max_kv_len, seen), decode_only)
                 if not decode_only:
-                    splits = self.choose_portion_splits(num_tokens, group, num_kv_heads, min(max_kv_len, portions_max_kv_len or max_kv_len))
+                    splits = self.choose_portion_splits(num_tokens, group, num_kv_heads, min(max_kv_len, portions_max_kv_len or max_kv_len, seen))
             if count * splits > 65535:
                 raise KernelError(f"{count} sequences x {splits} splits exceed the launch grid")
             part_o = part_lse = None
@@ -1677,7 +1846,8 @@ class HipOps:
                 _ptr(cu_q[first_seq:]), _ptr(kv_lens[first_seq:]), _ptr(rows_out), _ptr(part_o), _ptr(part_lse), count,
                 num_tokens if decode_only else tokens, longest, int(max_kv_len), num_heads, num_kv_heads,
                 block_size.bit_length() - 1, float(scale), int(window or 0), splits, 0 if decode_only else first_token, _code(qkv.dtype),
-                _ptr(distance_bias), bias_len, _ptr(sinks), self._stream())
+                _ptr(distance_bias), bias_len, _ptr(sinks), keep_first, float(softcap or 0.0), gate_rows(first_token if decode_only else 0), gate_stride,
+                int(gate_channels), self._stream())
             self._launched(status, "paged_attention")
 
         if not all_decode and splits is None and 0 < decode_prefix < num_seqs and group <= 16:

@@ -25,10 +25,11 @@ from .base import PAGE, Mixer, PagedNeed, Param, PositionEncoding, fused_rows, r
 SHORT_CONTEXT_KEYS = 384
 
 
-def kv_pages(num_kv_heads: int, head_dim: int, window: Optional[int] = None) -> PagedNeed:
+def kv_pages(num_kv_heads: int, head_dim: int, window: Optional[int] = None, keep_first: int = 0) -> PagedNeed:
     """What attention keeps per page: keys ``[kv_heads, page, head_dim]`` and values transposed, ``[kv_heads, head_dim,
     page]`` (a run of consecutive keys for one channel is then one contiguous access for the kernels' second product)."""
-    return PagedNeed((("k", (int(num_kv_heads), PAGE, int(head_dim)), None), ("v", (int(num_kv_heads), int(head_dim), PAGE), None)), window)
+    return PagedNeed((("k", (int(num_kv_heads), PAGE, int(head_dim)), None), ("v", (int(num_kv_heads), int(head_dim), PAGE), None)), window,
+                     int(keep_first) if window is not None else 0)
 
 
 class AttentionMixer(Mixer):

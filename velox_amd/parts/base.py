@@ -2,7 +2,7 @@
 
 A *part* owns tensors (declared as :class:`Param`) and one piece of arithmetic.
 It is given its sizes and constants at construction and never learns which
-model it sits in.  Six families exist, each with a registry from a kind name to a
+model it sits in.  Seven families exist, each with a registry from a kind name to a
 class so that an architecture (or a test) can add its own:
 
 ``Mixer``
@@ -19,6 +19,8 @@ class so that an architecture (or a test) can add its own:
 
 ``Embedding``
     token ids -> the residual stream, float32 ``[T, H]``.
+``PassInput``
+    what stands before every pass of a loop over layers.
 ``OutputHead``
     normalised rows -> float32 logits ``[R, vocab]``.
 
@@ -157,10 +159,12 @@ class PagedNeed:
 
     ``window`` = None keeps every token; an integer keeps the last ``window`` of them (a query at position p reads
     positions p-window+1 .. p), so pages wholly behind the window can be given back while the request is still running.
+    ``keep_first`` beside a window: the first ``keep_first`` tokens are read by every query and their pages stay.
     """
 
     tensors: Tuple[Tuple[str, Tuple[int, ...], Optional[torch.dtype]], ...]
     window: Optional[int] = None
+    keep_first: int = 0
 
     def __post_init__(self) -> None:
         if not self.tensors:
@@ -170,6 +174,8 @@ class PagedNeed:
                 raise ValueError(f"page tensor {name!r}: its shape {tuple(shape)} must hold PAGE exactly once")
         if self.window is not None and self.window < 1:
             raise ValueError(f"window={self.window} must be at least 1")
+        if self.keep_first < 0:
+            raise ValueError(f"keep_first={self.keep_first} must not be negative")
 
 
 @dataclass(frozen=True)
@@ -273,6 +279,19 @@ class NormedDelta:
 
 
 @dataclass
+class NormedSum:
+    """What sub-layers side by side hand on when some of their outputs still have norms of their own to pass: the block's
+    output is ``sum_i scales[i] * normalise(terms[i]) * weights[i] + plain``, with ``normalise(y) = y * rsqrt(mean(y^2) + eps)``.
+    Handed on in a delta's place; the norm that reads the residual next takes all of it in one kernel, in float32."""
+
+    terms: Tuple[torch.Tensor, ...]  # each [T, H] or float32 partial sums [S, T, H]
+    weights: Tuple[torch.Tensor, ...]  # float32 [H] each
+    scales: Tuple[float, ...]
+    eps: float
+    plain: Optional[torch.Tensor] = None  # [T, H] or float32 partial sums [S, T, H]
+
+
+@dataclass
 class ReadyInput:
     """What a sub-layer hands on when its last kernel has added its normed output to the residual AND taken the next
     norm: ``x`` is that norm's result, [T, H] in the run dtype.  It can only go to the norm it was made for."""
@@ -328,7 +347,8 @@ class Norm(Part):
 
         ``delta`` is [T, H] or float32 partial sums [S, T, H], which are added first to last, or a ``SumOf`` two such
         terms, or a ``DeferredNorm`` made for this very norm (then the residual is up to date and the ``DeferredNorm`` itself is what comes back),
-        or a ``NormedDelta`` (the delta passes a norm of its own first) or a ``ReadyInput`` made for this norm (its tensor comes back).
+        or a ``NormedDelta`` (the delta passes a norm of its own first) or a ``NormedSum`` (several do) or a ``ReadyInput`` made for this
+        norm (its tensor comes back).
         With ``rows`` None: ``residual += delta`` in place (delta may be None) and the
         normalised residual comes back in the run dtype, [T, H].  With ``rows`` (int32
         [R]): nothing is changed and ``normalise(residual[rows] + delta[rows])`` comes back.
@@ -360,6 +380,16 @@ class Embedding(Part):
     def forward(self, token_ids: torch.Tensor, ctx) -> torch.Tensor:
         """int32 ``[T]`` -> the residual stream before the first block, float32 ``[T, H]`` (a fresh tensor: blocks
         update it in place)."""
+        raise NotImplementedError
+
+
+class PassInput(Part):
+    """What stands before the first layer of every pass of a loop over layers: it makes the pass's residual of the
+    residual so far and of the embedding output."""
+
+    def forward(self, residual: torch.Tensor, pending, start: torch.Tensor, ctx):
+        """Takes the residual with what is pending on it and the embedding output; returns the new ``pending`` on a
+        ``residual`` that it has set (in place) such that the two together are the pass's residual."""
         raise NotImplementedError
 
 
@@ -400,8 +430,9 @@ _POSITIONS: Dict[str, Callable[..., PositionEncoding]] = {}
 _EMBEDDINGS: Dict[str, Callable[..., Embedding]] = {}
 _HEADS: Dict[str, Callable[..., OutputHead]] = {}
 _ARRANGEMENTS: Dict[str, Callable[..., Block]] = {}
+_PASS_INPUTS: Dict[str, Callable[..., PassInput]] = {}
 _TABLES = {"mixer": _MIXERS, "feed_forward": _FEED_FORWARDS, "norm": _NORMS, "position": _POSITIONS, "embedding": _EMBEDDINGS, "head": _HEADS,
-           "arrangement": _ARRANGEMENTS}
+           "arrangement": _ARRANGEMENTS, "pass_input": _PASS_INPUTS}
 
 
 def register_part(family: str, kind: str, factory: Callable[..., Part]) -> None:

@@ -14,19 +14,21 @@ before and one after each sub-layer.  The norm behind a sub-layer, the residual 
 sub-layer are one kernel: the output travels as a ``NormedDelta``.
 
 ``ParallelBlock`` (not in the reference): ``n = norm(h); h = h + (mixer(n) + ff(n))``, one norm that both
-sub-layers read.  It hands both outputs on as a ``SumOf``, which the next norm's kernel adds up in float32.
+sub-layers read.  It hands both outputs on as a ``SumOf`` (or, when the mixer's output still has norms to pass, as the
+mixer's ``NormedSum`` with the other output beside it), which the next norm's kernel adds up in float32.
 
 ``HyperConnectionBlock`` (not in the reference): pre-norm sub-layers over several copies of the residual that are read
 through learned weights and mixed by a learned matrix at every sub-layer.
 """
 from __future__ import annotations
 
+from dataclasses import replace
 from typing import Optional, Tuple
 
 import torch
 
 from .base import (
-    Block, FeedForward, Mixer, Norm, NormedDelta, OutputNormSink, Part, PartSpec, ResidualCopy, ResidualSink, StreamUpdate, SumOf, make_part, register_arrangement,
+    Block, FeedForward, Mixer, Norm, NormedDelta, NormedSum, OutputNormSink, Part, PartSpec, ResidualCopy, ResidualSink, StreamUpdate, SumOf, make_part, register_arrangement,
 )
 
 
@@ -90,6 +92,8 @@ class ParallelBlock(Block):
         other = self.feed_forward.forward(normed, ctx)
         if other is None:
             return mixed
+        if isinstance(mixed, NormedSum):
+            return replace(mixed, plain=other)
         if other.dim() == 3:
             mixed, other = other, mixed  # (the term that may be partial sums goes first)
         if other.dim() == 3:

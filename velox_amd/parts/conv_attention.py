@@ -14,6 +14,10 @@ Beside ``parts.attention`` and ``parts.normed_attention`` this mixer has
 * ``post_norm_eps``: queries and keys are divided by their root mean square per head BEHIND the rotation (no weight);
 * ``values_are_keys``: there is no value product, a key head's values are its keys as the projection left them, before
   rotation and norm (the cache still holds both: what is written as a key is no longer what is written as a value);
+* ``softcap``: the scaled score ``s`` becomes ``softcap * tanh(s / softcap)``;
+* ``gate="channel"``: the concatenated heads times ``sigmoid(W_g x)`` element by element, before the output projection; the gate's
+  rows stand in the same product as q, k and v (and pass no convolution), and the attention kernels apply it where they
+  finish a row;
 * ``sink_score``: one more key in every softmax, of that score and without a value (0: one is added to the denominator).
 
 How it meets the kernels: as for ``NormedAttentionMixer`` the paged cache holds heads of ``D = ceil16(max(dim, vdim))``
@@ -34,9 +38,9 @@ class ConvAttentionMixer(Mixer):
     def __init__(self, prefix: str, hidden_size: int, num_heads: int, num_kv_heads: int, dim: int, vdim: int, scale: float,
                  window: Optional[int] = None, conv_taps: int = 0, qkv_bias: bool = True, out_bias: bool = True,
                  position: Optional[PositionEncoding] = None, names: Tuple[Tuple[str, str], ...] = (), post_norm_eps: Optional[float] = None,
-                 values_are_keys: bool = False, sink_score: Optional[float] = None) -> None:
+                 values_are_keys: bool = False, sink_score: Optional[float] = None, softcap: Optional[float] = None, gate: Optional[str] = None) -> None:
         """``conv_taps``: columns of the convolution's weights (0 or 1 column less than 2: 0 = no convolution);
-        ``names``: pairs (tensor, name below the prefix) that replace the default names ``q``, ``k``, ``v``, ``o``; a
+        ``names``: pairs (tensor, name below the prefix) that replace the default names ``q``, ``k``, ``v``, ``g``, ``o``; a
         bias is the tensor's name with ``.b`` added, a convolution's weights with ``.conv``."""
         super().__init__(prefix)
         if num_heads % num_kv_heads != 0:
@@ -51,6 +55,12 @@ class ConvAttentionMixer(Mixer):
             raise ValueError("values that are the keys have the keys' size and come without a convolution")
         if post_norm_eps is not None and not float(post_norm_eps) > 0:
             raise ValueError("post_norm_eps must be positive")
+        if softcap is not None and not float(softcap) > 0:
+            raise ValueError(f"softcap={softcap} must be positive")
+        if gate not in (None, "channel"):
+            raise ValueError(f"gate must be None or 'channel', got {gate!r}")
+        self.softcap = float(softcap) if softcap is not None else None
+        self.gate = gate
         self.post_norm_eps = float(post_norm_eps) if post_norm_eps is not None else None
         self.values_are_keys = bool(values_are_keys)
         self.sink_score = float(sink_score) if sink_score is not None else None
@@ -70,12 +80,14 @@ class ConvAttentionMixer(Mixer):
         self.position = position
         if position is not None and getattr(position, "rotary_dim", 0) > self.dim:
             raise ValueError(f"the rotation spans {position.rotary_dim} channels but a query head has {self.dim}")
-        self.names = {"q": "q", "k": "k", "v": "v", "o": "o"}
+        self.names = {"q": "q", "k": "k", "v": "v", "g": "g", "o": "o"}
         self.names.update(dict(names))
         self.q_size = self.num_heads * self.dim
         self.k_size = self.num_kv_heads * self.dim
         self.v_size = 0 if self.values_are_keys else self.num_kv_heads * self.vdim
         self.channels = self.q_size + self.k_size + self.v_size
+        self.gate_size = self.num_heads * self.vdim if gate == "channel" else 0
+        self.row_bias: Optional[torch.Tensor] = None  # the bias of every column of the first product (zeros for the gate's)
         self.qkv_weight: Optional[torch.Tensor] = None
         self.qkv_bias_vec: Optional[torch.Tensor] = None
         self.conv_weight: Optional[torch.Tensor] = None
@@ -88,7 +100,8 @@ class ConvAttentionMixer(Mixer):
         sources, sizes = (n["q"], n["k"], n["v"]), (self.q_size, self.k_size, self.v_size)
         if self.values_are_keys:
             sources, sizes = sources[:2], sizes[:2]
-        out = {"qkv_weight": fused_rows(sources, tuple((s, h) for s in sizes))}
+        rows = tuple(zip(sources, sizes)) + (((n["g"], self.gate_size),) if self.gate_size else ())
+        out = {"qkv_weight": fused_rows(tuple(r[0] for r in rows), tuple((r[1], h) for r in rows))}
         if self.qkv_bias:
             out["qkv_bias_vec"] = fused_rows(tuple(s + ".b" for s in sources), tuple((s,) for s in sizes), role="vector")
         if self.conv_taps:
@@ -110,7 +123,10 @@ class ConvAttentionMixer(Mixer):
         self.refresh_derived()
 
     def refresh_derived(self) -> None:
-        """The output weight at the kernels' head size; to be called again after a tensor was bound anew."""
+        """The bias of the first product's rows and the output weight at the kernels' head size; to be called again after a
+        tensor was bound anew."""
+        if self.qkv_bias and self.qkv_bias_vec is not None:
+            self.row_bias = torch.nn.functional.pad(self.qkv_bias_vec, (0, self.gate_size)) if self.gate_size else self.qkv_bias_vec
         self.o_padded = None
         if self.o_weight is not None and self.cached_dim != self.vdim:
             wide = torch.zeros((self.hidden_size, self.num_heads, self.cached_dim), dtype=self.o_weight.dtype, device=self.o_weight.device)
@@ -121,7 +137,7 @@ class ConvAttentionMixer(Mixer):
     def prepare_kernels(self, ops) -> None:
         load = getattr(ops, "attention_library", None)
         if load is not None and self.cached_dim <= getattr(ops, "MAX_TILED_HEAD_DIM", self.cached_dim):
-            load(self.cached_dim)
+            load(self.cached_dim, capped=self.softcap is not None, gated=self.gate is not None)
         self.prepare_weight(ops, "qkv_weight")
         self.prepare_weight(ops, "o_padded" if self.o_padded is not None else "o_weight")
 
@@ -146,7 +162,8 @@ class ConvAttentionMixer(Mixer):
         else:
             pages, state = cache, None
         meta = pages.batch
-        qkv = ops.linear(x, self.operand("qkv_weight"), self.qkv_bias_vec if self.qkv_bias else None, ctx.dtype)
+        qkv = ops.linear(x, self.operand("qkv_weight"), self.row_bias if self.qkv_bias else None, ctx.dtype)
+        projected = qkv
         if self.conv_taps >= 1:
             qkv = ops.short_conv(qkv, self.channels, self.conv_weight, state.tensors["conv_tail"] if state is not None else None,
                                  ctx.slots, ctx.cu_q, ctx.max_q_len, activation="none", update_state=owns_cache)
@@ -166,8 +183,11 @@ class ConvAttentionMixer(Mixer):
             ctx.all_decode, ctx.workspace,
             decode_prefix=getattr(ctx, "decode_prefix", 0), portions_max_kv_len=getattr(meta, "max_kv_len_of_portions", 0) or None,
             **({"sinks": self.sinks} if self.sinks is not None else {}),
+            **({"softcap": self.softcap} if self.softcap is not None else {}),
+            **({"gate": (projected, self.channels, self.vdim)} if self.gate is not None else {}),
         )
-        return ops.linear(attn, self.operand("o_padded" if self.o_padded is not None else "o_weight"), self.o_bias_vec if self.out_bias else None, ctx.dtype)
+        return ops.linear(attn, self.operand("o_padded" if self.o_padded is not None else "o_weight"), self.o_bias_vec if self.out_bias else None, ctx.dtype,
+                          partials_ok=self.gate is not None and not self.out_bias)
 
 
 register_part("mixer", "conv_attention", ConvAttentionMixer)

@@ -32,8 +32,8 @@ class GatedMLP(FeedForward):
         """``names``: the gate, up and down tensors below the prefix."""
         super().__init__(prefix)
         self.names = tuple(names)
-        if activation not in ("silu", "gelu_tanh"):
-            raise ValueError(f"activation {activation!r} is not implemented ('silu' or 'gelu_tanh')")
+        if activation not in ("silu", "gelu_tanh", "relu"):
+            raise ValueError(f"activation {activation!r} is not implemented ('silu', 'gelu_tanh' or 'relu')")
         self.activation = activation
         self.hidden_size = int(hidden_size)
         self.intermediate_size = int(intermediate_size)
@@ -59,7 +59,7 @@ class GatedMLP(FeedForward):
         if self.activation == "silu":
             act = ops.linear_silu_mul(x, self.operand("gate_up_weight"), ctx.dtype)
         else:
-            # gelu_tanh(z) = z / 2 * (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))), in float32 with one rounding at the store
+            # gelu_tanh(z) = z / 2 * (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))), relu(z) = max(z, 0), in float32 with one rounding at the store
             fused = getattr(ops, "linear_gated_act", None)  # (one kernel for decode-sized batches where the operations have it)
             if fused is not None:
                 act = fused(x, self.operand("gate_up_weight"), ctx.dtype, self.activation)

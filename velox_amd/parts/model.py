@@ -5,7 +5,8 @@
 norm kinds with their constants), shared position encodings, and ``schedule``, the
 order in which layers run.  The schedule is a list of ``ScheduleEntry``: an entry may
 name a layer that an earlier entry already named (the layer's weights run twice, each
-run with a cache of its own), or set ``cache_from`` to an earlier entry to read that
+run with a cache of its own), begin a pass of a loop over layers (``begins_pass``: the
+model's ``pass_input`` then makes that pass's residual first), or set ``cache_from`` to an earlier entry to read that
 entry's cache instead of owning one.
 
 ``DecoderModel`` runs the whole thing the way the reference's ``QwenDecoderModel``
@@ -20,7 +21,7 @@ from typing import Dict, List, Optional, Tuple
 import torch
 
 from . import block as _block  # noqa: F401  (registers the built-in arrangement)
-from .base import Embedding, OutputHead, Param, Part, PartSpec, StateNeed, make_part, register_part, single
+from .base import Embedding, OutputHead, Param, Part, PartSpec, PassInput, StateNeed, make_part, register_part, single
 
 
 @dataclass(frozen=True)
@@ -44,6 +45,7 @@ class LayerSpec:
 class ScheduleEntry:
     layer: int
     cache_from: Optional[int] = None
+    begins_pass: bool = False
 
 
 @dataclass
@@ -70,6 +72,9 @@ class ModelSpec:
     # Copies of the residual that the blocks keep side by side (hyper-connections): the residual is then float32
     # ``[T, residual_streams * H]``, every copy starts as the embedding output, and the final norm reads their sum.
     residual_streams: int = 1
+    # What makes the residual of every schedule entry that begins a pass (a kind registered under "pass_input"; it gets
+    # its ``args`` plus ``hidden_size``).
+    pass_input: Optional[PartSpec] = None
 
     def validate(self) -> None:
         if not self.layers:
@@ -82,6 +87,8 @@ class ModelSpec:
                     raise ValueError(f"schedule[{index}].cache_from must name an earlier entry")
                 if self.schedule[entry.cache_from].cache_from is not None:
                     raise ValueError(f"schedule[{index}].cache_from must name an entry that owns its cache")
+            if entry.begins_pass and (self.pass_input is None or self.residual_streams != 1):
+                raise ValueError(f"schedule[{index}] begins a pass: the model needs a pass_input, and one residual stream")
 
 
 class TableEmbedding(Embedding):
@@ -141,14 +148,40 @@ class BigramEmbedding(TableEmbedding):
                                     ctx.positions, ctx.cu_q, ctx.slots, cache.tensors["previous_token"], ctx.max_q_len)
 
 
+class LinearPassInput(PassInput):
+    """``x <- W [x; start]``: the residual and the embedding output side by side through one product without bias, whose
+    float32 result is the pass's residual.  The kernel that adds what is pending writes both halves of the product's
+    input and clears the residual, so the product is what the next norm adds, like any sub-layer's output."""
+
+    def __init__(self, hidden_size: int, name: str = "pass.in") -> None:
+        super().__init__("")
+        self.hidden_size = int(hidden_size)
+        self.name = name
+        self.weight: Optional[torch.Tensor] = None
+
+    def params(self) -> Dict[str, Param]:
+        return {"weight": single(self.name, (self.hidden_size, 2 * self.hidden_size))}
+
+    def prepare_kernels(self, ops) -> None:
+        self.prepare_weight(ops, "weight")
+
+    def forward(self, residual, pending, start, ctx):
+        joined = ctx.ops.join_rows(residual, pending, start, ctx.dtype)
+        return ctx.ops.linear(joined, self.operand("weight"), None, torch.float32, partials_ok=True)
+
+
 class LinearHead(OutputHead):
     """``logits = (hidden @ W^T) * scale`` without bias; ``W`` is the embedding table when tied
-    (reference ``src/transformer.py:60-62``; it has no scale, which is ``scale`` = 1).  Logits are returned in float32
-    and the scale is applied to them there."""
+    (reference ``src/transformer.py:60-62``; it has no scale, which is ``scale`` = 1), then ``cap * tanh(logits / cap)`` with
+    ``softcap``.  Logits are returned in float32 and both are applied to them there."""
 
-    def __init__(self, name: str, vocab_size: int, hidden_size: int, tied_to: Optional[str] = None, scale: float = 1.0) -> None:
+    def __init__(self, name: str, vocab_size: int, hidden_size: int, tied_to: Optional[str] = None, scale: float = 1.0,
+                 softcap: Optional[float] = None) -> None:
         super().__init__("")
+        if softcap is not None and not float(softcap) > 0:
+            raise ValueError(f"softcap={softcap} must be positive")
         self.scale = float(scale)
+        self.softcap = float(softcap) if softcap is not None else None
         self.name = name
         self.vocab_size = vocab_size
         self.hidden_size = hidden_size
@@ -166,12 +199,17 @@ class LinearHead(OutputHead):
 
     def forward(self, hidden_rows: torch.Tensor, ctx) -> torch.Tensor:
         logits = ctx.ops.linear(hidden_rows, self.operand("weight"), None, torch.float32)
+        if self.softcap is not None:
+            return ctx.ops.softcap_(logits, self.softcap, self.scale)
         return logits if self.scale == 1.0 else ctx.ops.scale_(logits, self.scale)
 
 
 register_part("embedding", "table", TableEmbedding)
 register_part("embedding", "bigram_table", BigramEmbedding)
 register_part("head", "linear", LinearHead)
+register_part("pass_input", "linear", LinearPassInput)
+
+EMBEDDING_OUTPUT = "embedding_output"  # key in a step's shared values: the embedding output, for models whose passes read it
 
 
 class DecoderModel(Part):
@@ -197,11 +235,13 @@ class DecoderModel(Part):
         head = spec.head or PartSpec.of("linear")
         self.head = make_part("head", head.kind, name=spec.head_name, vocab_size=spec.vocab_size, hidden_size=spec.hidden_size,
                               tied_to=spec.embed_name if spec.tie_head else None, **head.kwargs())
+        self.pass_input = make_part("pass_input", spec.pass_input.kind, hidden_size=spec.hidden_size, **spec.pass_input.kwargs()) if spec.pass_input is not None else None
         self.schedule = list(spec.schedule)
 
     # -- structure ----------------------------------------------------------------------
     def children(self) -> Tuple[Part, ...]:
-        return (self.embedding, *self.positions.values(), *self.blocks, self.final_norm, self.head)
+        joint = (self.pass_input,) if self.pass_input is not None else ()
+        return (self.embedding, *self.positions.values(), *joint, *self.blocks, self.final_norm, self.head)
 
     def all_parts(self) -> List[Part]:
         out: List[Part] = []
@@ -256,13 +296,17 @@ class DecoderModel(Part):
             cache = ctx.cache_view(owner)
             # the norm that reads this block's output: the one the next entry's block begins with, if it begins with one
             # (the final norm works on chosen rows and takes its input as it is)
-            following = self.blocks[self.schedule[index + 1].layer].input_norm() if index + 1 < len(self.schedule) else None
+            following = self.blocks[self.schedule[index + 1].layer].input_norm() if index + 1 < len(self.schedule) and not self.schedule[index + 1].begins_pass else None
+            if entry.begins_pass:
+                pending = self.pass_input.forward(residual, pending, ctx.shared[EMBEDDING_OUTPUT], ctx)
             pending = self.blocks[entry.layer].forward(residual, pending, ctx, cache, entry.cache_from is None, next_norm=following)
         return pending
 
     def forward(self, token_ids: torch.Tensor, ctx):
         """Runs every block; returns ``(residual float32 [T, H], pending [T, H])``."""
         residual = self.embed(token_ids, ctx)
+        if self.pass_input is not None:
+            ctx.shared[EMBEDDING_OUTPUT] = ctx.ops.kept_copy(residual, ctx.dtype)  # (blocks update the residual in place)
         return residual, self.run_schedule(residual, None, ctx)
 
     def logits(self, residual: torch.Tensor, pending, rows: torch.Tensor, ctx) -> torch.Tensor:

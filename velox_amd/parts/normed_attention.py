@@ -6,6 +6,12 @@ Beside ``parts.attention`` (rotated queries and keys of one size for keys and va
   (``qk_norm="whole"``: one weight of ``heads * dim`` and one of ``kv_heads * dim`` entries) or per head
   (``"per_head"``: one weight of ``dim`` entries for all query heads, one for all key heads);
 * its own sizes for query/key heads (``dim``) and value heads (``vdim``);
+* optionally biases on the q, k and v projections and on the output projection, added in the projection;
+* optionally a sliding window (``window``: a query at ``i`` sees ``j`` with ``0 <= i - j < window``; pages behind it are given back)
+  that keeps the first tokens of the sequence (``keep_first``: those are seen from everywhere, at their true distance, and
+  their pages stay);
+* optionally an output gate per head (``gate="head"``): head ``h``'s output times ``sigmoid(W_g x)_h``, the gate's rows in the same
+  product as q, k and v, applied where the attention kernels finish a row;
 * optionally a query temperature, ``q <- q * (1 + coef * ln(floor((p + 1) / every) + 1))`` at position ``p``;
 * optionally a learned bias by distance, added to the scaled score: ``rel[bucket(i - j), head]`` with ``B`` buckets of
   which the first ``B // 2`` hold one distance each and the others grow logarithmically up to distance ``far``:
@@ -76,12 +82,22 @@ class NormedAttentionMixer(Mixer):
         value_mix_key: str = "first_values",
         has_mix_weight: Optional[bool] = None,
         names: Tuple[Tuple[str, str], ...] = (),
+        qkv_bias: bool = False,
+        out_bias: bool = False,
+        window: Optional[int] = None,
+        keep_first: int = 0,
+        gate: Optional[str] = None,
     ) -> None:
         """``q_temp = (coef, every)``; ``distance_bias = (buckets, far)``; ``value_mix``: None, ``"first"`` (publishes its
         values) or ``"blend"`` (blends with the published ones); ``has_mix_weight``: whether the checkpoint holds the
         blending weight for this layer (default: whenever ``value_mix`` is set; the publishing layer's is not used);
-        ``names``: pairs (tensor, name below the prefix) that replace the default names."""
+        ``names``: pairs (tensor, name below the prefix) that replace the default names; a bias is the tensor's name with ``.b``
+        added."""
         super().__init__(prefix)
+        if window is not None and window < 1 or keep_first < 0:
+            raise ValueError(f"window={window} must be at least 1 and keep_first={keep_first} not negative")
+        if gate not in (None, "head"):
+            raise ValueError(f"gate must be None or 'head', got {gate!r}")
         if num_heads % num_kv_heads != 0:
             raise ValueError(f"num_heads={num_heads} must be a multiple of num_kv_heads={num_kv_heads}")
         if qk_norm not in ("whole", "per_head"):
@@ -108,13 +124,21 @@ class NormedAttentionMixer(Mixer):
         self.value_mix = value_mix
         self.value_mix_key = value_mix_key
         self.has_mix_weight = (value_mix is not None) if has_mix_weight is None else bool(has_mix_weight)
-        self.names = {"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "o": "o_proj.weight", "q_norm": "q_norm.weight",
+        self.qkv_bias, self.out_bias = bool(qkv_bias), bool(out_bias)
+        self.window = int(window) if window is not None else None
+        self.keep_first = int(keep_first) if window is not None else 0
+        self.gate = gate
+        self.names = {"gate": "gate_proj.weight", "q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "o": "o_proj.weight", "q_norm": "q_norm.weight",
                       "k_norm": "k_norm.weight", "rel": "distance_bias", "mix": "value_mix"}
         self.names.update(dict(names))
         self.q_size = self.num_heads * self.dim
         self.k_size = self.num_kv_heads * self.dim
         self.v_size = self.num_kv_heads * self.vdim
+        self.gate_size = self.num_heads if gate == "head" else 0
         self.qkv_weight: Optional[torch.Tensor] = None
+        self.qkv_bias_vec: Optional[torch.Tensor] = None
+        self.row_bias: Optional[torch.Tensor] = None  # the bias of every column of the first product (zeros for the gate's)
+        self.o_bias_vec: Optional[torch.Tensor] = None
         self.o_weight: Optional[torch.Tensor] = None
         self.q_norm_weight: Optional[torch.Tensor] = None
         self.k_norm_weight: Optional[torch.Tensor] = None
@@ -126,8 +150,10 @@ class NormedAttentionMixer(Mixer):
     def params(self) -> Dict[str, Param]:
         h, names = self.hidden_size, self.names
         whole = self.qk_norm == "whole"
+        sources, sizes = (names["q"], names["k"], names["v"]), (self.q_size, self.k_size, self.v_size)
+        rows = tuple(zip(sources, sizes)) + (((names["gate"], self.gate_size),) if self.gate_size else ())
         out = {
-            "qkv_weight": fused_rows((names["q"], names["k"], names["v"]), ((self.q_size, h), (self.k_size, h), (self.v_size, h))),
+            "qkv_weight": fused_rows(tuple(r[0] for r in rows), tuple((r[1], h) for r in rows)),
             "q_norm_weight": single(names["q_norm"], (self.q_size if whole else self.dim,), role="vector", init="one_plus_normal"),
             "k_norm_weight": single(names["k_norm"], (self.k_size if whole else self.dim,), role="vector", init="one_plus_normal"),
         }
@@ -135,18 +161,24 @@ class NormedAttentionMixer(Mixer):
             out["rel"] = single(names["rel"], (self.distance_bias[0], self.num_heads), role="vector")
         if self.has_mix_weight:
             out["mix_weight"] = single(names["mix"], (), role="vector")
+        if self.qkv_bias:
+            out["qkv_bias_vec"] = fused_rows(tuple(s + ".b" for s in sources), tuple((n,) for n in sizes), role="vector")
         out["o_weight"] = single(names["o"], (h, self.num_heads * self.vdim))
+        if self.out_bias:
+            out["o_bias_vec"] = single(names["o"] + ".b", (h,), role="vector")
         return out
 
     def cache_need(self):
-        return kv_pages(self.num_kv_heads, self.cached_dim)
+        return kv_pages(self.num_kv_heads, self.cached_dim, self.window, self.keep_first)
 
     def finalize(self, device, dtype) -> None:
         self.refresh_derived()
 
     def refresh_derived(self) -> None:
-        """What is derived from the bound tensors: the bias by distance and the output weight at the kernels' head size.
-        To be called again after a tensor was bound anew."""
+        """What is derived from the bound tensors: the bias by distance, the bias of the first product's rows and the output
+        weight at the kernels' head size.  To be called again after a tensor was bound anew."""
+        if self.qkv_bias and self.qkv_bias_vec is not None:
+            self.row_bias = torch.nn.functional.pad(self.qkv_bias_vec, (0, self.gate_size)) if self.gate_size else self.qkv_bias_vec
         if self.distance_bias is not None and self.rel is not None:
             self.bias_table = bias_by_distance(self.rel, self.distance_bias[1])
         self.o_padded = None
@@ -159,7 +191,7 @@ class NormedAttentionMixer(Mixer):
     def prepare_kernels(self, ops) -> None:
         load = getattr(ops, "attention_library", None)
         if load is not None and self.cached_dim <= getattr(ops, "MAX_TILED_HEAD_DIM", self.cached_dim):
-            load(self.cached_dim, self.distance_bias is not None)
+            load(self.cached_dim, self.distance_bias is not None, kept=self.keep_first > 0, gated=self.gate is not None)
         self.prepare_weight(ops, "qkv_weight")
         self.prepare_weight(ops, "o_padded" if self.o_padded is not None else "o_weight")
 
@@ -180,7 +212,7 @@ class NormedAttentionMixer(Mixer):
     def forward(self, x, ctx, cache, owns_cache: bool = True):
         ops = ctx.ops
         meta = cache.batch
-        qkv = ops.linear(x, self.operand("qkv_weight"), None, ctx.dtype)
+        qkv = ops.linear(x, self.operand("qkv_weight"), self.row_bias if self.qkv_bias else None, ctx.dtype)
         first = None
         if self.value_mix == "blend":
             first = ctx.shared.get(self.value_mix_key)
@@ -199,12 +231,15 @@ class NormedAttentionMixer(Mixer):
             q, self.num_heads, self.num_kv_heads, self.cached_dim,
             cache.tensors["k"], cache.tensors["v"], cache.block_size,
             meta.block_tables, ctx.cu_q, meta.kv_lens,
-            ctx.max_q_len, meta.max_kv_len, self.scale, None,
+            ctx.max_q_len, meta.max_kv_len, self.scale, self.window,
             ctx.all_decode, ctx.workspace,
             decode_prefix=getattr(ctx, "decode_prefix", 0), portions_max_kv_len=getattr(meta, "max_kv_len_of_portions", 0) or None,
             distance_bias=self.bias_table,
+            **({"keep_first": self.keep_first} if self.keep_first > 0 else {}),
+            **({"gate": (qkv, self.q_size + self.k_size + self.v_size, 0)} if self.gate is not None else {}),
         )
-        return ops.linear(attn, self.operand("o_padded" if self.o_padded is not None else "o_weight"), None, ctx.dtype)
+        return ops.linear(attn, self.operand("o_padded" if self.o_padded is not None else "o_weight"), self.o_bias_vec if self.out_bias else None, ctx.dtype,
+                          partials_ok=self.gate is not None and not self.out_bias)
 
 
 register_part("mixer", "normed_attention", NormedAttentionMixer)

@@ -13,7 +13,7 @@ from typing import Dict, Optional
 
 import torch
 
-from .base import DeferredNorm, Norm, NormedDelta, Param, ReadyInput, ResidualCopy, ScaledSum, StreamUpdate, register_part, single
+from .base import DeferredNorm, Norm, NormedDelta, NormedSum, Param, ReadyInput, ResidualCopy, ScaledSum, StreamUpdate, register_part, single
 
 
 class RMSNorm(Norm):
@@ -48,6 +48,8 @@ class RMSNorm(Norm):
             if form is None:
                 raise ValueError(f"{type(delta.norm).__name__} cannot norm a sub-layer's output inside the next norm's kernel")
             return ctx.ops.norm_add_norm(residual, delta.y, form[0], form[1], self.weight, self.eps, ctx.dtype, rows=rows)
+        if isinstance(delta, NormedSum):
+            return ctx.ops.normed_sum_norm(residual, delta, self.weight, self.eps, ctx.dtype, rows=rows)
         if isinstance(delta, ResidualCopy):
             delta = None  # (the block before has added everything itself)
         if rows is None:

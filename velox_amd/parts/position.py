@@ -16,6 +16,11 @@ Two options beyond the reference's: ``layout`` says which channels are a pair (`
 ``r_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1)`` the frequency becomes
 ``f_i / factor * r_i + f_i (1 - r_i)``, and cos and sin are both multiplied by
 ``0.1 ln(factor) + 1``, which the tables hold already.
+
+``bands = (factor, low, high, original)`` stretches by wavelength instead (as Llama 3.1 does), and only with
+``exact_angles``: a frequency that turns more than ``high`` times within ``original`` tokens stays, one that turns less than
+``low`` times is divided by ``factor``, and between the two, with ``s = (turns - low) / (high - low)``, it becomes
+``(1 - s) f / factor + s f``.  cos and sin are not multiplied.
 """
 from __future__ import annotations
 
@@ -29,7 +34,7 @@ from .base import PositionEncoding, register_part
 
 class RotaryEncoding(PositionEncoding):
     def __init__(self, rotary_dim: int, theta: float, max_position: int, scaling_factor: float = 1.0, layout: str = "halves",
-                 stretch: Optional[Sequence[float]] = None, exact_angles: bool = False) -> None:
+                 stretch: Optional[Sequence[float]] = None, exact_angles: bool = False, bands: Optional[Sequence[float]] = None) -> None:
         """``exact_angles``: frequencies ``theta^(-2i/d) / scaling_factor`` and the angles ``p * f_i`` are worked out in
         float64 and only cosine and sine are rounded to float32 (the tables then do not carry the float32 error of the
         angle, which grows with the position)."""
@@ -41,6 +46,9 @@ class RotaryEncoding(PositionEncoding):
             raise ValueError(f"layout must be 'halves' or 'interleaved', got {layout!r}")
         if stretch is not None and (len(stretch) != 4 or not stretch[0] > 0 or not stretch[1] > 0 or not stretch[2] > 0 or not stretch[3] > 0):
             raise ValueError(f"stretch must be four positive numbers (factor, original, fast, slow), got {stretch!r}")
+        if bands is not None and (len(bands) != 4 or not min(bands) > 0 or not bands[2] > bands[1] or not exact_angles or stretch is not None):
+            raise ValueError(f"bands must be four positive numbers (factor, low, high > low, original), with exact angles and no stretch; got {bands!r}")
+        self.bands = tuple(float(v) for v in bands) if bands is not None else None
         self.layout = layout
         self.stretch = tuple(float(v) for v in stretch) if stretch is not None else None
         self.rotary_dim = int(rotary_dim)
@@ -72,6 +80,11 @@ class RotaryEncoding(PositionEncoding):
         if self.exact_angles and self.stretch is None:
             index = torch.arange(self.rotary_dim // 2, dtype=torch.float64)
             freq = self.theta ** (-2.0 * index / self.rotary_dim) / self.scaling_factor
+            if self.bands is not None:
+                factor, low, high, original = self.bands
+                turns = original * freq / (2.0 * math.pi)
+                share = ((turns - low) / (high - low)).clamp(0.0, 1.0)  # (0 below ``low`` turns, 1 above ``high``)
+                freq = (1.0 - share) * freq / factor + share * freq
             angles = torch.outer(torch.arange(self.max_position, dtype=torch.float64), freq)
             self.cos = angles.cos().float().contiguous().to(device)
             self.sin = angles.sin().float().contiguous().to(device)
