@@ -16,6 +16,9 @@ over the steps in which all of them decode, ``..._frac``: that step's share of t
 ``e2e_b<B>_p512_g256``: generated tokens / wall time with the prompts' time included, which is how
 the reference's ``benchmark.py:204`` counts).
 
+``--design kukulorn`` measures the Kukulorn design (norm, then mixer and feed-forward side by side; attention over a window that keeps its
+first tokens beside a state space, attention with capped scores and gates; layers that run several times) at layer sizes of real models, beside
+Gosulorn, Kedanex and the dense decoder.
 ``--design kedanex`` measures the Kedanex design (a norm on both sides of every sub-layer, the generalized delta rule, a gated recurrence per
 channel, window attention whose values are the keys, PolyNorm, experts) beside Gosulorn with one stream (the closest recurrent mixers) and
 Tiverax with the same experts.
@@ -356,6 +359,26 @@ def kedanex_config(size: dict) -> dict:
     return {"architecture": "Kedanex", "vocab": DESIGN_VOCAB, "width": size["width"], "norm": {"eps": 1e-6}, "layers": layers}
 
 
+# Layer sizes for --design kukulorn: eight layer runs, two layers of two mixers side by side (attention over a window that keeps its first
+# tokens beside a state space) that run twice, an attention layer over all keys, one more of each.  Beside it: Gosulorn at the same
+# width with one stream (attention beside a delta rule, the same feed-forward), Kedanex, and the dense decoder.
+KUKULORN_SIZES = {
+    "2k": dict(width=2048, heads=16, kv_heads=4, dim=128, window=1024, keep_first=64, buckets=32, far=1024, space_heads=32, state=128, space_vdim=64, groups=1, ff=5632),
+    "4k": dict(width=4096, heads=32, kv_heads=8, dim=128, window=2048, keep_first=64, buckets=32, far=2048, space_heads=64, state=128, space_vdim=64, groups=8, ff=11008),
+}
+
+
+def kukulorn_config(size: dict) -> dict:
+    heads = {"heads": size["heads"], "kv_heads": size["kv_heads"], "dim": size["dim"], "vdim": size["dim"], "scale": size["dim"] ** -0.5}
+    full = dict(heads, conv=4, softcap=30.0, rot={"dims": size["dim"], "base": 5e5, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}})
+    left = dict(heads, buckets=size["buckets"], bias_max=size["far"], mask={"size": size["window"], "keep_first": size["keep_first"]})
+    right = {"heads": size["space_heads"], "groups": size["groups"], "state": size["state"], "vdim": size["space_vdim"], "conv": 4, "norm_groups": size["groups"]}
+    mlp = {"kind": "dense", "ff": size["ff"]}
+    pair, attention = {"type": "parallel", "mixer": {"left": left, "right": right}, "mlp": mlp}, {"type": "attention", "mixer": full, "mlp": mlp}
+    return {"architecture": "Kukulorn", "vocab": DESIGN_VOCAB, "width": size["width"], "norm": {"eps": 1e-5}, "logit_softcap": 30.0,
+            "layers": [pair, pair, attention, pair, attention], "loop": {"start": 0, "stop": 3, "times": 2}}
+
+
 def tiverax_all_routed(size: dict) -> dict:
     """Tiverax at the width of ``size`` with the same experts per layer and per token (no shared expert, no dense layers)."""
     config = tiverax_config(dict(TIVERAX_SIZES["2k" if size["width"] == 2048 else "4k"], experts=size["experts"], top=size["top"], expert_ff=size["expert_ff"]))
@@ -375,6 +398,10 @@ def designs_at(design: str, name: str):
     if design == "kedanex":
         size = KEDANEX_SIZES[name]
         return (("kedanex", kedanex_config(size)), ("gosulorn", gosulorn_config(dict(GOSULORN_SIZES[name], streams=1))), ("tiverax", tiverax_all_routed(size)))
+    if design == "kukulorn":
+        size = KUKULORN_SIZES[name]
+        return (("kukulorn", kukulorn_config(size)), ("gosulorn", gosulorn_config(dict(GOSULORN_SIZES[name], streams=1))), ("kedanex", kedanex_config(KEDANEX_SIZES[name])),
+                ("qwen2", qwen2_like(dict(size, rot_dim=0))))
     if design == "lelutar":
         size = LELUTAR_SIZES[name]
         dense = dict(width=size["width"], heads=size["heads"], kv_heads=size["kv_heads"], dim=size["dim"], rot_dim=0, ff=size["top"] * size["expert_ff"])
@@ -428,7 +455,7 @@ def main() -> int:
     parser.add_argument("--shape", default="7b", choices=sorted(SHAPES), help="layer sizes: the headline is 7b; 1.5b and 32b are the reference's other two")
     parser.add_argument("--far", action="store_true",
                         help="further sizes under `points`: decode at batch 1 and 8 behind 32,256 tokens, a prefill of 8,192 tokens, and a decode step of a true float32 run (batch 8)")
-    parser.add_argument("--design", default=None, choices=["tiverax", "dipisun", "gosulorn", "lelutar", "kedanex"],
+    parser.add_argument("--design", default=None, choices=["tiverax", "dipisun", "gosulorn", "lelutar", "kedanex", "kukulorn"],
                         help="instead of the headline: prefill and decode of this design at real layer sizes beside the framework's closest models of equal size")
     parser.add_argument("--only", default="", help="with --design: which of the models that are measured side by side (names with commas between them; default: all)")
     parser.add_argument("--sizes", default="2k,4k", help="with --design: which of the sizes (2k, 4k = the models' widths)")
@@ -442,7 +469,7 @@ def main() -> int:
         points = design_points(args)
         first = args.sizes.split(",")[0]
         head = points.get(f"{args.design}_{first}") or next(iter(points.values()))
-        sizes = {"tiverax": TIVERAX_SIZES, "dipisun": DIPISUN_SIZES, "gosulorn": GOSULORN_SIZES, "lelutar": LELUTAR_SIZES, "kedanex": KEDANEX_SIZES}[args.design]
+        sizes = {"tiverax": TIVERAX_SIZES, "dipisun": DIPISUN_SIZES, "gosulorn": GOSULORN_SIZES, "lelutar": LELUTAR_SIZES, "kedanex": KEDANEX_SIZES, "kukulorn": KUKULORN_SIZES}[args.design]
         print(json.dumps({
             "metric": "decode_tokens_per_second", "value": head["decode_tok_s"], "unit": "tok/s", "n_gpus": 1, "steps": args.steps,
             "warmup": args.warmup, "ms_per_step": head["decode_ms"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None,

@@ -286,6 +286,13 @@ class DecoderModel(Part):
             residual = self.positions[self.spec.embedding_position].on_embeddings(residual, ctx)
         return residual.repeat(1, streams) if streams > 1 else residual
 
+    def begin(self, token_ids: torch.Tensor, ctx) -> torch.Tensor:
+        """``embed``, with the embedding output kept for the passes that read it."""
+        residual = self.embed(token_ids, ctx)
+        if self.pass_input is not None:
+            ctx.shared[EMBEDDING_OUTPUT] = ctx.ops.kept_copy(residual, ctx.dtype)  # (blocks update the residual in place)
+        return residual
+
     def run_schedule(self, residual: torch.Tensor, pending, ctx, first: int = 0, last: Optional[int] = None):
         """Runs schedule entries ``first .. last - 1`` on ``residual`` (updated in place); takes and returns ``pending``,
         the sub-layer output that the next norm still has to add."""
@@ -304,9 +311,7 @@ class DecoderModel(Part):
 
     def forward(self, token_ids: torch.Tensor, ctx):
         """Runs every block; returns ``(residual float32 [T, H], pending [T, H])``."""
-        residual = self.embed(token_ids, ctx)
-        if self.pass_input is not None:
-            ctx.shared[EMBEDDING_OUTPUT] = ctx.ops.kept_copy(residual, ctx.dtype)  # (blocks update the residual in place)
+        residual = self.begin(token_ids, ctx)
         return residual, self.run_schedule(residual, None, ctx)
 
     def logits(self, residual: torch.Tensor, pending, rows: torch.Tensor, ctx) -> torch.Tensor:
