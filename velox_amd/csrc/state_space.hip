@@ -129,9 +129,11 @@ __global__ void __launch_bounds__(256) state_space_step_kernel(const StateSpaceA
 #define SS_CHUNK 64
 #define SS_ROWS 128  // entries of B (rows of the state) a workgroup works on at a time
 #define SS_COLS 64   // columns of the state a workgroup works on
+#define SS_HALF 32   // tokens of a chunk that state_space_local_kernel holds in LDS at a time
 #define SS_LOCAL_B (SS_ROWS + 16)  // LDS row strides: 16 (mod 64) for reads of four rows x 16 neighbours,
 #define SS_LOCAL_X (SS_COLS + 16)
-#define SS_OUT_B (SS_ROWS + 4)     // 4 (mod 64) for 16 rows x 16 bytes, and for every fourth row x 16 neighbours
+#define SS_SLICE 32  // entries of B and C the read-out takes at a time
+#define SS_OUT_B (SS_SLICE + 4)    // 4 (mod 32) for 16 rows x 16 bytes, and for every fourth row x 16 neighbours
 #define SS_OUT_X (SS_COLS + 4)
 
 __device__ __forceinline__ float4_t mma4(float a, float b, float4_t c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
@@ -153,23 +155,53 @@ __device__ __forceinline__ void chunk_steps(const StateSpaceArgs& a, int t0, int
   }
 }
 
-// `count` rows of 64 from row t0: columns at .. at + width - 1 of xbc into LDS rows of `stride` floats, zeros up to `padded` columns and
-// for the rows beyond
-template <typename T>
-__device__ __forceinline__ void stage_rows(const T* rows, int ld, int t0, int count, int at, int width, int padded, float* to, int stride, bool vec) {
-  const int quads = padded / 4;
-  for (int e = threadIdx.x; e < SS_CHUNK * quads; e += 256) {
-    const int r = e / quads, c = (e - r * quads) * 4;
-    float v[4];
-    load4<T>(rows, (size_t)(t0 + r) * ld + at, c, width, r < count, vec, v);
-    *reinterpret_cast<float4_t*>(to + r * stride + c) = float4_t{v[0], v[1], v[2], v[3]};
+// ROWS rows of COLS columns from `from` on (`ld` elements apart) into LDS rows of `stride` floats: the first `count` rows and `width`
+// columns are there, the others become zeros.  In two halves, so that a lane's loads are all under way before one is waited for
+// (load) and something else can stand between them and the stores (store).
+template <typename T, int ROWS, int COLS>
+struct StagedRows {
+  static constexpr int QUADS = COLS / 4, EACH = ROWS * QUADS / 256;
+  static_assert(ROWS * QUADS % 256 == 0, "every lane carries the same number of pieces");
+  float v[EACH][4];
+  __device__ __forceinline__ void load(const T* from, int ld, int count, int width, bool vec) {
+    if (vec) {  // (widths are multiples of four, and so is every row's start)
+#pragma unroll
+      for (int e = 0; e < EACH; ++e) {
+        const int index = threadIdx.x + e * 256, r = index / QUADS, c = index % QUADS * 4;
+        // (a piece that is not there is read from the first row and then cleared: no branch around the load)
+        const bool there = r < count && c < width;
+        const T* p = there ? from + (size_t)r * ld + c : from;
+        if constexpr (sizeof(T) == 4) {
+          const float4_t x = *reinterpret_cast<const float4_t*>(p);
+#pragma unroll
+          for (int j = 0; j < 4; ++j) v[e][j] = there ? x[j] : 0.f;
+        } else {
+          const short4_t x = *reinterpret_cast<const short4_t*>(p);
+#pragma unroll
+          for (int j = 0; j < 4; ++j) v[e][j] = there ? __uint_as_float(((uint32_t)(uint16_t)x[j]) << 16) : 0.f;
+        }
+      }
+    } else {
+#pragma unroll
+      for (int e = 0; e < EACH; ++e) {
+        const int index = threadIdx.x + e * 256, r = index / QUADS, c = index % QUADS * 4;
+        load4<T>(from, (size_t)r * ld, c, width, r < count, false, v[e]);
+      }
+    }
   }
-}
+  __device__ __forceinline__ void store(float* to, int stride) const {
+#pragma unroll
+    for (int e = 0; e < EACH; ++e) {
+      const int index = threadIdx.x + e * 256, r = index / QUADS, c = index % QUADS * 4;
+      *reinterpret_cast<float4_t*>(to + r * stride + c) = float4_t{v[e][0], v[e][1], v[e][2], v[e][3]};
+    }
+  }
+};
 
 template <typename T>
-__global__ void __launch_bounds__(256) state_space_local_kernel(const StateSpaceArgs a, int row_slices, int col_slices, int vec) {
-  __shared__ __attribute__((aligned(16))) float bs[SS_CHUNK * SS_LOCAL_B];
-  __shared__ __attribute__((aligned(16))) float xs[SS_CHUNK * SS_LOCAL_X];
+__global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(4, 8))) state_space_local_kernel(const StateSpaceArgs a, int row_slices, int col_slices, int vec) {
+  __shared__ __attribute__((aligned(16))) float bs[SS_HALF * SS_LOCAL_B];  // half of the chunk's tokens at a time
+  __shared__ __attribute__((aligned(16))) float xs[SS_HALF * SS_LOCAL_X];
   __shared__ float steps[64];
   __shared__ double sums[64];
   const int h = blockIdx.y, b = blockIdx.z;
@@ -186,48 +218,64 @@ __global__ void __launch_bounds__(256) state_space_local_kernel(const StateSpace
   const int n0 = rs * SS_ROWS, v0 = cs * SS_COLS;
   const int n_width = N - n0 < SS_ROWS ? N - n0 : SS_ROWS, v_width = vdim - v0 < SS_COLS ? vdim - v0 : SS_COLS;
   const int n_tiles = (n_width + 15) / 16, v_tiles = (v_width + 15) / 16;
+  StagedRows<T, SS_HALF, SS_ROWS> b_rows;
+  StagedRows<T, SS_HALF, SS_COLS> x_rows;
+  auto load_half = [&](int half) {
+    const int first = half * SS_HALF, here = count > first ? count - first : 0;
+    const T* from = rows + (size_t)(t0 + (here > 0 ? first : 0)) * a.ld;
+    x_rows.load(from + h * vdim + v0, a.ld, here, v_width, vec);
+    b_rows.load(from + inner + g * N + n0, a.ld, here, n_width, vec);
+  };
+  load_half(0);
   chunk_steps<T>(a, t0, count, h, steps, sums);
-  stage_rows<T>(rows, a.ld, t0, count, inner + g * N + n0, n_width, n_tiles * 16, bs, SS_LOCAL_B, vec);
-  stage_rows<T>(rows, a.ld, t0, count, h * vdim + v0, v_width, v_tiles * 16, xs, SS_LOCAL_X, vec);
   __syncthreads();
   const double end = sums[63];
-  {  // x_s times exp(A_Q - A_s) d_s
-    const int quads = v_tiles * 4;
-    for (int e = threadIdx.x; e < SS_CHUNK * quads; e += 256) {
-      const int r = e / quads, c = (e - r * quads) * 4;
-      float4_t* at = reinterpret_cast<float4_t*>(xs + r * SS_LOCAL_X + c);
-      *at = *at * (expf((float)(end - sums[r])) * steps[r]);
-    }
-  }
-  __syncthreads();
   const size_t slot = (size_t)(lo / SS_CHUNK) + b + chunk;
   if (threadIdx.x == 0 && rs == 0 && cs == 0) a.carry[slot * a.heads + h] = expf((float)end);
+  if (threadIdx.x < 64) steps[threadIdx.x] *= expf((float)(end - sums[threadIdx.x]));  // what x_s is multiplied by
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int gg = lane >> 4, i = lane & 15;
   float* local = a.local + (slot * a.heads + h) * (size_t)N * vdim;
-  // a wave takes pairs of row tiles, all column tiles (four at most)
-  for (int nt = 2 * wave; nt < n_tiles; nt += 8) {
-    const bool second = nt + 1 < n_tiles;
-    float4_t acc[2][4];
+  // a wave takes a pair of row tiles, all column tiles (four at most)
+  const int nt = 2 * wave;
+  const bool first = nt < n_tiles, second = nt + 1 < n_tiles;
+  float4_t acc[2][4];
 #pragma unroll
-    for (int p = 0; p < 2; ++p)
+  for (int p = 0; p < 2; ++p)
 #pragma unroll
-      for (int c = 0; c < 4; ++c) acc[p][c] = float4_t{0.f, 0.f, 0.f, 0.f};
-    const float* b0 = bs + gg * SS_LOCAL_B + nt * 16 + i;
-    const float* b1 = b0 + (second ? 16 : 0);
-    const float* x0 = xs + gg * SS_LOCAL_X + i;
-#pragma unroll 4
-    for (int k = 0; k < SS_CHUNK / 4; ++k) {
-      const float first_row = b0[k * 4 * SS_LOCAL_B], second_row = b1[k * 4 * SS_LOCAL_B];
+    for (int c = 0; c < 4; ++c) acc[p][c] = float4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int c = 0; c < 4; ++c) {
-        if (c < v_tiles) {
-          const float xv = x0[k * 4 * SS_LOCAL_X + 16 * c];
-          acc[0][c] = mma4(first_row, xv, acc[0][c]);
-          acc[1][c] = mma4(second_row, xv, acc[1][c]);
+  for (int half = 0; half < SS_CHUNK / SS_HALF; ++half) {
+    __syncthreads();  // (the factors are in place; later: everyone is done with the half before)
+    b_rows.store(bs, SS_LOCAL_B);
+#pragma unroll
+    for (int e = 0; e < x_rows.EACH; ++e) {
+      const float factor = steps[half * SS_HALF + (threadIdx.x + e * 256) / x_rows.QUADS];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) x_rows.v[e][j] *= factor;
+    }
+    x_rows.store(xs, SS_LOCAL_X);
+    __syncthreads();
+    if (half + 1 < SS_CHUNK / SS_HALF) load_half(half + 1);  // (in flight while this half is worked)
+    if (first) {
+      const float* b0 = bs + gg * SS_LOCAL_B + nt * 16 + i;
+      const float* b1 = b0 + (second ? 16 : 0);
+      const float* x0 = xs + gg * SS_LOCAL_X + i;
+#pragma unroll
+      for (int k = 0; k < SS_HALF / 4; ++k) {
+        const float first_row = b0[k * 4 * SS_LOCAL_B], second_row = b1[k * 4 * SS_LOCAL_B];
+#pragma unroll
+        for (int c = 0; c < 4; ++c) {
+          if (c < v_tiles) {
+            const float xv = x0[k * 4 * SS_LOCAL_X + 16 * c];
+            acc[0][c] = mma4(first_row, xv, acc[0][c]);
+            acc[1][c] = mma4(second_row, xv, acc[1][c]);
+          }
         }
       }
     }
+  }
+  if (first) {
 #pragma unroll
     for (int p = 0; p < 2; ++p) {
       if (p == 1 && !second) break;
@@ -282,9 +330,9 @@ __global__ void __launch_bounds__(256) state_space_chain_kernel(const StateSpace
 }
 
 template <typename T>
-__global__ void __launch_bounds__(256) state_space_output_kernel(const StateSpaceArgs a, int col_slices, int vec) {
-  // B's rows of the chunk [64][128 + 4], later Z's rows [128][64 + 4]
-  __shared__ __attribute__((aligned(16))) float shared_rows[SS_ROWS * SS_OUT_X > SS_CHUNK * SS_OUT_B ? SS_ROWS * SS_OUT_X : SS_CHUNK * SS_OUT_B];
+__global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(4, 4))) state_space_output_kernel(const StateSpaceArgs a, int col_slices, int vec) {
+  __shared__ __attribute__((aligned(16))) float bs[SS_CHUNK * SS_OUT_B];  // a slice of B's columns, of Z's rows
+  __shared__ __attribute__((aligned(16))) float zs[SS_SLICE * SS_OUT_X];
   __shared__ __attribute__((aligned(16))) float xs[SS_CHUNK * SS_OUT_X];
   __shared__ float steps[64];
   __shared__ double sums[64];
@@ -304,53 +352,68 @@ __global__ void __launch_bounds__(256) state_space_output_kernel(const StateSpac
   const int my_row = wave * 16 + i;  // the token of the chunk whose read-out this lane's column is
   const bool row_ok = my_row < count;
   const bool busy = wave * 16 < count;  // (the same for the whole wave)
-  const size_t c_row = (size_t)(t0 + (row_ok ? my_row : 0)) * a.ld + inner + a.groups * N + g * N;
+  const T* chunk_rows = rows + (size_t)t0 * a.ld;
+  const T* c_row = chunk_rows + (size_t)(row_ok ? my_row : 0) * a.ld + inner + a.groups * N + g * N;
   const size_t slot = (size_t)(lo / SS_CHUNK) + b + chunk;
   const float* Z = a.local + (slot * a.heads + h) * (size_t)N * vdim;
   const bool z_vec = vdim % 4 == 0;
   float4_t scores[4], acc[4];  // (B_s . C_t) of the four tiles of s; the read-out's four column tiles
 #pragma unroll
   for (int c = 0; c < 4; ++c) scores[c] = acc[c] = float4_t{0.f, 0.f, 0.f, 0.f};
+  StagedRows<T, SS_CHUNK, SS_COLS> x_rows;
+  StagedRows<T, SS_CHUNK, SS_SLICE> b_rows;
+  StagedRows<float, SS_SLICE, SS_COLS> z_rows;
+  float c_held[SS_SLICE / 16][4];  // this lane's entries of C_t: 16 kb + 4 gg .. + 3 of the slice
+  auto load_slice = [&](int n0) {
+    const int n_width = N - n0 < SS_SLICE ? N - n0 : SS_SLICE;
+    b_rows.load(chunk_rows + inner + g * N + n0, a.ld, count, n_width, vec);
+    z_rows.load(Z + (size_t)n0 * vdim + v0, vdim, n_width, v_width, z_vec);
+#pragma unroll
+    for (int kb = 0; kb < SS_SLICE / 16; ++kb) {
+      if (vec) {
+        const bool there = row_ok && 16 * kb + 4 * gg < n_width;
+        float x[4];
+        load4<T>(there ? c_row + n0 + 16 * kb + 4 * gg : c_row, 0, 0, 4, true, true, x);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) c_held[kb][j] = there ? x[j] : 0.f;
+      } else {
+        load4<T>(c_row + n0, 0, 16 * kb + 4 * gg, n_width, row_ok, false, c_held[kb]);
+      }
+    }
+  };
+  x_rows.load(chunk_rows + h * vdim + v0, a.ld, count, v_width, vec);
+  load_slice(0);
   chunk_steps<T>(a, t0, count, h, steps, sums);
-  stage_rows<T>(rows, a.ld, t0, count, h * vdim + v0, v_width, v_tiles * 16, xs, SS_OUT_X, vec);
-  for (int n0 = 0; n0 < N; n0 += SS_ROWS) {
-    const int n_width = N - n0 < SS_ROWS ? N - n0 : SS_ROWS, n_tiles = (n_width + 15) / 16;
-    __syncthreads();  // everyone is done with the rows before
-    stage_rows<T>(rows, a.ld, t0, count, inner + g * N + n0, n_width, n_tiles * 16, shared_rows, SS_OUT_B, vec);
+  x_rows.store(xs, SS_OUT_X);
+  for (int n0 = 0; n0 < N; n0 += SS_SLICE) {
+    b_rows.store(bs, SS_OUT_B);
+    z_rows.store(zs, SS_OUT_X);
     __syncthreads();
+    float c_now[SS_SLICE / 16][4];
+#pragma unroll
+    for (int kb = 0; kb < SS_SLICE / 16; ++kb)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) c_now[kb][j] = c_held[kb][j];
+    if (n0 + SS_SLICE < N) load_slice(n0 + SS_SLICE);  // (in flight while this slice is worked)
     if (busy) {
-      for (int kb = 0; kb < n_tiles; ++kb) {
-        float cv[4];
-        load4<T>(rows, c_row + n0, 16 * kb + 4 * gg, n_width, row_ok, vec, cv);
+#pragma unroll
+      for (int kb = 0; kb < SS_SLICE / 16; ++kb) {
 #pragma unroll
         for (int t = 0; t < 4; ++t) {
           if (t > wave) continue;  // (tokens behind this wave's)
-          const float4_t bv = *reinterpret_cast<const float4_t*>(shared_rows + (16 * t + i) * SS_OUT_B + 16 * kb + 4 * gg);
+          const float4_t bv = *reinterpret_cast<const float4_t*>(bs + (16 * t + i) * SS_OUT_B + 16 * kb + 4 * gg);
 #pragma unroll
-          for (int r = 0; r < 4; ++r) scores[t] = mma4(bv[r], cv[r], scores[t]);
+          for (int r = 0; r < 4; ++r) scores[t] = mma4(bv[r], c_now[kb][r], scores[t]);
         }
-      }
-    }
-    __syncthreads();
-    for (int e = threadIdx.x; e < n_tiles * 16 * v_tiles * 4; e += 256) {
-      const int r = e / (v_tiles * 4), c = (e - r * v_tiles * 4) * 4;
-      float v[4];
-      load4<float>(Z, (size_t)(n0 + r) * vdim + v0, c, v_width, r < n_width, z_vec, v);
-      *reinterpret_cast<float4_t*>(shared_rows + r * SS_OUT_X + c) = float4_t{v[0], v[1], v[2], v[3]};
-    }
-    __syncthreads();
-    if (busy) {
-      for (int kb = 0; kb < n_tiles; ++kb) {
-        float cv[4];
-        load4<T>(rows, c_row + n0, 16 * kb + 4 * gg, n_width, row_ok, vec, cv);
-        const float* z0 = shared_rows + (16 * kb + 4 * gg) * SS_OUT_X + i;
+        const float* z0 = zs + (16 * kb + 4 * gg) * SS_OUT_X + i;
 #pragma unroll
         for (int r = 0; r < 4; ++r)
 #pragma unroll
           for (int c = 0; c < 4; ++c)
-            if (c < v_tiles) acc[c] = mma4(z0[r * SS_OUT_X + 16 * c], cv[r], acc[c]);
+            if (c < v_tiles) acc[c] = mma4(z0[r * SS_OUT_X + 16 * c], c_now[kb][r], acc[c]);
       }
     }
+    __syncthreads();  // everyone is done with the slice
   }
   if (!busy) return;  // (no barrier follows)
   const double mine = sums[my_row];
