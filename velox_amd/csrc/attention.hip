@@ -1267,6 +1267,7 @@ __global__ void __launch_bounds__(64 * WAVES) decode_attention_kernel(
   struct Tile {
     typename KO::Operand k[KO::STEPS];
     Frag<T> v[NC];
+    float bias[BIASED ? 4 : 1];  // of the keys 4 g .. 4 g + 3, asked for with them
   };
   // No branch surrounds a load, so the loads of a tile do not wait for those of the tiles before it: a key beyond the
   // sequence is read from the last valid place instead; its score is masked and its values are zeroed when the
@@ -1277,6 +1278,14 @@ __global__ void __launch_bounds__(64 * WAVES) decode_attention_kernel(
     int n_v = n0 + 4 * g;  // the first of the four keys whose values this lane reads
     n_k = n_k < kv_len ? n_k : kv_len - 1;
     n_v = n_v < kv_len ? n_v : (kv_len - 1) & ~3;
+    if constexpr (BIASED) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        int d = pos - (n0 + 4 * g + j);
+        d = d < 0 ? 0 : (d > bias_len - 1 ? bias_len - 1 : d);
+        tile.bias[j] = bias_table[(size_t)head * bias_len + d];
+      }
+    }
     const T* kp = k_cache + ((page_of(n_k) * nkv + kvh) * page_size + (n_k & (page_size - 1))) * D + KO::LANE * g;
     const T* vp = v_cache + ((page_of(n_v) * nkv + kvh) * D + i) * page_size + (n_v & (page_size - 1));
 #pragma unroll
@@ -1316,9 +1325,7 @@ __global__ void __launch_bounds__(64 * WAVES) decode_attention_kernel(
       const bool keep = row_ok && n < kv_len && (window <= 0 || n > pos - window || (KEEPS && n < extras.keep_first));
       const float scaled = CAPPED ? cap(s[j]) : s[j] * scale;
       if constexpr (BIASED) {
-        int d = pos - n;
-        d = d < 0 ? 0 : (d > bias_len - 1 ? bias_len - 1 : d);
-        const float bias = bias_table[(size_t)head * bias_len + d];
+        const float bias = tile.bias[j];
         s[j] = keep ? (CAPPED ? scaled + bias : fmaf(s[j], scale, bias)) : -INFINITY;
       } else {
         s[j] = keep ? scaled : -INFINITY;
