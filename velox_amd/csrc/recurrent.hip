@@ -9,6 +9,8 @@
 //   gated_head_norm     RMS norm of each head's read-out, a shared weight, a gate
 // Everything between a load and a store is float32; stores round once.  No result depends on how a sequence's tokens
 // were cut into steps or on what else is in the batch: sums run in an order that only the sizes fix.
+#include <type_traits>
+
 #include "common.h"
 
 __device__ __forceinline__ float load_as_f32(const void* p, int is_bf16, size_t i) {
@@ -252,20 +254,56 @@ extern "C" int velox_embed_copies(const int* ids, const void* table, int table_d
 // ---------------------------------------------------------------------------------------------
 __device__ __forceinline__ float gelu_tanh_f32(float z) { return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))); }
 
+__device__ __forceinline__ float gate_act(float g, int kind) { return kind == 1 ? gelu_tanh_f32(g) : kind == 2 ? fmaxf(g, 0.f) : g * sigmoid_f32(g); }
+
+// 16-byte accesses; needs inter % (16 / sizeof(T)) == 0 and aligned rows
+template <typename T, int KIND>
+__global__ void __launch_bounds__(256) gated_act_mul_vec_kernel(const T* __restrict__ gate_up, T* __restrict__ out, int inter) {
+  constexpr int N = 16 / sizeof(T);
+  const size_t t = blockIdx.y;
+  const T* row = gate_up + t * 2 * (size_t)inter;
+  for (int at = (blockIdx.x * blockDim.x + threadIdx.x) * N; at < inter; at += gridDim.x * blockDim.x * N) {
+    const float4_t gv = *reinterpret_cast<const float4_t*>(row + at);
+    const float4_t uv = *reinterpret_cast<const float4_t*>(row + inter + at);
+    float4_t ov;
+    const T* ge = reinterpret_cast<const T*>(&gv);
+    const T* ue = reinterpret_cast<const T*>(&uv);
+    T* oe = reinterpret_cast<T*>(&ov);
+#pragma unroll
+    for (int j = 0; j < N; ++j) oe[j] = from_f32<T>(gate_act(to_f32(ge[j]), KIND) * to_f32(ue[j]));
+    *reinterpret_cast<float4_t*>(out + t * inter + at) = ov;
+  }
+}
+
+template <typename T>
+static void launch_gated_act_mul_vec(const void* gate_up, void* out, int tokens, int inter, int kind, hipStream_t stream) {
+  const int pieces = inter / (16 / (int)sizeof(T));
+  int bx = (pieces + 255) / 256;
+  if (bx > 32) bx = 32;
+  const dim3 grid(bx, tokens);
+  if (kind == 1) gated_act_mul_vec_kernel<T, 1><<<grid, 256, 0, stream>>>((const T*)gate_up, (T*)out, inter);
+  else if (kind == 2) gated_act_mul_vec_kernel<T, 2><<<grid, 256, 0, stream>>>((const T*)gate_up, (T*)out, inter);
+  else gated_act_mul_vec_kernel<T, 0><<<grid, 256, 0, stream>>>((const T*)gate_up, (T*)out, inter);
+}
+
 template <typename T>
 __global__ void __launch_bounds__(256) gated_act_mul_kernel(const T* __restrict__ gate_up, T* __restrict__ out, int inter, int kind) {
   const size_t t = blockIdx.y;
   const T* row = gate_up + t * 2 * (size_t)inter;
   for (int i = blockIdx.x * blockDim.x + threadIdx.x; i < inter; i += gridDim.x * blockDim.x) {
     const float g = to_f32(row[i]), u = to_f32(row[inter + i]);
-    const float act = kind == 1 ? gelu_tanh_f32(g) : kind == 2 ? fmaxf(g, 0.f) : g * sigmoid_f32(g);
-    out[t * inter + i] = from_f32<T>(act * u);
+    out[t * inter + i] = from_f32<T>(gate_act(g, kind) * u);
   }
 }
 
 extern "C" int velox_gated_act_mul(const void* gate_up, void* out, int tokens, int inter, int dtype, int kind, hipStream_t stream) {
   if (tokens <= 0 || inter <= 0) return 0;
-  if (tokens > 65535) return (int)hipErrorInvalidValue;
+  if (tokens > 65535 || kind < 0 || kind > 2) return (int)hipErrorInvalidValue;
+  if (inter % (dtype == VELOX_BF16 ? 8 : 4) == 0 && (((uintptr_t)gate_up | (uintptr_t)out) & 15) == 0) {
+    if (dtype == VELOX_BF16) launch_gated_act_mul_vec<bf16_t>(gate_up, out, tokens, inter, kind, stream);
+    else launch_gated_act_mul_vec<float>(gate_up, out, tokens, inter, kind, stream);
+    VELOX_RETURN_LAUNCH_STATUS();
+  }
   int bx = (inter + 255) / 256;
   if (bx > 64) bx = 64;
   const dim3 grid(bx, tokens);
@@ -283,6 +321,7 @@ extern "C" int velox_gated_act_mul(const void* gate_up, void* out, int tokens, i
 // ---------------------------------------------------------------------------------------------
 #define CONV_TAPS_MAX 8
 #define CONV_CHUNK 16
+#define CONV_FEW 4
 
 template <typename T>
 __global__ void __launch_bounds__(256) short_conv_kernel(const T* __restrict__ x, int ld, int C, const float* __restrict__ w, int taps, T* tail,
@@ -327,6 +366,61 @@ __global__ void __launch_bounds__(256) short_conv_kernel(const T* __restrict__ x
   }
 }
 
+// The same for channels and rows that come in aligned pieces of four: a lane owns four neighbouring channels, and the inputs of
+// its TOKENS tokens (1 or CONV_FEW: many short walks hide more than few long ones) are all asked for before the first is used.  TAPS: the columns, or CONV_TAPS_MAX for any number.
+template <typename T, int TAPS, int TOKENS>
+__global__ void __launch_bounds__(64) short_conv_vec_kernel(const T* __restrict__ x, int ld, int C, const float* __restrict__ w, int taps_given, T* tail,
+                                                            const int* __restrict__ slots, const int* __restrict__ cu_q, T* __restrict__ out, int silu,
+                                                            int update_here, const float* __restrict__ bias) {
+  constexpr int is_bf16 = sizeof(T) == 2;
+  const int taps = TAPS < CONV_TAPS_MAX ? TAPS : taps_given;
+  const int c = (blockIdx.x * 64 + threadIdx.x) * 4;
+  const int b = blockIdx.z;
+  const int lo = cu_q[b], hi = cu_q[b + 1];
+  const int first = lo + blockIdx.y * TOKENS;
+  if (c >= C || first >= hi) return;
+  const int count = hi - first < TOKENS ? hi - first : TOKENS;
+  float4_t now[TOKENS];
+#pragma unroll
+  for (int t = 0; t < TOKENS; ++t) now[t] = load4_as_f32(x, is_bf16, (size_t)(first + (t < count ? t : count - 1)) * ld + c);
+  float4_t wj[TAPS], u[TAPS];
+#pragma unroll
+  for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+    for (int k = 0; k < 4; ++k) wj[j][k] = j < taps ? w[(size_t)(c + k) * taps + j] : 0.f;
+  T* my_tail = tail ? tail + (size_t)slots[b] * (taps - 1) * C + c : nullptr;
+#pragma unroll
+  for (int j = 0; j < TAPS; ++j) {
+    u[j] = float4_t{0.f, 0.f, 0.f, 0.f};
+    if (j < taps - 1) {
+      const int t = first - (taps - 1) + j;
+      if (t >= lo) u[j] = load4_as_f32(x, is_bf16, (size_t)t * ld + c);
+      else if (my_tail) u[j] = load4_as_f32(my_tail, is_bf16, (size_t)(t - lo + taps - 1) * C);
+    }
+  }
+  const float4_t start = bias ? *reinterpret_cast<const float4_t*>(bias + c) : float4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int t = 0; t < TOKENS; ++t) {
+    if (t >= count) break;
+    float4_t y = start;
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j)  // (oldest input first, as in short_conv_kernel)
+      if (j < taps) y += wj[j] * (j == taps - 1 ? now[t] : u[j]);
+    if (silu) {
+#pragma unroll
+      for (int k = 0; k < 4; ++k) y[k] = y[k] * sigmoid_f32(y[k]);
+    }
+    store4_from_f32(out, is_bf16, (size_t)(first + t) * C + c, y);
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) u[j] = j == taps - 2 ? now[t] : (j + 1 < TAPS ? u[j + 1] : float4_t{0.f, 0.f, 0.f, 0.f});
+  }
+  if (update_here && my_tail && taps > 1) {
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j)
+      if (j < taps - 1) store4_from_f32(my_tail, is_bf16, (size_t)j * C, u[j]);
+  }
+}
+
 template <typename T>
 __global__ void __launch_bounds__(256) short_conv_tail_kernel(const T* __restrict__ x, int ld, int C, int taps, T* tail, const int* __restrict__ slots,
                                                               const int* __restrict__ cu_q) {
@@ -353,11 +447,31 @@ extern "C" int velox_short_conv(const void* x, int ld, int channels, const float
                                 int num_seqs, int max_q_len, int dtype, int silu, int update_state, const float* bias, hipStream_t stream) {
   if (num_seqs <= 0 || max_q_len <= 0) return 0;
   if (taps < 1 || taps > CONV_TAPS_MAX || num_seqs > 65535) return (int)hipErrorInvalidValue;
-  const int chunks = (max_q_len + CONV_CHUNK - 1) / CONV_CHUNK;
+  const size_t elem = dtype == VELOX_BF16 ? 2 : 4;
+  const bool pieces = channels % 4 == 0 && ld % 4 == 0 && (((uintptr_t)x | (uintptr_t)out | (uintptr_t)tail) % (4 * elem)) == 0 && (uintptr_t)bias % 16 == 0 &&
+                      max_q_len <= 65535 * CONV_FEW;
+  const int tokens_each = !pieces ? CONV_CHUNK : max_q_len == 1 ? 1 : CONV_FEW;
+  const int chunks = (max_q_len + tokens_each - 1) / tokens_each;
   if (chunks > 65535) return (int)hipErrorInvalidValue;
   const dim3 grid((channels + 255) / 256, chunks, num_seqs);
   const int here = (update_state && chunks == 1) ? 1 : 0;
-  if (dtype == VELOX_BF16)
+  auto in_pieces = [&](auto type, auto tokens) {
+    typedef decltype(type) T;
+    constexpr int TOKENS = decltype(tokens)::value;
+    const dim3 fours((channels / 4 + 63) / 64, chunks, num_seqs);
+#define VELOX_CONV_VEC(TAPS)                                                                                                                              \
+  short_conv_vec_kernel<T, TAPS, TOKENS><<<fours, 64, 0, stream>>>((const T*)x, ld, channels, w, taps, (T*)tail, slots, cu_q, (T*)out, silu, here, bias)
+    if (taps == 2) VELOX_CONV_VEC(2);
+    else if (taps == 3) VELOX_CONV_VEC(3);
+    else if (taps == 4) VELOX_CONV_VEC(4);
+    else VELOX_CONV_VEC(CONV_TAPS_MAX);
+#undef VELOX_CONV_VEC
+  };
+  typedef std::integral_constant<int, 1> one;
+  typedef std::integral_constant<int, CONV_FEW> few;
+  if (pieces && dtype == VELOX_BF16) { if (max_q_len == 1) in_pieces(bf16_t(), one()); else in_pieces(bf16_t(), few()); }
+  else if (pieces) { if (max_q_len == 1) in_pieces(float(), one()); else in_pieces(float(), few()); }
+  else if (dtype == VELOX_BF16)
     short_conv_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)x, ld, channels, w, taps, (bf16_t*)tail, slots, cu_q, (bf16_t*)out, silu, here, bias);
   else
     short_conv_kernel<float><<<grid, 256, 0, stream>>>((const float*)x, ld, channels, w, taps, (float*)tail, slots, cu_q, (float*)out, silu, here, bias);
@@ -432,6 +546,102 @@ __global__ void __launch_bounds__(256) rotate_pad_write_kernel(const T* __restri
   }
 }
 
+// The same in bfloat16 for channels i paired with i + half, with everything in 16-byte pieces (dim, vdim, D, half and ld multiples of 8):
+// P lanes (a power of two, at least D / 8) work one query or key head, a lane eight channels; the sum of a head's squares is built
+// from its lanes' sums.  Values go to [channel][offset]: where eight consecutive tokens fill eight consecutive offsets of a page
+// (slots s .. s + 7 with s a multiple of 8), the first of them writes all eight as one piece per channel and the others write
+// nothing; every workgroup finds the same answer from the slots alone.
+typedef __bf16 pad_bf16x8_t __attribute__((ext_vector_type(8)));
+
+template <int P>
+__global__ void __launch_bounds__(256) rotate_pad_write_vec_kernel(const bf16_t* __restrict__ qkv, int ld, bf16_t* __restrict__ q_out, const int* __restrict__ positions,
+                                                                   const float* __restrict__ cos_t, const float* __restrict__ sin_t, int half,
+                                                                   const int* __restrict__ slot_mapping, bf16_t* __restrict__ k_cache, bf16_t* __restrict__ v_cache,
+                                                                   int heads, int kv_heads, int dim, int vdim, int D, int page_shift, int write_kv,
+                                                                   float post_norm_eps, int values_are_keys) {
+  constexpr int AT_ONCE = 256 / P;
+  const int t = blockIdx.x;
+  const bf16_t* row = qkv + (size_t)t * ld;
+  const int q_size = heads * dim, k_size = kv_heads * dim;
+  const int page_size = 1 << page_shift;
+  int slot = 0, page = 0, offset = 0;
+  if (write_kv) {
+    slot = slot_mapping[t];
+    page = slot >> page_shift;
+    offset = slot & (page_size - 1);
+  }
+  const float* cs = half > 0 ? cos_t + (size_t)positions[t] * half : nullptr;
+  const float* sn = half > 0 ? sin_t + (size_t)positions[t] * half : nullptr;
+  const int c0 = (threadIdx.x % P) * 8;
+  const int qk_heads = heads + (write_kv ? kv_heads : 0);
+  for (int h = blockIdx.y * AT_ONCE + threadIdx.x / P; h < qk_heads; h += gridDim.y * AT_ONCE) {  // (a head's lanes go round together)
+    const bool is_q = h < heads;
+    const int g = is_q ? h : h - heads;
+    const bf16_t* src = row + (is_q ? h * dim : q_size + g * dim);
+    float y[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) y[j] = 0.f;
+    if (c0 < dim) {
+      const pad_bf16x8_t own = *reinterpret_cast<const pad_bf16x8_t*>(src + c0);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) y[j] = (float)own[j];
+      if (c0 < 2 * half) {
+        const bool low = c0 < half;
+        const int i0 = low ? c0 : c0 - half;
+        const pad_bf16x8_t other = *reinterpret_cast<const pad_bf16x8_t*>(src + (low ? c0 + half : c0 - half));
+        float c[8], s[8];
+#pragma unroll
+        for (int p = 0; p < 2; ++p) {
+          reinterpret_cast<float4_t*>(c)[p] = reinterpret_cast<const float4_t*>(cs + i0)[p];
+          reinterpret_cast<float4_t*>(s)[p] = reinterpret_cast<const float4_t*>(sn + i0)[p];
+        }
+#pragma unroll
+        for (int j = 0; j < 8; ++j) y[j] = low ? y[j] * c[j] - (float)other[j] * s[j] : y[j] * c[j] + (float)other[j] * s[j];
+      }
+    }
+    if (post_norm_eps > 0.f) {
+      float sum = 0.f;
+#pragma unroll
+      for (int j = 0; j < 8; ++j) sum += y[j] * y[j];
+#pragma unroll
+      for (int off = 1; off < P; off <<= 1) sum += __shfl_xor(sum, off, VELOX_WAVE);
+      const float inv = 1.f / sqrtf(sum / (float)dim + post_norm_eps);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) y[j] *= inv;
+    }
+    if (c0 < D) {
+      pad_bf16x8_t o;
+#pragma unroll
+      for (int j = 0; j < 8; ++j) o[j] = (bf16_t)y[j];
+      bf16_t* dst = is_q ? q_out + ((size_t)t * heads + h) * D : k_cache + (((size_t)page * kv_heads + g) * page_size + offset) * D;
+      *reinterpret_cast<pad_bf16x8_t*>(dst + c0) = o;
+    }
+  }
+  if (!write_kv || blockIdx.y != 0) return;
+  constexpr int RUN = 8;
+  const int values_at = values_are_keys ? q_size : q_size + k_size;  // (a value head is vdim long, and so is then its key head)
+  const int lead = t - offset % RUN;  // the token that would hold the run's first slot
+  bool in_run = page_size >= RUN && lead >= 0 && lead + RUN <= (int)gridDim.x;
+  if (in_run) {
+    const int first_slot = slot - offset % RUN;
+    for (int j = 0; j < RUN; ++j) in_run = in_run && slot_mapping[lead + j] == first_slot + j;
+  }
+  if (in_run && t != lead) return;
+  for (int item = threadIdx.x; item < kv_heads * D; item += 256) {  // (neighbouring lanes take neighbouring channels)
+    const int g = item / D, c = item % D;
+    bf16_t* dst = v_cache + (((size_t)page * kv_heads + g) * D + c) * page_size + offset;
+    const bf16_t* src = row + values_at + g * vdim + c;
+    if (in_run) {
+      pad_bf16x8_t o;
+#pragma unroll
+      for (int j = 0; j < RUN; ++j) o[j] = c < vdim ? src[(size_t)j * ld] : (bf16_t)0.f;
+      *reinterpret_cast<pad_bf16x8_t*>(dst) = o;
+    } else {
+      *dst = c < vdim ? *src : (bf16_t)0.f;
+    }
+  }
+}
+
 extern "C" int velox_rotate_pad_write(const void* qkv, int ld, void* q_out, const int* positions, const float* cos_t, const float* sin_t, int half,
                                       const int* slot_mapping, void* k_cache, void* v_cache, int tokens, int heads, int kv_heads, int dim, int vdim, int D,
                                       int page_size, int write_kv, int dtype, int interleaved, float post_norm_eps, int values_are_keys, hipStream_t stream) {
@@ -439,6 +649,27 @@ extern "C" int velox_rotate_pad_write(const void* qkv, int ld, void* q_out, cons
   int shift = 0;
   while ((1 << shift) < page_size) ++shift;
   if ((1 << shift) != page_size || 2 * half > dim || dim > D || vdim > D || (values_are_keys && vdim != dim)) return (int)hipErrorInvalidValue;
+  const bool in_pieces = dtype == VELOX_BF16 && !interleaved && D <= 256 && dim % 8 == 0 && vdim % 8 == 0 && D % 8 == 0 && half % 8 == 0 && ld % 8 == 0 &&
+                         (((uintptr_t)qkv | (uintptr_t)q_out | (uintptr_t)cos_t | (uintptr_t)sin_t | (uintptr_t)k_cache | (uintptr_t)v_cache) & 15) == 0;
+  if (in_pieces) {
+    int lanes_per_head = 1;
+    while (lanes_per_head * 8 < D) lanes_per_head <<= 1;
+    const int at_once = 256 / lanes_per_head, qk_heads = heads + (write_kv ? kv_heads : 0);
+    const dim3 pieces(tokens, tokens <= 256 ? (qk_heads + at_once - 1) / at_once : 1);
+#define VELOX_ROTATE_VEC(P)                                                                                                                                  \
+  rotate_pad_write_vec_kernel<P><<<pieces, 256, 0, stream>>>((const bf16_t*)qkv, ld, (bf16_t*)q_out, positions, cos_t, sin_t, half, slot_mapping,           \
+                                                             (bf16_t*)k_cache, (bf16_t*)v_cache, heads, kv_heads, dim, vdim, D, shift, write_kv,            \
+                                                             post_norm_eps, values_are_keys)
+    switch (lanes_per_head) {
+      case 1: case 2: VELOX_ROTATE_VEC(2); break;
+      case 4: VELOX_ROTATE_VEC(4); break;
+      case 8: VELOX_ROTATE_VEC(8); break;
+      case 16: VELOX_ROTATE_VEC(16); break;
+      default: VELOX_ROTATE_VEC(32); break;
+    }
+#undef VELOX_ROTATE_VEC
+    VELOX_RETURN_LAUNCH_STATUS();
+  }
   const int all_heads = heads + (write_kv ? 2 * kv_heads : 0);
   const dim3 grid(tokens, tokens <= 256 ? all_heads : (all_heads < 4 ? all_heads : 4));
   int lanes = (D + 63) / 64 * 64;
