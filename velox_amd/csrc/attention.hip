@@ -202,6 +202,13 @@ template <typename T> __device__ __forceinline__ float4_t gate_of(const Extras& 
   return out;
 }
 
+// The same for one channel.
+template <typename T> __device__ __forceinline__ float gate_of_one(const Extras& x, size_t token, int head, int c) {
+  if (x.gate_channels != 0 && c >= x.gate_channels) return 1.f;
+  const float z = to_f32(((const T*)x.gate)[token * x.gate_stride + (x.gate_channels == 0 ? head : head * x.gate_channels + c)]);
+  return 1.f / (1.f + expf(-z));
+}
+
 // Where the tiles of keys of a row block lie.  Without kept keys tile t starts at key n_begin + t * BN.  With a window and kept
 // keys the first `kept_tiles` tiles are those of keys 0 .. keep_first - 1 and the window's follow; when the two meet there is
 // one run of tiles from key 0.  Page ids are kept in one array, the kept tiles' first.
@@ -1432,32 +1439,50 @@ __global__ void __launch_bounds__(64 * WAVES) decode_attention_kernel(
 
 // out[token, head, :] = sum_s w_s * o_s / sum_s w_s,  w_s = exp(lse_s - max_s lse_s); a sink adds exp(sink - max_s lse_s)
 // to the denominator
+constexpr int MERGE_THREADS = (D + 63) / 64 * 64;  // a lane per channel, whole waves
+constexpr int MERGE_AHEAD = 32;
 template <typename T>
-__global__ void merge_splits_kernel(const float* __restrict__ part_o, const float* __restrict__ part_lse, T* __restrict__ out,
+__global__ void __launch_bounds__(MERGE_THREADS) merge_splits_kernel(const float* __restrict__ part_o, const float* __restrict__ part_lse, T* __restrict__ out,
                                     int nh, int splits, int total_tokens, int first_token, const float* __restrict__ sinks, const Extras extras) {
   const size_t token = (size_t)blockIdx.x + first_token;  // (the launch covers tokens [first_token, total_tokens))
   const int head = blockIdx.y;
   const size_t stride = (size_t)total_tokens * nh;  // slots per split
   const size_t slot0 = token * nh + head;
-  float mx = -INFINITY;
-#pragma unroll 8
-  for (int s = 0; s < splits; ++s) mx = fmaxf(mx, part_lse[s * stride + slot0]);
+  float gate = 1.f;  // (asked for before everything that has to be waited for)
+  if constexpr (GATED) gate = (int)threadIdx.x < D ? gate_of_one<T>(extras, token, head, threadIdx.x) : 1.f;
+  // Every lane asks for one split's log-sum (the next 64 splits', if there are more, in another round) and for its own channel
+  // of up to MERGE_AHEAD splits, all before it waits for any of them; a split's weight reaches the lanes from the one that holds it.
+  const int lane = threadIdx.x & 63;
+  auto log_sum = [&](int s) { return s < splits ? part_lse[(size_t)s * stride + slot0] : -INFINITY; };
+  const float my_lse = log_sum(lane);
+  const int dd = threadIdx.x;
+  const bool live = dd < D;
+  const float* parts = part_o + slot0 * D + (live ? dd : 0);
+  float o[MERGE_AHEAD];
+#pragma unroll
+  for (int j = 0; j < MERGE_AHEAD; ++j) o[j] = j < splits ? parts[(size_t)j * stride * D] : 0.f;  // (the same answer for every lane)
+  float mx = my_lse;
+  for (int s = 64 + lane; s < splits; s += 64) mx = fmaxf(mx, log_sum(s));
+  mx = wave_max(mx);
   const float m_safe = (mx == -INFINITY) ? 0.f : mx;
-  const float sink_term = (sinks != nullptr && mx != -INFINITY) ? expf(sinks[head] - m_safe) : 0.f;
-  for (int dd = threadIdx.x; dd < D; dd += blockDim.x) {
-    float acc = 0.f, denom = sink_term;
-#pragma unroll 8
-    for (int s = 0; s < splits; ++s) {
-      const size_t slot = s * stride + slot0;
-      const float lse = part_lse[slot];
-      const float w = (lse == -INFINITY) ? 0.f : expf(lse - m_safe);
-      acc += w * part_o[slot * D + dd];
-      denom += w;
+  auto weight_of = [&](float lse) { return (lse == -INFINITY) ? 0.f : expf(lse - m_safe); };
+  float my_weight = weight_of(my_lse);
+  float denom = wave_sum(my_weight), acc = 0.f;
+#pragma unroll
+  for (int j = 0; j < MERGE_AHEAD; ++j)
+    if (j < splits) acc += __shfl(my_weight, j, VELOX_WAVE) * o[j];
+  for (int s = MERGE_AHEAD; s < splits; ++s) {
+    if ((s & 63) == 0) {
+      my_weight = weight_of(log_sum(s + lane));
+      denom += wave_sum(my_weight);
     }
-    float o = acc / (denom > 0.f ? denom : 1.f);
-    if constexpr (GATED) o *= gate_of<T>(extras, token, head, dd & ~3)[dd & 3];
-    out[slot0 * D + dd] = from_f32<T>(o);
+    acc += __shfl(my_weight, s & 63, VELOX_WAVE) * parts[(size_t)s * stride * D];
   }
+  if (sinks != nullptr && mx != -INFINITY) denom += expf(sinks[head] - m_safe);
+  if (!live) return;
+  float result = acc / (denom > 0.f ? denom : 1.f);
+  if constexpr (GATED) result *= gate;
+  out[slot0 * D + dd] = from_f32<T>(result);
 }
 
 // Which kernel portions of prompts take: 0 = chosen by shape; 1 = never the kernel with direct loads; 2 = that kernel
@@ -1498,7 +1523,7 @@ static int launch(const void* qkv, int qkv_stride, const void* k_cache, const vo
         nh, nkv, page_shift, scale, window, splits, total_tokens, bias_table, bias_len, sinks, extras);
     int status = (int)hipGetLastError();
     if (status != 0 || splits == 1) return status;
-    merge_splits_kernel<T><<<dim3(total_tokens, nh), D < 64 ? 64 : D, 0, stream>>>(part_o, part_lse, (T*)out, nh, splits, total_tokens, 0, sinks, extras);
+    merge_splits_kernel<T><<<dim3(total_tokens, nh), MERGE_THREADS, 0, stream>>>(part_o, part_lse, (T*)out, nh, splits, total_tokens, 0, sinks, extras);
     return (int)hipGetLastError();
   }
   // The kernel whose tiles reach LDS by direct loads: bfloat16, head sizes 64 and 128, pages of at least 8 tokens.
@@ -1519,7 +1544,7 @@ static int launch(const void* qkv, int qkv_stride, const void* k_cache, const vo
     }
     int status = (int)hipGetLastError();
     if (status != 0 || splits == 1) return status;
-    merge_splits_kernel<T><<<dim3(total_tokens - first_token, nh), D < 64 ? 64 : D, 0, stream>>>(part_o, part_lse, (T*)out, nh, splits, total_tokens,
+    merge_splits_kernel<T><<<dim3(total_tokens - first_token, nh), MERGE_THREADS, 0, stream>>>(part_o, part_lse, (T*)out, nh, splits, total_tokens,
                                                                                                  first_token, sinks, extras);
     return (int)hipGetLastError();
   };
@@ -1599,7 +1624,7 @@ static int launch(const void* qkv, int qkv_stride, const void* k_cache, const vo
   }
   int status = (int)hipGetLastError();
   if (status != 0 || splits == 1) return status;
-  merge_splits_kernel<T><<<dim3(total_tokens - first_token, nh), D < 64 ? 64 : D, 0, stream>>>(part_o, part_lse, (T*)out, nh, splits, total_tokens,
+  merge_splits_kernel<T><<<dim3(total_tokens - first_token, nh), MERGE_THREADS, 0, stream>>>(part_o, part_lse, (T*)out, nh, splits, total_tokens,
                                                                                                first_token, sinks, extras);
   return (int)hipGetLastError();
 }
